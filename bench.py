@@ -25,6 +25,7 @@ Other workloads, each again one JSON line:
     python bench.py --design sodedra [--design-sizes 1024,2048,4096] [--layers 8]   # Sodedra beside Qwen3 at equal size
     python bench.py --design meronex [--design-sizes 1024,2048,4096] [--layers 9]   # Meronex beside Sodedra and Qwen3 at equal size
     python bench.py --design tarunex [--design-sizes 1024,2048,4096] [--layers 8]   # Tarunex beside Sodedra, Sefevik and Qwen3 at equal size
+    python bench.py --design balelorn [--design-sizes 1024,2048,4096] [--layers 8]  # Balelorn beside Sodedra, Tarunex and Qwen3 at equal size
 """
 import argparse
 import json
@@ -139,10 +140,24 @@ def tarunex_shape(width: int, layers: int, vocab: int) -> dict:
                 logit_softcap=50.0, loop=dict(start=0, stop=2, times=2), layers=out)
 
 
+def balelorn_shape(width: int, layers: int, vocab: int) -> dict:
+    """A Balelorn configuration with the layer sizes of a real model of that width: attention heads of 128 with 64 rotated
+    dims and a quarter as many kv heads, chunks of 1536 positions (every fourth layer reads everything), values blended in
+    every layer; of every four layers one with a dense feed-forward of three times the width and three with 32 experts of a
+    quarter of that, of which a table gives every token four (as many active weights)."""
+    heads = max(1, width // 128)
+    att = dict(heads=heads, kv_heads=max(1, heads // 4), dim=128, vdim=128, scale=128 ** -0.5, mask=dict(size=1536), v_mix=True,
+               rot=dict(base=10000.0, dims=64))
+    dense = dict(kind="dense", ff=3 * width)
+    moe = dict(kind="moe", expert=dict(ff=3 * width // 4, limit=7.0), router=dict(experts=32, top=4))
+    out = [dict(type="attention", mixer=dict(att, mask=None) if i % 4 == 3 else dict(att), mlp=dense if i % 4 == 0 else moe) for i in range(layers)]
+    return dict(architecture="Balelorn", vocab=vocab, width=width, norm=dict(eps=1e-5), layers=out)
+
+
 DESIGN_SHAPES = {"sefevik": ("Sefevik", sefevik_shape), "sodedra": ("Sodedra", sodedra_shape), "meronex": ("Meronex", meronex_shape),
-                 "tarunex": ("Tarunex", tarunex_shape)}
+                 "tarunex": ("Tarunex", tarunex_shape), "balelorn": ("Balelorn", balelorn_shape)}
 #: further designs that a design is measured beside (Qwen3 always is): the closest ones the engine has
-DESIGN_BESIDE = {"meronex": ("sodedra",), "tarunex": ("sodedra", "sefevik")}
+DESIGN_BESIDE = {"meronex": ("sodedra",), "tarunex": ("sodedra", "sefevik"), "balelorn": ("sodedra", "tarunex")}
 #: layers, where --layers does not say: a whole number of the design's turns of layer kinds
 DESIGN_LAYERS = {"meronex": 9}
 
@@ -258,7 +273,7 @@ def main() -> int:
     ap.add_argument("--serve", type=int, default=0, metavar="N",
                     help="instead of the decode steps: N requests arriving at once, prompts of 128..2048 and outputs of 64..512 "
                          "tokens (uniform), run until all have ended; the value is generated tokens per second of the whole run")
-    ap.add_argument("--design", default="", choices=["", "sefevik", "sodedra", "meronex", "tarunex"],
+    ap.add_argument("--design", default="", choices=["", "sefevik", "sodedra", "meronex", "tarunex", "balelorn"],
                     help="instead of the decode steps: prefill and decode throughput of that design at a few layer sizes "
                          "beside the Qwen3 shape of equal width, layers, heads and feed-forward size (--design-sizes)")
     ap.add_argument("--design-sizes", default="1024,2048,4096", help="widths for --design")

@@ -61,11 +61,8 @@ class PageGroup:
     pool: PagePool
 
     def first_needed_page(self, num_tokens: int) -> int:
-        """Logical page below which nothing is read once ``num_tokens`` are cached:
-        the next query sits at position >= num_tokens and reads keys > position - window."""
-        if self.spec.window is None:
-            return 0
-        return max(0, num_tokens - self.spec.window + 1) // self.page_size
+        """Logical page below which nothing is read once ``num_tokens`` are cached."""
+        return self.spec.first_needed(num_tokens) // self.page_size
 
 
 @dataclasses.dataclass
@@ -94,9 +91,9 @@ class RequestCache:
 
 
 def window_pages(window: int, page_size: int, step_tokens: int = 1) -> int:
-    """Most pages that one request holds in a group whose layers read the last ``window`` keys only, while it runs
-    ``step_tokens`` tokens in a step: the keys that the step's first query reads and the step's own, which begin and
-    end anywhere in a page."""
+    """Most pages that one request holds in a group whose layers read the last ``window`` keys only (or, a chunk's length,
+    the keys of one chunk), while it runs ``step_tokens`` tokens in a step: the keys that the step's first query reads and
+    the step's own, which begin and end anywhere in a page."""
     return -(-(window - 1 + step_tokens) // page_size) + 1
 
 
@@ -104,7 +101,7 @@ class CacheManager:
     def __init__(self, cache_specs: Sequence[Optional[object]], page_size: int, num_pages: int, max_num_seqs: int,
                  max_step_tokens: Optional[int] = None):
         """``cache_specs[i]`` is the need of layer cache ``i`` (None = nothing).
-        Every page group gets a pool of ``num_pages`` pages of ``page_size`` tokens; a group with a window gets no
+        Every page group gets a pool of ``num_pages`` pages of ``page_size`` tokens; a group with a window or chunks gets no
         more than ``max_num_seqs`` requests can hold at once when none runs more than ``max_step_tokens`` tokens in a
         step (if that is given)."""
         if page_size <= 0:
@@ -139,9 +136,9 @@ class CacheManager:
     @staticmethod
     def pages_of_group(spec: CacheKind, page_size: int, num_pages: int, max_num_seqs: int, max_step_tokens: Optional[int]) -> int:
         """Pages in the pool of a group of kind ``spec`` when ``num_pages`` are offered to every group."""
-        if spec.window is None or max_step_tokens is None:
+        if spec.reach is None or max_step_tokens is None:
             return num_pages
-        return max(1, min(num_pages, max_num_seqs * window_pages(spec.window, page_size, max_step_tokens)))
+        return max(1, min(num_pages, max_num_seqs * window_pages(spec.reach, page_size, max_step_tokens)))
 
     # ---- admission -------------------------------------------------------
     def can_admit(self) -> bool:
@@ -245,11 +242,11 @@ class CacheManager:
         return [g.pool.num_free for g in self.page_groups]
 
     def max_tokens_per_request(self) -> int:
-        """Most tokens one request alone can reach (the smallest group decides).  A group with a window gives back the
-        pages that the window has passed, so with room for the window and one token more it sets no limit."""
+        """Most tokens one request alone can reach (the smallest group decides).  A group with a window (or chunks) gives
+        back the pages that the window has passed, so with room for the window and one token more it sets no limit."""
         limit = 1 << 62
         for g in self.page_groups:
-            if g.spec.window is not None and g.pool.num_pages >= window_pages(g.spec.window, g.page_size):
+            if g.spec.reach is not None and g.pool.num_pages >= window_pages(g.spec.reach, g.page_size):
                 continue
             limit = min(limit, g.pool.num_pages * g.page_size)
         return limit

@@ -26,6 +26,20 @@ class CacheKind:
     paged: bool = True
     #: paged kinds: only the last ``window`` tokens are ever read again (None = all)
     window: Optional[int] = None
+    #: paged kinds: a token is read by the tokens of its own chunk of ``chunk`` positions only (None = no chunks); chunks
+    #: are counted from the request's first token
+    chunk: Optional[int] = None
+
+    def first_needed(self, num_tokens: int) -> int:
+        """First token that is read again once ``num_tokens`` are cached: the next query sits at position >= num_tokens."""
+        if self.chunk is not None:
+            return num_tokens // self.chunk * self.chunk
+        return 0 if self.window is None else max(0, num_tokens - self.window + 1)
+
+    @property
+    def reach(self) -> Optional[int]:
+        """Most tokens that a query reads, its own included (None = all before it)."""
+        return self.window if self.chunk is None else self.chunk
 
     def page_bytes(self, page_size: int, act_dtype: torch.dtype) -> int:
         """Device bytes of one page (paged) or one slot (not paged) in ONE layer."""
@@ -74,7 +88,8 @@ class StateLayer:
 @dataclasses.dataclass(frozen=True)
 class PagedKV(CacheKind):
     """Keys and values of every token, in pages; ``window`` = only the last
-    ``window`` tokens are ever read again (older pages are given back).
+    ``window`` tokens are ever read again (older pages are given back); ``chunk`` = tokens are read inside their own chunk
+    only (a chunk's pages are given back once the request has left it).
 
     Device layout per group of ``n`` layers: keys ``[n, pages, n_kv, page, d]``, values
     ``[n, pages, n_kv, d, page]`` in the activation dtype.  One head's part of a page is contiguous, so that a wave
@@ -84,6 +99,7 @@ class PagedKV(CacheKind):
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
+    chunk: Optional[int] = None
     paged = True
 
     def page_bytes(self, page_size, act_dtype):

@@ -645,3 +645,99 @@ class TarunexConfig(ModelConfig):
             f = layer["mlp"]
             if f and (f["ff"] <= 0 or f["experts"] <= 0 or not 0 < f["top"] <= f["experts"] or (f["shared_ff"] is not None and f["shared_ff"] <= 0)):
                 raise ConfigError("%s.mlp: inner sizes positive, 1 to %d choices" % (where, max(f["experts"], 1)))
+
+
+@dataclasses.dataclass
+class BalelornConfig(ModelConfig):
+    """Balelorn: token vectors normed before the first layer; layers that norm every sublayer's input and its result, the
+    latter times a learned vector; the token mixer 'attention' (grouped queries, heads rotated in part, keys of the query's
+    own chunk only, a learned sink per head, values blended with those of the first layer that blends, a sigmoid gate on the
+    result); feed-forwards 'dense' (gated, the tanh form of gelu) or 'moe' (clamped experts named by a table of the token
+    ids), or none.  The configuration is nested; ``layers`` lists every layer's type and sizes, and nothing is assumed equal
+    between layers."""
+
+    architecture: str = ""
+    vocab: int = -1
+    width: int = -1
+    norm_eps: float = 0.0
+    #: one dict per layer: type, mixer (sizes and constants of that mixer), mlp (None, {kind: dense, ff} or
+    #: {kind: moe, ff, limit, experts, top})
+    layers: List[Dict[str, Any]] = dataclasses.field(default_factory=list)
+
+    MIXERS: ClassVar[tuple] = ("attention",)
+
+    @classmethod
+    def from_dict(cls, raw: Dict[str, Any]) -> "BalelornConfig":
+        cfg = cls(architecture=str(raw.get("architecture") or (raw.get("architectures") or [""])[0]),
+                  vocab=_need(raw, "vocab", int), width=_need(raw, "width", int), norm_eps=float(_need(raw, "norm.eps", (int, float))))
+        cfg.layers = [cls._layer(i, l) for i, l in enumerate(_need(raw, "layers", list))]
+        cfg._raw = dict(raw)
+        cfg.validate()
+        return cfg
+
+    @classmethod
+    def _layer(cls, i: int, raw: Dict[str, Any]) -> Dict[str, Any]:
+        where = "config.json layers[%d]" % i
+        if not isinstance(raw, dict):
+            raise ConfigError("%s is no object" % where)
+        kind = _need(raw, "type", str, where)
+        if kind not in cls.MIXERS:
+            raise ConfigError("%s: mixer type %r is not known (%s)" % (where, kind, ", ".join(cls.MIXERS)))
+        m = _need(raw, "mixer", dict, where)
+        at = where + ".mixer"
+        mix = {k: _need(m, k, int, at) for k in ("heads", "dim")}
+        mix["vdim"] = _need(m, "vdim", int, at) if m.get("vdim") is not None else mix["dim"]
+        mix["kv_heads"] = _need(m, "kv_heads", int, at) if m.get("kv_heads") is not None else mix["heads"]
+        mix["scale"] = float(_need(m, "scale", (int, float), at))
+        mix["chunk"] = _need(m, "mask.size", int, at) if m.get("mask") else None
+        mix["v_mix"] = m.get("v_mix") or False
+        if not isinstance(mix["v_mix"], bool):
+            raise ConfigError("%s.v_mix has value %r, expected true or false" % (at, mix["v_mix"]))
+        rot = m.get("rot")
+        mix["rot"] = None
+        if rot:
+            mix["rot"] = {"base": float(_need(rot, "base", (int, float), at + ".rot")),
+                          "dims": _need(rot, "dims", int, at + ".rot") if rot.get("dims") is not None else mix["dim"]}
+        out = {"type": kind, "mixer": mix, "mlp": None}
+        mlp = raw.get("mlp")
+        if mlp is not None:
+            at = where + ".mlp"
+            fk = _need(mlp, "kind", str, at)
+            if fk == "dense":
+                out["mlp"] = {"kind": fk, "ff": _need(mlp, "ff", int, at)}
+            elif fk == "moe":
+                out["mlp"] = {"kind": fk, "ff": _need(mlp, "expert.ff", int, at), "limit": float(_need(mlp, "expert.limit", (int, float), at)),
+                              "experts": _need(mlp, "router.experts", int, at), "top": _need(mlp, "router.top", int, at)}
+            else:
+                raise ConfigError("%s: kind %r is not known (dense, moe)" % (at, fk))
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        return dict(getattr(self, "_raw", {}))
+
+    def validate(self) -> None:
+        if self.vocab <= 0 or self.width <= 0:
+            raise ConfigError("config.json: vocab and width must be positive")
+        if not (self.norm_eps > 0.0):
+            raise ConfigError("config.json: norm.eps must be positive")
+        if not self.layers:
+            raise ConfigError("config.json: no layers")
+        first = None
+        for i, layer in enumerate(self.layers):
+            m, where = layer["mixer"], "config.json layers[%d]" % i
+            if any(isinstance(v, int) and not isinstance(v, bool) and v <= 0 for v in m.values()):
+                raise ConfigError("%s.mixer: sizes must be positive" % where)
+            if m["heads"] % m["kv_heads"]:
+                raise ConfigError("%s.mixer: heads (%d) is not a multiple of kv_heads (%d)" % (where, m["heads"], m["kv_heads"]))
+            rot = m["rot"]
+            if rot and (rot["dims"] % 2 or not (0 < rot["dims"] <= m["dim"]) or not rot["base"] > 0.0):
+                raise ConfigError("%s.mixer.rot: dims must be even and at most dim, base positive" % where)
+            if m["v_mix"]:
+                first = m if first is None else first
+                if (first["kv_heads"], first["vdim"]) != (m["kv_heads"], m["vdim"]):
+                    raise ConfigError("%s.mixer: kv_heads and vdim must equal those of the first layer with v_mix, whose values are blended in" % where)
+            f = layer["mlp"]
+            if f and f["ff"] <= 0:
+                raise ConfigError("%s.mlp: the inner size must be positive" % where)
+            if f and f["kind"] == "moe" and (not f["limit"] > 0.0 or f["experts"] <= 0 or not 0 < f["top"] <= f["experts"]):
+                raise ConfigError("%s.mlp: a positive limit and 1 to %d choices" % (where, max(f["experts"], 1)))

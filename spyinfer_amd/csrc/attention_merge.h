@@ -9,6 +9,24 @@
 // right limit on both sides)
 __device__ __forceinline__ float capped_tanh(float x) { return 1.0f - 2.0f / (1.0f + __expf(2.0f * x)); }
 
+// First key that the query at position p reads: the start of its chunk (chunks of `chunk` positions, counted from the
+// sequence's first token), the start of its window, or 0.  It never falls as p grows, so a tile's first row has the
+// tile's first key.
+__device__ __forceinline__ int attention_first_key(int p, int window, int chunk) {
+    return chunk > 0 ? p - p % chunk : (window > 0 ? max(0, p - window + 1) : 0);
+}
+
+// A gate on the result, sigmoid(gate[t, head d + dd]) for the four columns from dd on: rows of a wider product, `gs` values
+// from one token's row to the next, 8-byte aligned at multiples of four columns.  null: no gate.
+struct OutGate { const bf16_t* g; long long gs; };
+__device__ __forceinline__ void apply_out_gate(const OutGate& og, int t, int col, float (&v)[4]) {
+    if (!og.g) return;
+    float gv[4];
+    Vec4<bf16_t>::load(og.g + (size_t)t * og.gs + col, gv);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= 1.0f / (1.0f + __expf(-gv[e]));
+}
+
 // Where element (row m, column n) lies when at most 16 * tiles rows are kept in MFMA operand order for a product that
 // reads them next: [n / 32 steps][tiles][64 lanes][8], lane 16 g + m % 16 of tile m / 16 holding columns 32 s + 8 g ...
 __device__ __forceinline__ size_t attention_out_operand_order(int m, int n, int tiles) {
@@ -25,7 +43,7 @@ template <int DMAX, bool SINGLE = false>
 __global__ __launch_bounds__(256) void attention_merge_kernel(bf16_t* __restrict__ out, const float* __restrict__ ws,
                                                               const int* __restrict__ cu_q, const int* __restrict__ tile_entry,
                                                               const int* __restrict__ tile_row0, int n_q, int n_kv, int d, int splits,
-                                                              int units_per_tile, int out_tiles = 0) {
+                                                              int units_per_tile, int out_tiles = 0, OutGate og = OutGate{}) {
     __shared__ float wgt[64 * 16];     // weight of part i for row r: [i][r], up to 64 parts
     __shared__ float pm[64 * 16], pl[64 * 16];
     __shared__ float inv_l[16];
@@ -75,6 +93,8 @@ __global__ __launch_bounds__(256) void attention_merge_kernel(bf16_t* __restrict
         }
         const int tq = row / G, head = hk * G + row % G;
         const size_t at = out_tiles ? attention_out_operand_order(q0 + tq, head * d + dd, out_tiles) : ((size_t)(q0 + tq) * n_q + head) * d + dd;
-        out[at] = f32_to_bf16(o * inv_l[r]);
+        float y = o * inv_l[r];
+        if (og.g) y *= 1.0f / (1.0f + __expf(-bf16_to_f32(og.g[(size_t)(q0 + tq) * og.gs + head * d + dd])));
+        out[at] = f32_to_bf16(y);
     }
 }

@@ -133,10 +133,12 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
     int P, int num_pages, const int* __restrict__ cu_q, const int* __restrict__ pos0, const int* __restrict__ kv_len,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tile_entry, const int* __restrict__ tile_row0,
     int n_q, int n_kv, int d, float scale, int window, float softcap, int splits, float* __restrict__ ws, FusedQKV fz, int out_tiles,
-    unsigned* counters, int log2p, const int* __restrict__ pieces, const float* __restrict__ dist, int sink) {
+    unsigned* counters, int log2p, const int* __restrict__ pieces, const float* __restrict__ dist,
+    const float* __restrict__ sink, int chunk, OutGate og) {
     // dist != null: [2, n_q] float32, a penalty on the distance taken off every (capped) score: dist[h] ln(1 + dist[n_q + h] (pos - key)).
-    // sink: the softmax's denominator holds one more term, e^0, that has no value: the first wave of the keys' first part
-    // starts its running maximum at 0 with a sum of 1 (in one of a row's four lanes, whose sums are added at the end).
+    // sink != null: [n_q] float32, the softmax's denominator holds one more term, e^sink[h], that has no value: the first wave
+    // of the keys' first part starts its running maximum at sink[h] with a sum of 1 (in one of a row's four lanes, whose sums
+    // are added at the end).  chunk > 0: keys before the start of a query's chunk are not seen.  og: a gate on the result.
     constexpr int KK = DMAX / 32;   // 32-wide chunks of the head dim for Q.K
     constexpr int DT = DMAX / 16;   // 16-row tiles of the head dim for P.V
     const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
@@ -181,7 +183,7 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
     const int tq = row_ok ? row / G : 0;
     const int head = hk * G + (row_ok ? row % G : 0);
     const int pos = p0 + tq;
-    const int lo_row = window > 0 ? max(0, pos - window + 1) : 0;
+    const int lo_row = attention_first_key(pos, window, chunk);
 
     bf16x8_t bq[KK];
     {
@@ -195,7 +197,7 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
     // keys this tile can see: from the first row's window start to the last row's position
     const int last_row = min(nrows, row0 + 16) - 1;
     const int hi = min(p0 + last_row / G, kvl - 1);
-    int lo = window > 0 ? max(0, p0 + row0 / G - window + 1) : 0;
+    int lo = attention_first_key(p0 + row0 / G, window, chunk);
     lo &= ~31;
     const int nblk = hi >= lo ? (hi - lo) / 32 + 1 : 0;
     const int per = (nblk + splits - 1) / splits;
@@ -205,7 +207,7 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.f;
-    if (sink && sp == 0 && wave == 0 && row_ok) { m = 0.f; l = g == 0 ? 1.f : 0.f; }
+    if (sink && sp == 0 && wave == 0 && row_ok) { m = sink[head]; l = g == 0 ? 1.f : 0.f; }
     const float d1 = dist ? dist[head] : 0.f, d2 = dist ? dist[n_q + head] : 0.f;
 
     // FUSED: the entry's one new token lies at position p0 = kvl - 1; its query rows have that position too.  The block
@@ -336,8 +338,8 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
                 vt[dt] = (v_ok && dd < d) ? *reinterpret_cast<const bf16x8_t*>(vp + (size_t)dd * P) : zero8();
             }
         }
-        if (FULL && window > 0 && !v_ok) {
-            // The window's first block of 32 keys may begin in a page that the window has passed and the request has
+        if (FULL && (window > 0 || chunk > 0) && !v_ok) {
+            // The window's (or chunk's) first block of 32 keys may begin in a page that the window has passed and the request has
             // given back: its keys are masked by their positions, but what page 0 holds in their values' place would
             // still be multiplied (by a weight of zero: harmless for numbers, not for a NaN or an infinity).
 #pragma unroll
@@ -521,9 +523,11 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
         for (int i = 0; i < MINE; ++i) {
             const int dd = (dt0 + i) * 16 + 4 * g;
             if (dd < d) {
+                float y[4] = {mo[i][0] * inv, mo[i][1] * inv, mo[i][2] * inv, mo[i][3] * inv};
+                if constexpr (!FUSED) apply_out_gate(og, q0 + tq, head * d + dd, y);
                 uint2 w;
-                w.x = pack_bf16x2(mo[i][0] * inv, mo[i][1] * inv);
-                w.y = pack_bf16x2(mo[i][2] * inv, mo[i][3] * inv);
+                w.x = pack_bf16x2(y[0], y[1]);
+                w.y = pack_bf16x2(y[2], y[3]);
                 // (four columns from a multiple of 4 never cross a group of 8: one store either way)
                 if (out_tiles) *reinterpret_cast<uint2*>(out + attention_out_operand_order(q0 + tq, head * d + dd, out_tiles)) = w;
                 else *reinterpret_cast<uint2*>(op + dd) = w;
@@ -622,9 +626,11 @@ __global__ __launch_bounds__(AW * 64, (FUSED && DMAX <= 128) ? 2 : 1) void atten
         for (int i = 0; i < MINE; ++i) {
             const int dd = (dt0 + i) * 16 + 4 * g;
             if (dd < d) {
+                float y[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+                if constexpr (!FUSED) apply_out_gate(og, q0 + tq, head * d + dd, y);
                 uint2 w2;
-                w2.x = pack_bf16x2(o[i][0] * inv, o[i][1] * inv);
-                w2.y = pack_bf16x2(o[i][2] * inv, o[i][3] * inv);
+                w2.x = pack_bf16x2(y[0], y[1]);
+                w2.y = pack_bf16x2(y[2], y[3]);
                 if (out_tiles) *reinterpret_cast<uint2*>(out + attention_out_operand_order(q0 + tq, head * d + dd, out_tiles)) = w2;
                 else *reinterpret_cast<uint2*>(op + dd) = w2;
             }
@@ -663,9 +669,13 @@ extern "C" int spy_attention_mfma(void* out, const void* q, void* kc, void* vc, 
                                   const int* tile_row0, int num_tiles, int S, int T, int n_q, int n_kv, int d, float scale,
                                   int window, float softcap, int splits, float* ws, const void* qkv, const void* qw, const void* kw, int w_dtype,
                                   float eps, const float* cos_t, const float* sin_t, int max_pos, int store, int out_tiles,
-                                  unsigned* counters, int n_counters, const int* pieces, int num_pieces, const float* dist, int sink,
-                                  hipStream_t st) {
-    SPY_REQUIRE(!qkv || (!dist && !sink), "spy_attention_mfma: the fused variant takes neither a penalty on the distance nor a sink");
+                                  unsigned* counters, int n_counters, const int* pieces, int num_pieces, const float* dist, const float* sink,
+                                  int chunk, const void* gate, long long gate_ld, hipStream_t st) {
+    SPY_REQUIRE(!qkv || (!dist && !sink && !gate && !chunk), "spy_attention_mfma: the fused variant takes neither a penalty on the distance nor a sink, chunks or a gate");
+    SPY_REQUIRE(chunk >= 0 && !(chunk > 0 && window > 0), "spy_attention_mfma: a window or chunks, not both");
+    SPY_REQUIRE(!gate || (gate_ld >= (long long)n_q * d && gate_ld % 4 == 0 && ((uintptr_t)gate % 8) == 0),
+                "spy_attention_mfma: the gate's rows are too short or not aligned");
+    const OutGate og = {(const bf16_t*)gate, gate_ld};
     SPY_REQUIRE(num_tiles > 0 && S > 0 && T > 0 && n_q > 0 && n_kv > 0 && num_pages > 0 && max_blocks > 0,
                 "spy_attention_mfma: empty operand");
     SPY_REQUIRE(d % 16 == 0 && d >= 16 && d <= 256, "spy_attention_mfma: head_dim %d is not a multiple of 16 in 16..256", d);
@@ -706,7 +716,7 @@ extern "C" int spy_attention_mfma(void* out, const void* q, void* kc, void* vc, 
 #define ATT_LAUNCH(DM, FZ, FL)                                                                                                \
     attention_mfma_kernel<DM, FZ, FL><<<grid, AW * 64, (DM <= 128 ? AW : AW - 1) * ((DM / 16) * 4 + 2) * 64 * sizeof(float), st>>>(  \
         (bf16_t*)out, (const bf16_t*)q, (bf16_t*)kc, (bf16_t*)vc, P, num_pages, cu_q, pos0, kv_len, block_table, max_blocks,  \
-        tile_entry, tile_row0, n_q, n_kv, d, scale, window, softcap, splits, ws, fz, out_tiles, cnt, log2p, pieces, dist, sink)
+        tile_entry, tile_row0, n_q, n_kv, d, scale, window, softcap, splits, ws, fz, out_tiles, cnt, log2p, pieces, dist, sink, chunk, og)
 #define ATT_CASE(DM)                                                                                                          \
     if (qkv && P <= 32) ATT_LAUNCH(DM, true, FULL_STREAMED); else if (qkv) ATT_LAUNCH(DM, true, FULL_KEPT);                      \
     else if (d == DM && P <= 32) ATT_LAUNCH(DM, false, FULL_STREAMED); else if (d == DM) ATT_LAUNCH(DM, false, FULL_KEPT);       \
@@ -715,7 +725,7 @@ extern "C" int spy_attention_mfma(void* out, const void* q, void* kc, void* vc, 
     else if (splits > 1 && qkv)                                                                                               \
         attention_merge_kernel<DM, true><<<mgrid, 256, 0, st>>>((bf16_t*)out, ws, cu_q, tile_entry, tile_row0, n_q, n_kv, d, splits, 1, out_tiles); \
     else if (splits > 1)                                                                                                      \
-        attention_merge_kernel<DM><<<mgrid, 256, 0, st>>>((bf16_t*)out, ws, cu_q, tile_entry, tile_row0, n_q, n_kv, d, splits, 1, out_tiles);
+        attention_merge_kernel<DM><<<mgrid, 256, 0, st>>>((bf16_t*)out, ws, cu_q, tile_entry, tile_row0, n_q, n_kv, d, splits, 1, out_tiles, og);
     switch (dmax_of(d)) {
         case 64: ATT_CASE(64) break;
         case 128: ATT_CASE(128) break;

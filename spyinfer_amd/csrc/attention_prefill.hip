@@ -38,10 +38,11 @@ __global__ __launch_bounds__(PF_ROWS / RT * 4, MINW) void attention_prefill_kern
     int P, int num_pages, const int* __restrict__ cu_q, const int* __restrict__ pos0, const int* __restrict__ kv_len,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tile_entry, const int* __restrict__ tile_row0,
     int n_q, int n_kv, int d, float scale, int window, float softcap, int log2p, int num_tiles, int splits, float* __restrict__ ws, int out_tiles,
-    const float* __restrict__ dist, int sink) {
+    const float* __restrict__ dist, const float* __restrict__ sink, int chunk, OutGate og) {
     // dist != null: [2, n_q] float32, a penalty on the distance taken off every (capped) score: dist[h] ln(1 + dist[n_q + h] (pos - key)).
-    // sink: the softmax's denominator holds one more term, e^0, that has no value: in the keys' first part a row's running
-    // maximum starts at 0 with a sum of 1 (in one of the row's four lanes, whose sums are added at the end).
+    // sink != null: [n_q] float32, the softmax's denominator holds one more term, e^sink[h], that has no value: in the keys'
+    // first part a row's running maximum starts at sink[h] with a sum of 1 (in one of the row's four lanes, whose sums are
+    // added at the end).  chunk > 0: keys before the start of a query's chunk are not seen.  og: a gate on the result.
     constexpr int KK = DMAX / 32, DT = DMAX / 16;
     // 16 elements of padding per staged row: the products' 16-byte reads then have no bank conflicts (measured with
     // SQ_LDS_BANK_CONFLICT: 40 % of the LDS cycles with 8, none with 16; the kernel's time follows only by 0-3 %)
@@ -101,7 +102,7 @@ __global__ __launch_bounds__(PF_ROWS / RT * 4, MINW) void attention_prefill_kern
         tq[t] = row_ok[t] ? row / G : 0;
         head[t] = hk * G + (row_ok[t] ? row % G : 0);
         pos[t] = p0 + tq[t];
-        lo_row[t] = window > 0 ? max(0, pos[t] - window + 1) : 0;
+        lo_row[t] = attention_first_key(pos[t], window, chunk);
         const bf16_t* qp = q + ((size_t)(q0 + tq[t]) * n_q + head[t]) * d;
 #pragma unroll
         for (int kk = 0; kk < KK; ++kk) {
@@ -112,16 +113,16 @@ __global__ __launch_bounds__(PF_ROWS / RT * 4, MINW) void attention_prefill_kern
     // keys the block can see, and those this wave can see (wave-uniform)
     const int blk_last_row = min(nrows, row0 + PF_ROWS) - 1;
     const int hi = min(p0 + blk_last_row / G, kvl - 1);
-    int lo = window > 0 ? max(0, p0 + row0 / G - window + 1) : 0;
+    int lo = attention_first_key(p0 + row0 / G, window, chunk);
     lo &= ~(PF_KEYS - 1);
     const int nblk = hi >= lo ? (hi - lo) / PF_KEYS + 1 : 0;
     const int w_first_row = row0 + 16 * RT * wave;
     const int w_last_row = min(nrows, w_first_row + 16 * RT) - 1;
     const int w_hi = w_last_row >= w_first_row ? p0 + w_last_row / G : -1;               // last key any row of the wave reads
-    const int w_lo = window > 0 ? max(0, p0 + w_first_row / G - window + 1) : 0;           // first key any row of the wave reads
+    const int w_lo = attention_first_key(p0 + w_first_row / G, window, chunk);             // first key any row of the wave reads
     const bool w_rows_full = w_first_row + 16 * RT - 1 < nrows;                             // all rows of the wave exist
     const int w_min_pos = p0 + w_first_row / G;                                            // keys up to here are before every row
-    const int w_max_lo = window > 0 ? max(0, w_hi - window + 1) : 0;                       // keys from here on are in every window
+    const int w_max_lo = w_hi >= 0 ? attention_first_key(w_hi, window, chunk) : 0;         // keys from here on are in every row's window or chunk
     const float cap_over_scale = softcap > 0.f ? softcap / scale : 0.f, scale_over_cap = softcap > 0.f ? scale / softcap : 0.f;
     const float scale2 = scale * 1.4426950408889634f;                                      // scores times log2(e)
 
@@ -139,7 +140,7 @@ __global__ __launch_bounds__(PF_ROWS / RT * 4, MINW) void attention_prefill_kern
     for (int t = 0; t < RT; ++t) {
         dl1[t] = dist ? dist[head[t]] * 0.6931471805599453f / scale : 0.f;
         dl2[t] = dist ? dist[n_q + head[t]] : 0.f;
-        if (sink && part == 0 && row_ok[t]) { m[t] = 0.f; l[t] = g == 0 ? 1.f : 0.f; }
+        if (sink && part == 0 && row_ok[t]) { m[t] = sink[head[t]] * 1.4426950408889634f; l[t] = g == 0 ? 1.f : 0.f; }
     }
 
     bf16x8_t pk[NV], pv[NV];
@@ -368,9 +369,11 @@ __global__ __launch_bounds__(PF_ROWS / RT * 4, MINW) void attention_prefill_kern
         for (int dt = 0; dt < DT; ++dt) {
             const int dd = dt * 16 + 4 * g;
             if (dd < d) {
+                float y[4] = {acc[t][dt][0] * inv, acc[t][dt][1] * inv, acc[t][dt][2] * inv, acc[t][dt][3] * inv};
+                apply_out_gate(og, q0 + tq[t], head[t] * d + dd, y);
                 uint2 w;
-                w.x = pack_bf16x2(acc[t][dt][0] * inv, acc[t][dt][1] * inv);
-                w.y = pack_bf16x2(acc[t][dt][2] * inv, acc[t][dt][3] * inv);
+                w.x = pack_bf16x2(y[0], y[1]);
+                w.y = pack_bf16x2(y[2], y[3]);
                 // (four columns from a multiple of 4 never cross a group of 8: one store either way)
                 if (out_tiles) *reinterpret_cast<uint2*>(out + attention_out_operand_order(q0 + tq[t], head[t] * d + dd, out_tiles)) = w;
                 else *reinterpret_cast<uint2*>(op + dd) = w;
@@ -406,8 +409,8 @@ static long long cu_count() {
 extern "C" int spy_attention_prefill(void* out, const void* q, const void* kc, const void* vc, int P, int num_pages, const int* cu_q,
                                      const int* pos0, const int* kv_len, const int* block_table, int max_blocks,
                                      const int* tile_entry, const int* tile_row0, int num_tiles, int tile_rows, int S, int T, int n_q,
-                                     int n_kv, int d, float scale, int window, float softcap, int splits, float* ws, int out_tiles, const float* dist, int sink,
-                                     hipStream_t st) {
+                                     int n_kv, int d, float scale, int window, float softcap, int splits, float* ws, int out_tiles, const float* dist, const float* sink,
+                                     int chunk, const void* gate, long long gate_ld, hipStream_t st) {
     SPY_REQUIRE(num_tiles > 0 && S > 0 && T > 0 && n_q > 0 && n_kv > 0 && num_pages > 0 && max_blocks > 0,
                 "spy_attention_prefill: empty operand");
     SPY_REQUIRE(d % 16 == 0 && d >= 16 && d <= 128, "spy_attention_prefill: head_dim %d is not a multiple of 16 in 16..128", d);
@@ -424,11 +427,16 @@ extern "C" int spy_attention_prefill(void* out, const void* q, const void* kc, c
     // decode product that reads it next
     SPY_REQUIRE(out_tiles >= 0 && out_tiles <= 8 && (!out_tiles || (T <= 16 * out_tiles && (n_q * d) % 32 == 0 && d % 8 == 0)),
                 "spy_attention_prefill: operand order is for at most 128 rows (%d here) of a width that is a multiple of 32", T);
+    SPY_REQUIRE(chunk >= 0 && !(chunk > 0 && window > 0), "spy_attention_prefill: a window or chunks, not both");
+    SPY_REQUIRE(!gate || (gate_ld >= (long long)n_q * d && gate_ld % 4 == 0 && ((uintptr_t)gate % 8) == 0),
+                "spy_attention_prefill: the gate's rows are too short or not aligned");
+    const OutGate og = {(const bf16_t*)gate, gate_ld};
     const dim3 grid(splits > 1 ? num_tiles : (num_tiles + 1) / 2, n_kv, splits);
     const dim3 mgrid(num_tiles * (tile_rows / 16), n_kv);
     const bool one_per_cu = (long long)grid.x * grid.y * grid.z <= cu_count();
 #define PF_ARGS (bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, P, num_pages, cu_q, pos0, kv_len, block_table,   \
-                max_blocks, tile_entry, tile_row0, n_q, n_kv, d, scale, window, softcap, log2p, num_tiles, splits, ws, out_tiles, dist, sink
+                max_blocks, tile_entry, tile_row0, n_q, n_kv, d, scale, window, softcap, log2p, num_tiles, splits, ws, out_tiles, dist, sink, \
+                chunk, og
     // (head sizes other than 64 and 128 keep the 4-wave shape: with conditions in the head-dim loops the other needs too many registers)
 #define PF_CASE(DM)                                                                                                              \
     if (tile_rows == 256) attention_prefill_kernel<DM, true, 2, 2, 256><<<grid, 512, 0, st>>>(PF_ARGS);                          \
@@ -438,7 +446,7 @@ extern "C" int spy_attention_prefill(void* out, const void* q, const void* kc, c
     } else attention_prefill_kernel<DM, false, 2, 2, 128><<<grid, 256, 0, st>>>(PF_ARGS);                                        \
     if (splits > 1)                                                                                                              \
         attention_merge_kernel<DM><<<mgrid, 256, 0, st>>>((bf16_t*)out, ws, cu_q, tile_entry, tile_row0, n_q, n_kv, d, splits,    \
-                                                          tile_rows / 16, out_tiles);
+                                                          tile_rows / 16, out_tiles, og);
     if (d <= 64) { PF_CASE(64) } else { PF_CASE(128) }
 #undef PF_CASE
 #undef PF_ARGS

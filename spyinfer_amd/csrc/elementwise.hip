@@ -19,9 +19,38 @@ __global__ void embedding_kernel(float* __restrict__ out, const TW* __restrict__
     for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = to_f32<TW>(row[i]) * scale;
 }
 
+// out[t, :] = row / sqrt(mean(row^2) + eps) * w, row = table[ids[t], :] * scale: an embedding that is normed before the first
+// layer.  The row is read twice, the second time from the caches.
+template <typename TW>
+__global__ void embedding_norm_kernel(float* __restrict__ out, const TW* __restrict__ table, const int* __restrict__ ids, int H, int V,
+                                      float scale, const float* __restrict__ w, float eps) {
+    __shared__ float red[16];
+    const int t = blockIdx.x;
+    const int id = ids[t];
+    float* o = out + (size_t)t * H;
+    if (id < 0 || id >= V) {
+        for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = 0.f;
+        return;
+    }
+    const TW* row = table + (size_t)id * H;
+    float ss = 0.f;
+#pragma unroll 4
+    for (int i = threadIdx.x; i < H; i += blockDim.x) { const float v = to_f32<TW>(row[i]) * scale; ss = fmaf(v, v, ss); }
+    ss = block_sum(ss, red);
+    const float r = 1.0f / sqrtf(ss / (float)H + eps);
+#pragma unroll 4
+    for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = (r * (to_f32<TW>(row[i]) * scale)) * w[i];
+}
+
+// norm_w (float32 [H], or null): the rows are normed
 extern "C" int spy_embedding(float* out, const void* table, int table_dtype, const int* ids, int T, int H, int V, float scale,
-                             hipStream_t st) {
+                             const float* norm_w, float eps, hipStream_t st) {
     SPY_REQUIRE(T > 0 && H > 0 && V > 0, "spy_embedding: empty operand");
+    if (norm_w) {
+        SPY_DISPATCH(table_dtype, TW, (embedding_norm_kernel<TW><<<T, H >= 1024 ? 256 : 64, 0, st>>>(out, (const TW*)table, ids, H, V, scale, norm_w, eps)));
+        SPY_CHECK_LAUNCH("spy_embedding");
+        return 0;
+    }
     SPY_DISPATCH(table_dtype, TW, embedding_kernel<TW><<<T, 256, 0, st>>>(out, (const TW*)table, ids, H, V, scale));
     SPY_CHECK_LAUNCH("spy_embedding");
     return 0;
@@ -309,21 +338,21 @@ extern "C" int spy_scale_cap(float* x, int64_t n, float scale, float cap, hipStr
 }
 
 // ---------------------------------------------------------------------------------------------
-// out[t, i] = silu(in[t, i]) * in[t, I + i]
+// out[t, i] = act(in[t, i]) * in[t, I + i], act silu or the tanh form of gelu (GateAct)
 template <typename TA>
-__global__ void swiglu_kernel(const TA* __restrict__ in, TA* __restrict__ out, int T, int I) {
+__global__ void swiglu_kernel(const TA* __restrict__ in, TA* __restrict__ out, int T, int I, GateAct act) {
     const size_t n = (size_t)T * I;
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < n; idx += (size_t)gridDim.x * blockDim.x) {
         const size_t t = idx / I, i = idx - t * I;
         const float g = to_f32<TA>(in[t * 2 * I + i]);
         const float u = to_f32<TA>(in[t * 2 * I + I + i]);
-        out[idx] = from_f32<TA>((g / (1.0f + expf(-g))) * u);
+        out[idx] = from_f32<TA>(gated_value(act, g, u));
     }
 }
 
 // the same, 4 values per thread and step with vector loads (I % 4 == 0, 16-byte aligned rows)
 template <typename TA>
-__global__ void swiglu_vec_kernel(const TA* __restrict__ in, TA* __restrict__ out, int T, int I4) {
+__global__ void swiglu_vec_kernel(const TA* __restrict__ in, TA* __restrict__ out, int T, int I4, GateAct act) {
     const size_t n = (size_t)T * I4;
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < n; idx += (size_t)gridDim.x * blockDim.x) {
         const size_t t = idx / I4, i = (idx - t * I4) * 4;
@@ -332,14 +361,14 @@ __global__ void swiglu_vec_kernel(const TA* __restrict__ in, TA* __restrict__ ou
         Vec4<TA>::load(in + t * 2 * I + i, g);
         Vec4<TA>::load(in + t * 2 * I + I + i, u);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) y[e] = (g[e] / (1.0f + expf(-g[e]))) * u[e];
+        for (int e = 0; e < 4; ++e) y[e] = gated_value(act, g[e], u[e]);
         Vec4<TA>::store(out + t * I + i, y);
     }
 }
 
 // bfloat16, 8 values per thread and step: 16-byte loads that do not stay in the caches (the product's output passes
 // once), one 16-byte store (the next product reads it)
-__global__ void swiglu_bf16x8_kernel(const bf16_t* __restrict__ in, bf16_t* __restrict__ out, int T, int I8) {
+__global__ void swiglu_bf16x8_kernel(const bf16_t* __restrict__ in, bf16_t* __restrict__ out, int T, int I8, GateAct act) {
     typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4_t;
     const size_t n = (size_t)T * I8, I = (size_t)I8 * 8;
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < n; idx += (size_t)gridDim.x * blockDim.x) {
@@ -351,13 +380,15 @@ __global__ void swiglu_bf16x8_kernel(const bf16_t* __restrict__ in, bf16_t* __re
         for (int e = 0; e < 4; ++e) {
             const float g0 = __uint_as_float(g[e] << 16), g1 = __uint_as_float(g[e] & 0xffff0000u);
             const float u0 = __uint_as_float(u[e] << 16), u1 = __uint_as_float(u[e] & 0xffff0000u);
-            y[e] = pack_bf16x2((g0 / (1.0f + expf(-g0))) * u0, (g1 / (1.0f + expf(-g1))) * u1);
+            y[e] = pack_bf16x2(gated_value(act, g0, u0), gated_value(act, g1, u1));
         }
         *reinterpret_cast<u32x4_t*>(out + t * I + i) = y;
     }
 }
 
-extern "C" int spy_swiglu(const void* in, void* out, int dtype, int T, int I, hipStream_t st) {
+extern "C" int spy_swiglu(const void* in, void* out, int dtype, int T, int I, int act_code, hipStream_t st) {
+    GateAct act;
+    SPY_REQUIRE(gate_act_of(act_code, &act), "spy_swiglu: unknown activation %d", act_code);
     SPY_REQUIRE(T > 0 && I > 0, "spy_swiglu: empty operand");
     const bool vec = I % 8 == 0 && ((uintptr_t)in % 16) == 0 && ((uintptr_t)out % 16) == 0;
     const size_t n = (size_t)T * I / (vec ? 4 : 1);
@@ -365,11 +396,11 @@ extern "C" int spy_swiglu(const void* in, void* out, int dtype, int T, int I, hi
     if (vec && dtype == SPY_BF16) {
         const size_t n8 = (size_t)T * I / 8;
         const unsigned b8 = (unsigned)((n8 + 255) / 256 > 65536 ? 65536 : (n8 + 255) / 256);
-        swiglu_bf16x8_kernel<<<b8, 256, 0, st>>>((const bf16_t*)in, (bf16_t*)out, T, I / 8);
+        swiglu_bf16x8_kernel<<<b8, 256, 0, st>>>((const bf16_t*)in, (bf16_t*)out, T, I / 8, act);
     } else if (vec) {
-        SPY_DISPATCH(dtype, TA, swiglu_vec_kernel<TA><<<blocks, 256, 0, st>>>((const TA*)in, (TA*)out, T, I / 4));
+        SPY_DISPATCH(dtype, TA, swiglu_vec_kernel<TA><<<blocks, 256, 0, st>>>((const TA*)in, (TA*)out, T, I / 4, act));
     } else {
-        SPY_DISPATCH(dtype, TA, swiglu_kernel<TA><<<blocks, 256, 0, st>>>((const TA*)in, (TA*)out, T, I));
+        SPY_DISPATCH(dtype, TA, swiglu_kernel<TA><<<blocks, 256, 0, st>>>((const TA*)in, (TA*)out, T, I, act));
     }
     SPY_CHECK_LAUNCH("spy_swiglu");
     return 0;

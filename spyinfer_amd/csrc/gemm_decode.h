@@ -68,6 +68,7 @@ __device__ __forceinline__ void gd_residual_epilogue(const f32x4_t& v, const f32
 struct GdArgs {
     const bf16_t* x; const bf16_t* w; void* c; float* resid; bf16_t* xw_out; const bf16_t* w_next; float* ss_out; const float* ss_in;
     int n_parts; float eps; int M, N, K; bool xt, ot; hipStream_t st;
+    GateAct act;                           // the gated epilogue's activation
     void* ws; long long ws_bytes;          // the device's workspace of the products that split K over blocks (or none)
 };
 

@@ -9,7 +9,7 @@
 //             x . W^T with x = norm(h), the scale applied after the sum instead of before it.  The one
 //             rounding of the operand to bfloat16 happens before the scale, which changes nothing in its
 //             relative size.
-//   EPI_GATED W = [gate | up] tiles, the block stores silu(gate) * up.
+//   EPI_GATED W = [gate | up] tiles, the block stores act(gate) * up (silu or the tanh form of gelu).
 //   XT / OT   the input X / the bfloat16 output that the next product reads (bf16(h w) of EPI_RESID, the result of
 //             EPI_GATED) in MFMA operand order instead of row-major: [K/32 steps][64 lanes][8], lane 16 g + r of step s
 //             holding x[r][32 s + 8 g ..] for the 16 rows of the tile (rows beyond M hold anything).  An operand is then
@@ -40,7 +40,7 @@ template <int EPI, bool SCALED, typename TC, int GD_WAVES, bool XT, bool OT, int
 __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_kernel(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ Wt, TC* __restrict__ C, float* __restrict__ resid_out,
     bf16_t* __restrict__ xw_out, const bf16_t* __restrict__ w_next, float* __restrict__ ss_out, const float* __restrict__ ss_in,
-    int n_parts, float eps, int M, int N, int K) {
+    int n_parts, float eps, int M, int N, int K, GateAct gact) {
     constexpr bool H3 = HT != 0;
     static_assert(!H3 || (EPI == EPI_STORE && (HT == 3 || HT == 5)), "three or five halves of column tiles, the stored product only");
     constexpr int NT = H3 ? (HT + 1) / 2 : (EPI == EPI_GATED ? 2 : 1);
@@ -190,7 +190,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         float v = acc[0][i];
-        if (EPI == EPI_GATED) { const float up = acc[NT - 1][i]; v = (v / (1.0f + expf(-v))) * up; }
+        if (EPI == EPI_GATED) v = gated_value(gact, v, acc[NT - 1][i]);
         if (act) v = xielu_f(v, act_p, act_q);
         out[i] = from_f32<TC>(v);
     }
@@ -206,7 +206,7 @@ template <int EPI, bool SCALED, typename TC, int MT, int CT, int GD_WAVES, bool 
 __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_rows_kernel(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ Wt, TC* __restrict__ C, float* __restrict__ resid_out,
     bf16_t* __restrict__ xw_out, const bf16_t* __restrict__ w_next, float* __restrict__ ss_out, const float* __restrict__ ss_in,
-    int n_parts, float eps, int M, int N, int K) {
+    int n_parts, float eps, int M, int N, int K, GateAct gact) {
     static_assert(!H3 || (EPI == EPI_STORE && CT == 2), "halves of column tiles: the stored product, two tiles a block");
     constexpr int NT = (EPI == EPI_GATED ? 2 : 1) * CT;      // W tiles per block: [gate tiles | up tiles] for the gated product
     constexpr int MP = 16 * MT;
@@ -374,7 +374,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_rows_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 float v = acc[ct][mt][i];
-                if (EPI == EPI_GATED) { const float up = acc[CT + ct][mt][i]; v = (v / (1.0f + expf(-v))) * up; }
+                if (EPI == EPI_GATED) v = gated_value(gact, v, acc[CT + ct][mt][i]);
                 if (act) v = xielu_f(v, act_p, act_q);
                 out[i] = from_f32<TC>(v);
             }
@@ -399,7 +399,7 @@ int gd_compute_units() {
 template <int EPI, bool SCALED, typename TC, bool XT, bool OT>
 static bool gd_launch2(const GdArgs& a) {
     constexpr int W = EPI == EPI_GATED ? GD_WAVES_GATED : 8;
-#define GD_ARGS a.x, a.w, (TC*)a.c, a.resid, a.xw_out, a.w_next, a.ss_out, a.ss_in, a.n_parts, a.eps, a.M, a.N, a.K
+#define GD_ARGS a.x, a.w, (TC*)a.c, a.resid, a.xw_out, a.w_next, a.ss_out, a.ss_in, a.n_parts, a.eps, a.M, a.N, a.K, a.act
     // Two column tiles per block where that leaves enough blocks (measured, 64 rows: qkv of 6144 columns 26.8 -> 20.5
     // us; with 4096 columns, 128 blocks, 15.4 -> 19.4 us; the gated product 53 -> 61 us: its block has one wave per SIMD then)
     const bool two = EPI == EPI_STORE && a.N % 32 == 0 && a.N / 32 >= 192;
@@ -482,12 +482,12 @@ extern "C" int64_t spy_gemm_decode_workspace() { return gd_splitk_workspace_byte
 // x: bfloat16 [M, K], M <= 128; MP = 16 times the row tiles the kernel is built with (M rounded up to 16 up to 64 rows, 96
 // or 128 beyond).  scaled != 0: x = bf16(h * w_norm) and ss_in
 // [n_parts, MP] holds the parts of sum(h^2); the result is multiplied by rsqrt(sum / K + eps).
-// epi 0: C [M, N] (c_dtype), with w_next = two bfloat16 numbers (p, q): xIELU of the result;  epi 1: W = [gate | up], C [M, N] = silu(gate) * up;  epi 2: resid [M, N] += result,
+// epi 0: C [M, N] (c_dtype), with w_next = two bfloat16 numbers (p, q): xIELU of the result;  epi 1: W = [gate | up], C [M, N] = act(gate) * up (act: SPY_ACT_*);  epi 2: resid [M, N] += result,
 // xw_out [M, N] = bf16(resid * w_next), ss_out [N / 16, MP] = every block's part of the rows' sums of squares.
 // x_tiled / out_tiled: X / the bfloat16 output for the next product (xw_out of epi 2, C of epi 1) are in operand order.
 extern "C" int spy_gemm_decode(const void* X, int scaled, const float* ss_in, int n_parts, float eps, const void* Wt, int epi,
                                void* C, int c_dtype, float* resid, void* xw_out, const void* w_next, float* ss_out, int M, int N,
-                               int K, int x_tiled, int out_tiled, void* ws, int64_t ws_bytes, hipStream_t st) {
+                               int K, int x_tiled, int out_tiled, int act, void* ws, int64_t ws_bytes, hipStream_t st) {
     SPY_REQUIRE(M > 0 && M <= 128, "spy_gemm_decode: M = %d rows (1..128 allowed)", M);
     SPY_REQUIRE(N > 0 && N % 16 == 0 && K > 0 && K % 128 == 0, "spy_gemm_decode: N = %d must be a multiple of 16 and K = %d of 128", N, K);
     SPY_REQUIRE(epi >= 0 && epi <= 2, "spy_gemm_decode: unknown epilogue %d", epi);
@@ -501,8 +501,10 @@ extern "C" int spy_gemm_decode(const void* X, int scaled, const float* ss_in, in
     SPY_REQUIRE((long long)N * 256 + 8192 < (1ll << 32), "spy_gemm_decode: N = %d is too large for 32-bit offsets inside a chunk", N);
     SPY_REQUIRE(!out_tiled || (N % 32 == 0 && (epi == EPI_RESID || (epi == EPI_GATED && c_dtype == SPY_BF16))),
                 "spy_gemm_decode: operand order is for the bfloat16 output of the gated and the residual epilogue, N a multiple of 32");
+    GateAct gact;
+    SPY_REQUIRE(gate_act_of(act, &gact), "spy_gemm_decode: unknown activation %d of the gated epilogue", act);
     GdArgs a = {(const bf16_t*)X, (const bf16_t*)Wt, C, resid, (bf16_t*)xw_out, (const bf16_t*)w_next, ss_out, ss_in, n_parts, eps, M, N, K,
-                x_tiled != 0, out_tiled != 0, st, ws, (long long)ws_bytes};
+                x_tiled != 0, out_tiled != 0, st, gact, ws, (long long)ws_bytes};
     const bool f32 = c_dtype == SPY_F32;
     // (a stored product with an activation is built in this file's kernels only)
     const bool store_act = epi == EPI_STORE && w_next != nullptr;

@@ -18,7 +18,7 @@
 template <int EPI, bool SCALED, typename TC, int MT, int CT, bool XT, bool OT, int GW = 8>
 __global__ __launch_bounds__(GW * 64, 1) void gemm_decode_wide_kernel(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ Wt, TC* __restrict__ C, const float* __restrict__ ss_in,
-    int n_parts, float eps, int M, int N, int K) {
+    int n_parts, float eps, int M, int N, int K, GateAct gact) {
     static_assert(EPI == EPI_STORE || EPI == EPI_GATED, "the wide kernel has no residual epilogue");
     static_assert(GW == 8 || GW == 4, "four or eight waves");
     static_assert((EPI == EPI_GATED ? 2 : 1) * CT * MT <= (GW == 8 ? 24 : 48), "the accumulators of a group must fit the registers");
@@ -195,7 +195,7 @@ __global__ __launch_bounds__(GW * 64, 1) void gemm_decode_wide_kernel(
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         float y = v[i] * scale;
-                        if (EPI == EPI_GATED) { const float u = up[i] * scale; y = (y / (1.0f + expf(-y))) * u; }
+                        if (EPI == EPI_GATED) y = gated_value(gact, y, up[i] * scale);
                         out[i] = from_f32<TC>(y);
                     }
                 }
@@ -239,7 +239,7 @@ static bool gd_launch_wide_with(const GdArgs& a, int ct, int blocks) {
     if constexpr (C <= MAX_CT && C >= MIN_CT) {                                                                       \
         if (ct == C) {                                                                                                \
             gemm_decode_wide_kernel<EPI, SCALED, TC, MT, C, XT, OT, GW><<<blocks, GW * 64, 0, a.st>>>(                    \
-                a.x, a.w, (TC*)a.c, a.ss_in, a.n_parts, a.eps, a.M, a.N, a.K);                                        \
+                a.x, a.w, (TC*)a.c, a.ss_in, a.n_parts, a.eps, a.M, a.N, a.K, a.act);                                      \
             return true;                                                                                              \
         }                                                                                                             \
     }

@@ -22,12 +22,12 @@ __device__ __forceinline__ bf16x8_t load8(const bf16_t* p, bool ok) {
 }
 
 // GATED (with NT = 2): W holds [gate rows | up rows], N is the number of gate rows; tile 0 of a block is
-// 16 gate rows, tile 1 the 16 up rows of the same columns, and the block stores silu(gate) * up [M, N]:
-// the SwiGLU of a gated feed-forward without a pass of its own.
+// 16 gate rows, tile 1 the 16 up rows of the same columns, and the block stores act(gate) * up [M, N]:
+// the activation of a gated feed-forward without a pass of its own.
 // (The products of at most 16 rows with weights copied into MFMA tile order are in gemm_decode.hip.)
 template <int MT, int NT, int WAVES, typename TC, bool GATED = false>
 __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
-                                                                 TC* __restrict__ C, int M, int N, int K) {
+                                                                 TC* __restrict__ C, int M, int N, int K, GateAct gact = GateAct{}) {
     __shared__ float red[(WAVES - 1) * NT * MT * 64 * 4];
     // the wave index is the same in all lanes: keep it in a scalar register so that loops over it are scalar too
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
@@ -159,7 +159,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* _
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const float gt = acc[0][mt][i], up = acc[NT - 1][mt][i];
-                if (n + i < N) out[i] = from_f32<TC>((gt / (1.0f + expf(-gt))) * up);
+                if (n + i < N) out[i] = from_f32<TC>(gated_value(gact, gt, up));
             }
         }
         return;
@@ -191,8 +191,10 @@ static void pick_skinny(const bf16_t* X, const bf16_t* W, void* C, int M, int N,
     launch_skinny<MT, 1, 8, TC>(X, W, C, M, N, K, st);
 }
 
-// out[M, I] = silu(X . Wgate^T) * (X . Wup^T) with W = [Wgate | Wup] stored [2 I, K]
-extern "C" int spy_gemm_skinny_swiglu(const void* X, const void* W, void* C, int c_dtype, int M, int I, int K, hipStream_t st) {
+// out[M, I] = act(X . Wgate^T) * (X . Wup^T) with W = [Wgate | Wup] stored [2 I, K]
+extern "C" int spy_gemm_skinny_swiglu(const void* X, const void* W, void* C, int c_dtype, int M, int I, int K, int act, hipStream_t st) {
+    GateAct gact;
+    SPY_REQUIRE(gate_act_of(act, &gact), "spy_gemm_skinny_swiglu: unknown activation %d", act);
     SPY_REQUIRE(M > 0 && I > 0 && K > 0, "spy_gemm_skinny_swiglu: empty operand");
     SPY_REQUIRE(M <= 16, "spy_gemm_skinny_swiglu: M = %d exceeds 16 rows", M);
     SPY_REQUIRE(K % 8 == 0, "spy_gemm_skinny_swiglu: K = %d is not a multiple of 8", K);
@@ -200,9 +202,9 @@ extern "C" int spy_gemm_skinny_swiglu(const void* X, const void* W, void* C, int
     SPY_REQUIRE((long long)(I + 16) * K * 2 < (1ll << 32), "spy_gemm_skinny_swiglu: the gate and up rows lie too far apart");
     const int blocks = (I + 15) / 16;
     if (c_dtype == SPY_F32)
-        gemm_skinny_kernel<1, 2, 8, float, true><<<blocks, 8 * 64, 0, st>>>((const bf16_t*)X, (const bf16_t*)W, (float*)C, M, I, K);
+        gemm_skinny_kernel<1, 2, 8, float, true><<<blocks, 8 * 64, 0, st>>>((const bf16_t*)X, (const bf16_t*)W, (float*)C, M, I, K, gact);
     else
-        gemm_skinny_kernel<1, 2, 8, bf16_t, true><<<blocks, 8 * 64, 0, st>>>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, I, K);
+        gemm_skinny_kernel<1, 2, 8, bf16_t, true><<<blocks, 8 * 64, 0, st>>>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, I, K, gact);
     SPY_CHECK_LAUNCH("spy_gemm_skinny_swiglu");
     return 0;
 }

@@ -10,7 +10,8 @@
 //   gemm:    C[row] = A[source of row] . W[expert of the row's tile]^T, float32 products and sums; optionally gated:
 //            W = [gate rows | up rows], C = silu(gate) * up; or (MoeAct kind 1) with the row's weight w multiplied into both
 //            sums first, g = min(w gate, limit), u = clamp(w up, -limit, limit), C = g sigmoid(1.702 g) (u + 1).
-//   combine: out[t] = sum_k weight[t, k] * Y[row of pair (t, k)].
+//            Where tables name the experts by token id, the align step of all mixtures is one launch ahead of the layers.
+//   combine: out[t] = scale * sum_k weight[t, k] * Y[row of pair (t, k)].
 #include "common.h"
 #include <math.h>
 
@@ -128,17 +129,18 @@ extern "C" int spy_moe_route(int* ids, float* weights, const float* z, const flo
     return 0;
 }
 
-// One block.  ids [P] -> sorted_pair [max_tiles MOE_TM] (pair or -1), pair_row [P], tile_expert [max_tiles] (expert or -1).
-__global__ __launch_bounds__(1024) void moe_align_kernel(int* __restrict__ sorted_pair, int* __restrict__ pair_row,
-                                                         int* __restrict__ tile_expert, const int* __restrict__ ids, int P, int E,
-                                                         int max_tiles) {
+// One block.  Pair p's expert is expert_of(p) (outside 0 .. E - 1: the pair has no row) -> sorted_pair [max_tiles MOE_TM]
+// (pair or -1), pair_row [P], tile_expert [max_tiles] (expert or -1).
+template <typename F>
+__device__ __forceinline__ void moe_align_block(int* __restrict__ sorted_pair, int* __restrict__ pair_row, int* __restrict__ tile_expert,
+                                                F expert_of, int P, int E, int max_tiles) {
     __shared__ int count[MOE_MAX_EXPERTS], first[MOE_MAX_EXPERTS], cursor[MOE_MAX_EXPERTS];
     __shared__ int total_tiles;
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += blockDim.x) { count[e] = 0; cursor[e] = 0; }
     __syncthreads();
     for (int p = tid; p < P; p += blockDim.x) {
-        const int e = ids[p];
+        const int e = expert_of(p);
         if (e >= 0 && e < E) atomicAdd(&count[e], 1);
     }
     __syncthreads();
@@ -160,12 +162,57 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(int* __restrict__ sorte
     for (int i = total_tiles + tid; i < max_tiles; i += blockDim.x) tile_expert[i] = -1;
     for (int r = total_tiles * MOE_TM + tid; r < max_tiles * MOE_TM; r += blockDim.x) sorted_pair[r] = -1;
     for (int p = tid; p < P; p += blockDim.x) {
-        const int e = ids[p];
+        const int e = expert_of(p);
         if (e < 0 || e >= E) { pair_row[p] = -1; continue; }
         const int row = first[e] * MOE_TM + atomicAdd(&cursor[e], 1);
         if (row < max_tiles * MOE_TM) sorted_pair[row] = p;
         pair_row[p] = row < max_tiles * MOE_TM ? row : -1;
     }
+}
+
+__global__ __launch_bounds__(1024) void moe_align_kernel(int* __restrict__ sorted_pair, int* __restrict__ pair_row,
+                                                         int* __restrict__ tile_expert, const int* __restrict__ ids, int P, int E,
+                                                         int max_tiles) {
+    moe_align_block(sorted_pair, pair_row, tile_expert, [=](int p) { return ids[p]; }, P, E, max_tiles);
+}
+
+// Experts named by tables of the token ids: all of a step's mixtures at once, one block per mixture.  Mixture l: the table
+// [V, top] (int32), E experts; pair p = (token p / top, choice p % top).  out: the mixtures' arrays one after the other, each
+// sorted_pair [max_tiles MOE_TM], pair_row [T top], tile_expert [max_tiles], every array rounded up to four ints.
+struct MoeTable { const int* table; int E, top; };
+__device__ __forceinline__ int moe_up4(int n) { return (n + 3) & ~3; }
+__global__ __launch_bounds__(1024) void moe_align_tables_kernel(int* __restrict__ out, const MoeTable* __restrict__ tables,
+                                                                const int* __restrict__ ids, int T, int V) {
+    size_t off = 0;
+    int P = 0, max_tiles = 0;
+    for (int l = 0; l <= (int)blockIdx.x; ++l) {
+        if (l) off += moe_up4(max_tiles * MOE_TM) + moe_up4(P) + moe_up4(max_tiles);
+        P = T * tables[l].top;
+        max_tiles = P / MOE_TM + min(tables[l].E, P);
+    }
+    const MoeTable tb = tables[blockIdx.x];
+    int* sorted_pair = out + off;
+    int* pair_row = sorted_pair + moe_up4(max_tiles * MOE_TM);
+    int* tile_expert = pair_row + moe_up4(P);
+    const int top = tb.top;
+    const int* table = tb.table;
+    moe_align_block(sorted_pair, pair_row, tile_expert, [=](int p) {
+        const int t = p / top, id = ids[t];
+        return id >= 0 && id < V ? table[(size_t)id * top + (p - t * top)] : -1;
+    }, P, tb.E, max_tiles);
+}
+
+// tables: MoeTable [n] on the device; max_experts, max_top: the largest E and top among them (the caller's account of what the
+// device array holds).
+extern "C" int spy_moe_align_tables(int* out, int64_t out_ints, const void* tables, int n, int max_experts, int max_top, const int* ids,
+                                    int T, int V, hipStream_t st) {
+    SPY_REQUIRE(n > 0 && n <= 65535 && T > 0 && V > 0 && max_experts > 0 && max_experts <= MOE_MAX_EXPERTS && max_top > 0,
+                "spy_moe_align_tables: %d tables of up to %d experts (1..%d)", n, max_experts, MOE_MAX_EXPERTS);
+    SPY_REQUIRE((int64_t)T * max_top <= (1 << 26), "spy_moe_align_tables: too many (token, choice) pairs");
+    SPY_REQUIRE(out && out_ints > 0 && ((uintptr_t)tables % 8) == 0, "spy_moe_align_tables: no output");
+    moe_align_tables_kernel<<<n, 1024, 0, st>>>(out, (const MoeTable*)tables, ids, T, V);
+    SPY_CHECK_LAUNCH("spy_moe_align_tables");
+    return 0;
 }
 
 extern "C" int spy_moe_align(int* sorted_pair, int* pair_row, int* tile_expert, const int* ids, int P, int E, int max_tiles,
@@ -551,11 +598,11 @@ extern "C" int spy_moe_gemm(void* C, int c_dtype, const void* A, int a_dtype, co
     return 0;
 }
 
-// out[t, :] = sum_k weights[t, k] * Y[pair_row[t top + k], :], added in ascending k (no weights: all one); add != null:
+// out[t, :] = scale * sum_k weights[t, k] * Y[pair_row[t top + k], :], added in ascending k (no weights: all one); add != null:
 // plus add[t, :], the result of a layer that every token uses, in the same pass
 template <typename TC, bool VEC>
 __global__ void moe_combine_kernel(TC* __restrict__ out, const float* __restrict__ Y, const float* __restrict__ weights,
-                                   const int* __restrict__ pair_row, int top, int H, const TC* __restrict__ add) {
+                                   const int* __restrict__ pair_row, int top, int H, const TC* __restrict__ add, float scale) {
     // a block has one token and a run of columns (blockIdx.y): few tokens still spread over the device.  VEC: a thread has
     // four neighbouring columns (H % 4 == 0 and 16-byte aligned rows, checked by the launcher), else one.
     constexpr int N = VEC ? 4 : 1;
@@ -566,7 +613,7 @@ __global__ void moe_combine_kernel(TC* __restrict__ out, const float* __restrict
     for (int k = 0; k < top; ++k) {
         const int row = pair_row[(size_t)t * top + k];
         if (row < 0) continue;
-        const float w = weights ? weights[(size_t)t * top + k] : 1.f;
+        const float w = (weights ? weights[(size_t)t * top + k] : 1.f) * scale;
         float y[N];
         if (VEC) Vec4<float>::load(Y + (size_t)row * H + c, y); else y[0] = Y[(size_t)row * H + c];
 #pragma unroll
@@ -582,16 +629,16 @@ __global__ void moe_combine_kernel(TC* __restrict__ out, const float* __restrict
 }
 
 extern "C" int spy_moe_combine(void* out, int dtype, const float* Y, const float* weights, const int* pair_row, int T, int top, int H,
-                               const void* add, hipStream_t st) {
+                               const void* add, float scale, hipStream_t st) {
     SPY_REQUIRE(T > 0 && top > 0 && H > 0, "spy_moe_combine: empty operand");
     const bool vec = H % 4 == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)Y % 16) == 0 && ((uintptr_t)add % 16) == 0;
     const int per_block = vec ? 512 : 128;
     const dim3 grid(T, (H + per_block - 1) / per_block);
     SPY_REQUIRE(grid.y <= 65535, "spy_moe_combine: rows of %d values are too long", H);
     if (vec) {
-        SPY_DISPATCH(dtype, TC, (moe_combine_kernel<TC, true><<<grid, 128, 0, st>>>((TC*)out, Y, weights, pair_row, top, H, (const TC*)add)));
+        SPY_DISPATCH(dtype, TC, (moe_combine_kernel<TC, true><<<grid, 128, 0, st>>>((TC*)out, Y, weights, pair_row, top, H, (const TC*)add, scale)));
     } else {
-        SPY_DISPATCH(dtype, TC, (moe_combine_kernel<TC, false><<<grid, 128, 0, st>>>((TC*)out, Y, weights, pair_row, top, H, (const TC*)add)));
+        SPY_DISPATCH(dtype, TC, (moe_combine_kernel<TC, false><<<grid, 128, 0, st>>>((TC*)out, Y, weights, pair_row, top, H, (const TC*)add, scale)));
     }
     SPY_CHECK_LAUNCH("spy_moe_combine");
     return 0;

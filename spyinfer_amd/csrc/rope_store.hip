@@ -16,7 +16,10 @@ template <typename TA, typename TW>
 __global__ __launch_bounds__(RS_WAVES * 64) void bias_rope_store_kernel(
     const TA* __restrict__ x, long long xs, TA* __restrict__ q_out, int n_q, int n_kv, int d, const TW* __restrict__ bias,
     const float* __restrict__ freq, int rot, const int* __restrict__ positions, TA* __restrict__ kc, TA* __restrict__ vc, int P,
-    int num_pages, const int* __restrict__ slots, float mag, float v_eps, int v_n, float qt_coef, int qt_every) {
+    int num_pages, const int* __restrict__ slots, float mag, float v_eps, int v_n, float qt_coef, int qt_every,
+    const TA* __restrict__ v1, long long v1s, int v1d, float lam, int dv) {
+    // v1 != null: values of another layer for the same tokens (head hv's at v1 + t v1s + hv v1d, dv of them); what is stored
+    // is (1 - lam) v + lam v1 (float32, rounded once).
     // qt_every > 0: a query is multiplied by 1 + qt_coef ln(floor((position + 1) / qt_every) + 1), float32 (queries that grow
     // with the logarithm of the position, in steps of qt_every positions)
     const int t = blockIdx.x, lane = threadIdx.x & 63;
@@ -47,7 +50,12 @@ __global__ __launch_bounds__(RS_WAVES * 64) void bias_rope_store_kernel(
             }
             r = 1.0f / sqrtf(wave_sum(ss) / (float)v_n + v_eps);
         }
-        for (int j = lane; j < d; j += 64) dst[(size_t)j * P] = from_f32<TA>((to_f32<TA>(row[j]) + (b ? to_f32<TW>(b[j]) : 0.f)) * r);
+        const TA* other = v1 ? v1 + (size_t)t * v1s + (size_t)hv * v1d : nullptr;
+        for (int j = lane; j < d; j += 64) {
+            float v = (to_f32<TA>(row[j]) + (b ? to_f32<TW>(b[j]) : 0.f)) * r;
+            if (other && j < dv) v = (1.0f - lam) * v + lam * to_f32<TA>(other[j]);
+            dst[(size_t)j * P] = from_f32<TA>(v);
+        }
         return;
     }
     const int half = rot >> 1;
@@ -68,17 +76,18 @@ __global__ __launch_bounds__(RS_WAVES * 64) void bias_rope_store_kernel(
 extern "C" int spy_bias_rope_store(const void* x, long long xs, int dtype, void* q_out, int T, int n_q, int n_kv, int d,
                                    const void* bias, int b_dtype, const float* freq, int rot, const int* positions, void* kc,
                                    void* vc, int P, int num_pages, const int* slots, float mag, float v_eps, int v_n, float qt_coef, int qt_every,
-                                   hipStream_t st) {
+                                   const void* v1, long long v1s, int v1d, float lam, int dv, hipStream_t st) {
     SPY_REQUIRE(T > 0 && n_q > 0 && n_kv > 0 && d > 0 && xs >= (long long)(n_q + 2 * n_kv) * d, "spy_bias_rope_store: bad sizes");
     SPY_REQUIRE(d <= RS_MAX_D, "spy_bias_rope_store: head size %d exceeds the supported %d", d, RS_MAX_D);
     SPY_REQUIRE(rot >= 0 && rot <= d && rot % 2 == 0 && (rot == 0 || freq), "spy_bias_rope_store: %d rotated dims do not fit a head of %d", rot, d);
     SPY_REQUIRE(!slots || (kc && vc && P > 0 && num_pages > 0), "spy_bias_rope_store: slots without a cache");
     SPY_REQUIRE(n_q + 2 * n_kv <= 65535 * RS_WAVES, "spy_bias_rope_store: too many heads");
     SPY_REQUIRE(v_n >= 0 && v_n <= d, "spy_bias_rope_store: a value norm over %d of %d values", v_n, d);
+    SPY_REQUIRE(!v1 || (dv > 0 && dv <= d && v1d >= dv && v1s >= (long long)(n_kv - 1) * v1d + dv), "spy_bias_rope_store: the other layer's values do not fit");
     const dim3 grid(T, (n_q + 2 * n_kv + RS_WAVES - 1) / RS_WAVES);
     SPY_DISPATCH(dtype, TA, SPY_DISPATCH(b_dtype, TW, (bias_rope_store_kernel<TA, TW><<<grid, RS_WAVES * 64, 0, st>>>(
         (const TA*)x, xs, (TA*)q_out, n_q, n_kv, d, (const TW*)bias, freq, rot, positions, (TA*)kc, (TA*)vc, P, num_pages, slots, mag, v_eps, v_n,
-        qt_coef, qt_every))));
+        qt_coef, qt_every, (const TA*)v1, v1s, v1d, lam, dv))));
     SPY_CHECK_LAUNCH("spy_bias_rope_store");
     return 0;
 }

@@ -79,7 +79,7 @@ class _Hip:
                      "spy_gemm_strided", "spy_latent_attention", "spy_latent_attention_mfma", "spy_latent_attention_mfma_workspace", "spy_head_products",
                      "spy_bias_rope_store", "spy_sigmoid_gate", "spy_mlstm", "spy_causal_conv_silu", "spy_delta_rule", "spy_moe_route",
                      "spy_moe_align", "spy_moe_gemm", "spy_moe_combine", "spy_moe_tile_rows", "spy_token_shift", "spy_tanh", "spy_time_mix",
-                     "spy_norm_pair_mean", "spy_scale_cap"):
+                     "spy_norm_pair_mean", "spy_scale_cap", "spy_result_norm", "spy_moe_align_tables"):
             if not hasattr(self.lib, name):
                 raise KernelError("the kernel library %s lacks %s: it is older than its sources; build it again "
                                   "(spyinfer_amd.kernels.build.build())" % (self.lib._name, name))
@@ -87,7 +87,7 @@ class _Hip:
         # the entry point that a step calls most: with its argument types declared, plain numbers go in as they are (no
         # ctypes object per argument: 3 us of the host's 14 per call)
         P, I = ctypes.c_void_p, ctypes.c_int
-        self.lib.spy_gemm_decode.argtypes = [P, I, P, I, ctypes.c_float, P, I, P, I, P, P, P, P, I, I, I, I, I, P, ctypes.c_int64, P]
+        self.lib.spy_gemm_decode.argtypes = [P, I, P, I, ctypes.c_float, P, I, P, I, P, P, P, P, I, I, I, I, I, I, P, ctypes.c_int64, P]
 
     def call(self, name, *args):
         rc = getattr(self.lib, name)(*args)
@@ -123,16 +123,21 @@ def library_path() -> str:
 
 
 # --------------------------------------------------------------------------
-def embedding(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
-    """out[t, :] = table[ids[t], :] * scale widened to float32 (the start of the residual stream)."""
-    _dev(ids, table)
+def embedding(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, norm=None) -> torch.Tensor:
+    """out[t, :] = table[ids[t], :] * scale widened to float32 (the start of the residual stream).  ``norm`` = (weight
+    float32 [H], eps): every row is then divided by its root mean square and multiplied by the weight, in float32."""
+    norm_w, norm_eps = norm if norm is not None else (None, 0.0)
+    _dev(ids, table, norm_w)
+    _check(norm_w is None or (norm_w.dtype == torch.float32 and table.dim() == 2 and norm_w.shape == (table.shape[1],)),
+           "embedding: the norm's weight must be float32 [H]")
     _check(ids.dtype == torch.int32 and ids.dim() == 1, "embedding: ids must be int32 [T]")
     _check(table.dim() == 2, "embedding: table must be [V, H]")
     T, (V, H) = ids.shape[0], table.shape
     out = torch.empty((T, H), dtype=torch.float32, device=table.device)
     if T:
         hip().call("spy_embedding", _ptr(out), _ptr(table), _code(table, "embedding table"), _ptr(ids),
-                   ctypes.c_int(T), ctypes.c_int(H), ctypes.c_int(V), ctypes.c_float(scale), _Hip.stream())
+                   ctypes.c_int(T), ctypes.c_int(H), ctypes.c_int(V), ctypes.c_float(scale), _ptr(norm_w), ctypes.c_float(norm_eps),
+                   _Hip.stream())
     return out
 
 
@@ -179,6 +184,34 @@ def add_rms_norm(resid: torch.Tensor, delta: Optional[torch.Tensor], weight: tor
                    ctypes.c_int(T), ctypes.c_int(H), ctypes.c_int(groups), _ptr(g_rows), _ptr(g_bias), ctypes.c_float(g_mult),
                    _ptr(base), _ptr(vec), _ptr(weight2), _ptr(out2), _Hip.stream())
     return out if weight2 is None else (out, out2)
+
+
+def result_norm(resid: torch.Tensor, y, result_weight: torch.Tensor, result_eps: float, weight: torch.Tensor, eps: float,
+                out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """resid += y / sqrt(mean(y^2) + result_eps) * result_weight (float32, in place; ``result_weight`` float32 [H]), then the
+    RMS norm of the sum in ``out_dtype``, both in one pass.  ``y``: rows [T, H] of the activation dtype, or ``ExpertRows`` (a
+    mixture's unsummed rows: they are summed here).  ``rows`` (int32 [R]): only those rows -> [R, H]; resid stays as it is."""
+    experts = y if isinstance(y, ExpertRows) else None
+    plain = None if experts is not None else y
+    _dev(resid, plain, result_weight, weight, rows)
+    _check(resid.dtype == torch.float32 and resid.dim() == 2, "result_norm: the residual stream must be float32 [T, H]")
+    T, H = resid.shape
+    _check(result_weight.dtype == torch.float32 and result_weight.shape == (H,) and weight.shape == (H,), "result_norm: weights must be [H], the result's float32")
+    if experts is not None:
+        _check(experts.shape == (T, H) and experts.dtype == out_dtype, "result_norm: the experts' rows must be those of the step's tokens")
+        _dev(experts.y, experts.pair_row, experts.weights, experts.add)
+    else:
+        _check(y.shape == (T, H) and y.dtype == out_dtype, "result_norm: the result must be [T, H] of the activation dtype")
+    _check(rows is None or (rows.dtype == torch.int32 and rows.dim() == 1), "result_norm: rows must be int32 [R]")
+    n_out = T if rows is None else rows.shape[0]
+    out = torch.empty((n_out, H), dtype=out_dtype, device=resid.device)
+    if n_out:
+        ex = (experts.y, experts.pair_row, experts.weights, experts.add, experts.top, experts.scale) if experts is not None else (None, None, None, None, 0, 1.0)
+        hip().call("spy_result_norm", _ptr(resid), _ptr(plain), _code(out, "norm output"), _ptr(ex[0]), _ptr(ex[1]), _ptr(ex[2]), _ptr(ex[3]),
+                   ctypes.c_int(ex[4]), ctypes.c_float(ex[5]), _ptr(result_weight), ctypes.c_float(result_eps), _ptr(weight),
+                   _code(weight, "norm weight"), ctypes.c_float(eps), _ptr(out), _ptr(rows), ctypes.c_int(n_out), ctypes.c_int(T), ctypes.c_int(H),
+                   _Hip.stream())
+    return out
 
 
 def rms_norm(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
@@ -377,10 +410,15 @@ def linear_few(x: torch.Tensor, w: torch.Tensor, tiled: Optional[torch.Tensor] =
     return linear(x, w, out_dtype, tiled=tiled, out=out)
 
 
-def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, tiled: Optional[torch.Tensor] = None, few_rows: int = 0) -> torch.Tensor:
-    """silu(x . Wgate^T) * (x . Wup^T) with ``w_gate_up [2 I, K]`` = [Wgate | Wup] -> [M, I].  For few bfloat16 rows
-    (decode) one kernel does both products and the SwiGLU; otherwise it is linear() followed by swiglu().  ``few_rows``:
-    most rows that the tiled kernel takes here (0: SKINNY_MAX_ROWS)."""
+#: activations of a gated feed-forward: "silu", or the tanh form of gelu, z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
+GATED_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+
+
+def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, tiled: Optional[torch.Tensor] = None, few_rows: int = 0,
+                  activation: str = "silu") -> torch.Tensor:
+    """act(x . Wgate^T) * (x . Wup^T) with ``w_gate_up [2 I, K]`` = [Wgate | Wup] -> [M, I].  For few bfloat16 rows
+    (decode) one kernel does both products and the activation; otherwise it is linear() followed by swiglu().  ``few_rows``:
+    most rows that the tiled kernel takes here (0: SKINNY_MAX_ROWS).  ``activation``: one of GATED_ACTIVATIONS."""
     _dev(x, w_gate_up)
     _check(x.dim() == 2 and w_gate_up.dim() == 2 and x.shape[1] == w_gate_up.shape[1] and w_gate_up.shape[0] % 2 == 0,
            "linear_swiglu: x [M, K] and w [2 I, K] expected")
@@ -388,14 +426,14 @@ def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, tiled: Optional[torc
     I = w_gate_up.shape[0] // 2
     if x.dtype == torch.bfloat16 and tiled is not None and 0 < M <= max(SKINNY_MAX_ROWS, few_rows) and I % 16 == 0 and x.is_contiguous():
         _check(tiled.shape == w_gate_up.shape, "linear_swiglu: the tiled copy does not fit")
-        return decode_linear_swiglu(x, tiled)
+        return decode_linear_swiglu(x, tiled, activation=activation)
     if x.dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16 and 0 < M <= SKINNY_MAX_ROWS and K % 8 == 0 \
             and (I + 16) * K * 2 < (1 << 32):
         out = torch.empty((M, I), dtype=x.dtype, device=x.device)
         hip().call("spy_gemm_skinny_swiglu", _ptr(x), _ptr(w_gate_up), _ptr(out), _code(out, "out"), ctypes.c_int(M),
-                   ctypes.c_int(I), ctypes.c_int(K), _Hip.stream())
+                   ctypes.c_int(I), ctypes.c_int(K), ctypes.c_int(GATED_ACTIVATIONS[activation]), _Hip.stream())
         return out
-    return swiglu(linear(x, w_gate_up))
+    return swiglu(linear(x, w_gate_up), activation)
 
 
 # --------------------------------------------------------------------------
@@ -444,6 +482,21 @@ class GatedAddend:
         return sigmoid_gate(self.y, self.gate, self.bias, self.mult)
 
 
+class NormedAddend:
+    """A sublayer's result that is normed before it meets the stream: the addend is ``y / rms(y) * weight`` (``weight``
+    float32 [H]).  The norm that sums it into the stream forms it in the same pass (``result_norm``); whoever cannot calls
+    ``resolve``.  ``y``: rows of the activation dtype, or ``ExpertRows``."""
+    __slots__ = ("y", "weight", "eps")
+
+    def __init__(self, y, weight, eps):
+        self.y, self.weight, self.eps = y, weight, float(eps)
+
+    def resolve(self):
+        """The addend as float32 rows."""
+        y = self.y.combine() if isinstance(self.y, ExpertRows) else self.y
+        return norm_residual(torch.zeros(y.shape, dtype=torch.float32, device=y.device), y, self.weight, self.eps)[0]
+
+
 class EntryAddends:
     """What meets the stream where a walk over a run of layers begins: whatever the block before left pending (None, an
     addend, a pair of addends), an earlier state of the stream (``base``, float32 [T, H], or None) and a vector that
@@ -459,7 +512,7 @@ class EntryAddends:
         pend = None if isinstance(self.pending, ScaledInput) else self.pending
         for addend in (pend if isinstance(pend, (tuple, list)) else (pend,)):
             if addend is not None:
-                resid.add_((addend.resolve() if isinstance(addend, GatedAddend) else addend).float())
+                resid.add_((addend.resolve() if isinstance(addend, (GatedAddend, NormedAddend)) else addend).float())
         if self.base is not None:
             resid.add_(self.base)
         if self.vec is not None:
@@ -535,7 +588,7 @@ def workspace_counters_clean(device) -> bool:
     return ws is None or not bool(ws[:4 * ATTENTION_COUNTERS].any())
 
 
-def _gemm_decode(x, tiled: torch.Tensor, epi: int, n_out: int, out, resid, xw_out, w_next, ss_out) -> None:
+def _gemm_decode(x, tiled: torch.Tensor, epi: int, n_out: int, out, resid, xw_out, w_next, ss_out, act: int = 0) -> None:
     _check(tiled.dtype == torch.bfloat16 and tiled.dim() == 2, "decode product: the tiled matrix must be bfloat16 [N, K]")
     K = tiled.shape[1]
     if isinstance(x, ScaledInput):
@@ -568,7 +621,7 @@ def _gemm_decode(x, tiled: torch.Tensor, epi: int, n_out: int, out, resid, xw_ou
     at = lambda t: None if t is None else t.data_ptr()              # (argument types are declared: see _Hip)
     hip().call("spy_gemm_decode", at(xs), 0 if ss is None else 1, at(ss), 0 if ss is None else ss.shape[0], eps, at(tiled), epi,
                at(out_t), 0 if out_t is None else _code(out_t, "out"), at(resid), at(xw_t), at(w_next), at(ss_out), M, n_out, K,
-               1 if x_tiled else 0, 1 if out_tiled else 0, at(ws), 0 if ws is None else ws.numel(), _Hip.stream())
+               1 if x_tiled else 0, 1 if out_tiled else 0, act, at(ws), 0 if ws is None else ws.numel(), _Hip.stream())
 
 
 def _rows_of(x) -> int:
@@ -594,8 +647,8 @@ def decode_linear(x, tiled: torch.Tensor, out_dtype: torch.dtype = torch.bfloat1
     return out
 
 
-def decode_linear_swiglu(x, tiled_gate_up: torch.Tensor, for_product: bool = False):
-    """silu(x . Wgate^T) * (x . Wup^T) for at most 128 rows (beyond 64: a normed input in operand order only); ``tiled_gate_up [2 I, K]`` = tiles of [Wgate | Wup].
+def decode_linear_swiglu(x, tiled_gate_up: torch.Tensor, for_product: bool = False, activation: str = "silu"):
+    """act(x . Wgate^T) * (x . Wup^T) (GATED_ACTIVATIONS) for at most 128 rows (beyond 64: a normed input in operand order only); ``tiled_gate_up [2 I, K]`` = tiles of [Wgate | Wup].
     ``for_product``: the result goes into another decode product only, and may come as OperandRows."""
     _check(tiled_gate_up.shape[0] % 32 == 0, "decode_linear_swiglu: [2 I, K] with I a multiple of 16 expected")
     I = tiled_gate_up.shape[0] // 2
@@ -603,7 +656,7 @@ def decode_linear_swiglu(x, tiled_gate_up: torch.Tensor, for_product: bool = Fal
         out = OperandRows.empty(_rows_of(x), I, tiled_gate_up.device)
     else:
         out = torch.empty((_rows_of(x), I), dtype=torch.bfloat16, device=tiled_gate_up.device)
-    _gemm_decode(x, tiled_gate_up, 1, I, out, None, None, None, None)
+    _gemm_decode(x, tiled_gate_up, 1, I, out, None, None, None, None, GATED_ACTIVATIONS[activation])
     return out
 
 
@@ -801,13 +854,16 @@ def fused_attention_ok(dtype, meta: AttentionMeta, n_q: int, n_kv: int, d: int, 
 
 def paged_attention(q: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor, page_size: int, meta: AttentionMeta,
                     n_q: int, n_kv: int, d: int, scale: float, window: Optional[int], raw: Optional[RawQKV] = None,
-                    for_product: bool = False, softcap: float = 0.0, distance: Optional[torch.Tensor] = None, zero_sink: bool = False):
+                    for_product: bool = False, softcap: float = 0.0, distance: Optional[torch.Tensor] = None,
+                    sink: Optional[torch.Tensor] = None, chunk: Optional[int] = None, gate: Optional[torch.Tensor] = None):
     """Causal grouped-query attention of the step's query tokens over the paged cache
     (which already holds this step's keys and values, or gets them from ``raw`` in this call).  Query at position p
     reads keys max(0, p - window + 1) .. p.  Scores, softmax and the weighted sum are float32.  ``softcap`` > 0: a
     score is softcap tanh(q . k scale / softcap).  ``distance``: float32 [2, n_q]: head h's (capped) score of a key that lies
-    x positions back is lowered by distance[0, h] ln(1 + distance[1, h] x).  ``zero_sink``: the softmax's denominator
-    holds one more term, e^0, that has no value: p_j = e^(s_j) / (1 + sum e^(s_j)).
+    x positions back is lowered by distance[0, h] ln(1 + distance[1, h] x).  ``sink``: float32 [n_q]; the softmax's denominator
+    holds one more term, e^sink[h], that has no value: p_j = e^(s_j) / (e^sink[h] + sum e^(s_j)).  ``chunk``: the query at
+    position p reads keys p - p mod chunk .. p only (in place of a window).  ``gate``: rows [T, n_q d] of the activation dtype
+    (a view into a wider product may be given); the result is multiplied by sigmoid(gate).
     ``for_product``: the result goes into a decode product only and may come as OperandRows (it does for steps of at
     most 128 tokens, ``attention_hands_over_operand_rows``)."""
     T, S = meta.T, meta.S
@@ -844,8 +900,19 @@ def paged_attention(q: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: t
     _dev(distance)
     _check(distance is None or (distance.dtype == torch.float32 and tuple(distance.shape) == (2, n_q) and distance.is_contiguous()),
            "paged_attention: the distance penalty's numbers must be float32 [2, n_q]")
-    _check(raw is None or (distance is None and not zero_sink), "paged_attention: the raw product takes neither a distance penalty nor a sink")
-    extras = (_ptr(distance), ctypes.c_int(1 if zero_sink else 0))
+    chunk = int(chunk or 0)
+    _check(chunk >= 0 and not (chunk and win), "paged_attention: a window or chunks, not both")
+    _dev(sink)
+    _check(sink is None or (sink.dtype == torch.float32 and tuple(sink.shape) == (n_q,)), "paged_attention: the sinks must be float32 [n_q]")
+    _check(raw is None or (distance is None and sink is None and not chunk and gate is None),
+           "paged_attention: the raw product takes neither a distance penalty nor a sink, chunks or a gate")
+    gate_ld = 0
+    if gate is not None:
+        gate_ld = _row_view(gate, "paged_attention")
+        _check(tuple(gate.shape) == (T, n_q * d) and gate.dtype == q.dtype and gate.device == q.device, "paged_attention: gate rows [T, n_q d] like q expected")
+    extras = (_ptr(distance), _ptr(sink), ctypes.c_int(chunk), ctypes.c_void_p(0 if gate is None else gate.data_ptr()), ctypes.c_longlong(gate_ld))
+    # the most keys that a query of this step reads: what there is to split
+    max_keys = meta.max_kv_len if not chunk else min(meta.max_kv_len, chunk)
     out = q if raw is not None else torch.empty_like(q)
     if T == 0:
         return out
@@ -872,7 +939,7 @@ def paged_attention(q: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: t
             # few tiles with many keys (a late portion of a long prompt): their keys are split into parts as well
             bsplits = 1
             if n_big * n_kv < PREFILL_SPLIT_BELOW:
-                bsplits = max(1, min(PREFILL_SPLIT_BELOW * 2 // (n_big * n_kv), meta.max_kv_len // 256, 16))
+                bsplits = max(1, min(PREFILL_SPLIT_BELOW * 2 // (n_big * n_kv), max_keys // 256, 16))
             _check(meta.big_rows in (128, 256), "paged_attention: tiles of 128 or 256 rows expected")
             bws_floats = hip().lib.spy_attention_prefill_workspace(ctypes.c_int(n_big), ctypes.c_int(meta.big_rows), ctypes.c_int(n_kv),
                                                                    ctypes.c_int(d), ctypes.c_int(bsplits))
@@ -884,7 +951,7 @@ def paged_attention(q: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: t
             # Few 16-row tiles cannot fill the chip by themselves (decoding requests, short portions): their keys are
             # split into parts, each part a block of 4 waves that wants 128 keys at least, and a second kernel merges.
             want = max(1, DECODE_SPLIT_TARGET // max(1, n_small * n_kv))
-            splits = max(1, min(want, key_parts_for(meta.max_kv_len)))
+            splits = max(1, min(want, key_parts_for(max_keys)))
             # a step of single tokens whose keys the host has cut into pieces (decode_pieces): one block per record
             pieces = meta.pieces.get((n_kv, win, d)) if raw is not None and d <= 128 and n_small * n_kv <= ATTENTION_COUNTERS else None
             counters = decode_workspace(q.device) if splits > 1 or pieces is not None else None
@@ -923,15 +990,15 @@ def paged_attention(q: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: t
     return out
 
 
-def swiglu(gate_up: torch.Tensor) -> torch.Tensor:
-    """``gate_up [T, 2 I]`` = [gate | up]  ->  silu(gate) * up  [T, I], float32 arithmetic."""
+def swiglu(gate_up: torch.Tensor, activation: str = "silu") -> torch.Tensor:
+    """``gate_up [T, 2 I]`` = [gate | up]  ->  act(gate) * up  [T, I] (GATED_ACTIVATIONS), float32 arithmetic."""
     _dev(gate_up)
     _check(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "swiglu: [T, 2 I] expected")
     T, I = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((T, I), dtype=gate_up.dtype, device=gate_up.device)
     if T * I:
         hip().call("spy_swiglu", _ptr(gate_up), _ptr(out), _code(gate_up, "gate_up"), ctypes.c_int(T), ctypes.c_int(I),
-                   _Hip.stream())
+                   ctypes.c_int(GATED_ACTIVATIONS[activation]), _Hip.stream())
     return out
 
 
@@ -1234,19 +1301,27 @@ def _row_view(x: torch.Tensor, what: str) -> int:
 
 def bias_rope_store(x: torch.Tensor, n_q: int, n_kv: int, d: int, bias: Optional[torch.Tensor], freq: Optional[torch.Tensor],
                     rotary_dim: int, positions: torch.Tensor, k_cache, v_cache, page_size: int, slots: Optional[torch.Tensor],
-                    mag: float = 1.0, value_norm=None, query_temperature=None) -> torch.Tensor:
+                    mag: float = 1.0, value_norm=None, query_temperature=None, value_mix=None) -> torch.Tensor:
     """From rows ``x [T, >= (n_q + 2 n_kv) d]`` = [q heads | k heads | v heads] (a view into a wider product may be
     given): the biases ``bias [(n_q + 2 n_kv) d]`` added, the first ``rotary_dim`` dims of every q and k head rotated
     (pair (j, j + rotary_dim/2), angle float32(position) * freq[j]), q written to the result [T, n_q d], k and v into
     the cache pages at ``slots`` (skipped when None).  ``mag``: factor on cos and sin.  ``value_norm`` = (eps, n): every
     value head is divided by sqrt(mean of its first n values squared + eps) before it is stored.  ``query_temperature`` =
-    (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1), in float32."""
+    (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1), in float32.
+    ``value_mix`` = (other, head, n, lam): what is stored as a value is (1 - lam) v + lam v', v' the n values that ``other`` (rows
+    of another layer's values for the same tokens, ``head`` values from one head to the next) holds for the head."""
     xs = _row_view(x, "bias_rope_store")
     qt_coef, qt_every = (float(query_temperature[0]), int(query_temperature[1])) if query_temperature is not None else (0.0, 0)
     _check(query_temperature is None or qt_every > 0, "bias_rope_store: the query temperature's step must be positive")
     v_eps, v_n = (float(value_norm[0]), int(value_norm[1])) if value_norm is not None else (0.0, 0)
     _check(0 <= v_n <= d, "bias_rope_store: a value norm over %d of %d values", v_n, d)
     T = x.shape[0]
+    other, other_ld, other_head, mix_n, lam = None, 0, 0, 0, 0.0
+    if value_mix is not None:
+        other, other_head, mix_n, lam = value_mix[0], int(value_mix[1]), int(value_mix[2]), float(value_mix[3])
+        other_ld = _row_view(other, "bias_rope_store")
+        _check(other.dtype == x.dtype and other.device == x.device and other.shape[0] == T and 0 < mix_n <= min(d, other_head)
+               and other.shape[1] >= (n_kv - 1) * other_head + mix_n, "bias_rope_store: the other layer's values must be rows of the step's tokens")
     _dev(bias, freq, positions, k_cache, v_cache, slots)
     _check(x.shape[1] >= (n_q + 2 * n_kv) * d, "bias_rope_store: rows of %d values hold no %d heads of %d", x.shape[1], n_q + 2 * n_kv, d)
     _check(bias is None or bias.shape == ((n_q + 2 * n_kv) * d,), "bias_rope_store: one bias per projected value expected")
@@ -1266,7 +1341,9 @@ def bias_rope_store(x: torch.Tensor, n_q: int, n_kv: int, d: int, bias: Optional
                    ctypes.c_int(n_q), ctypes.c_int(n_kv), ctypes.c_int(d), _ptr(bias), _code(bias, "bias") if bias is not None else F32,
                    _ptr(freq), ctypes.c_int(rotary_dim), _ptr(positions), _ptr(k_cache if slots is not None else None),
                    _ptr(v_cache if slots is not None else None), ctypes.c_int(page_size), ctypes.c_int(num_pages), _ptr(slots),
-                   ctypes.c_float(mag), ctypes.c_float(v_eps), ctypes.c_int(v_n), ctypes.c_float(qt_coef), ctypes.c_int(qt_every), _Hip.stream())
+                   ctypes.c_float(mag), ctypes.c_float(v_eps), ctypes.c_int(v_n), ctypes.c_float(qt_coef), ctypes.c_int(qt_every),
+                   ctypes.c_void_p(0 if other is None else other.data_ptr()), ctypes.c_longlong(other_ld), ctypes.c_int(other_head),
+                   ctypes.c_float(lam), ctypes.c_int(mix_n), _Hip.stream())
     return q
 
 
@@ -1506,40 +1583,133 @@ def moe_route(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, gro
 MOE_MFMA = True            # False forces the plain float32 kernel for bfloat16 too (tests flip it; nothing else does)
 
 
-def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-                activation: str = "silu", limit: float = 0.0, weight_input: bool = False, add: Optional[torch.Tensor] = None) -> torch.Tensor:
+class MoEAlignment:
+    """A step's (token, choice) pairs of one mixture sorted by expert, on the device: ``sorted_pair`` [tiles * rows of a tile]
+    (the pair of a sorted row, -1: none), ``pair_row`` [T * top] (the row of a pair), ``tile_expert`` [tiles] (-1: no rows)."""
+    __slots__ = ("sorted_pair", "pair_row", "tile_expert", "T", "top", "experts")
+
+    def __init__(self, sorted_pair, pair_row, tile_expert, T, top, experts):
+        self.sorted_pair, self.pair_row, self.tile_expert = sorted_pair, pair_row, tile_expert
+        self.T, self.top, self.experts = T, top, experts
+
+
+def _align_sizes(T: int, top: int, experts: int):
+    """(sorted rows, pairs, tiles) of a mixture's alignment: they follow the numbers of tokens and choices alone."""
+    tm = hip().lib.spy_moe_tile_rows()
+    P = T * top
+    tiles = P // tm + min(experts, P)
+    return tiles * tm, P, tiles
+
+
+class ExpertTables:
+    """The mixtures of a model whose experts are named by tables of the token ids (int32 [V, top] each): with the ids all of
+    a step's choices are known, so ``align`` sorts the pairs of all of them in one launch."""
+
+    def __init__(self):
+        self.tables, self.experts = [], []
+        self._desc = None
+
+    def add(self, table: torch.Tensor, experts: int, number: Optional[int] = None) -> int:
+        """Takes a table up (in the place of table ``number``, if that is given); returns its number."""
+        _check(table.dtype == torch.int32 and table.dim() == 2 and table.is_contiguous(), "ExpertTables: an int32 table [V, top] expected")
+        _check(not self.tables or table.shape[0] == self.tables[0].shape[0], "ExpertTables: the tables must have one vocabulary")
+        self._desc = None
+        if number is not None:
+            self.tables[number], self.experts[number] = table, int(experts)
+            return number
+        self.tables.append(table)
+        self.experts.append(int(experts))
+        return len(self.tables) - 1
+
+    def prepare(self) -> None:
+        """The device's list of the tables: address, experts, choices (made ahead of any capture)."""
+        words = [w for t, e in zip(self.tables, self.experts) for w in (t.data_ptr(), e | (t.shape[1] << 32))]
+        self._desc = torch.tensor(words, dtype=torch.int64).to(self.tables[0].device)
+
+    def align(self, token_ids: torch.Tensor):
+        """[MoEAlignment] of the step's tokens, one per table, from one launch."""
+        _dev(token_ids, *self.tables)
+        _check(token_ids.dtype == torch.int32 and token_ids.dim() == 1 and token_ids.shape[0] > 0, "ExpertTables: token ids int32 [T] expected")
+        if self._desc is None:
+            self.prepare()
+        T = token_ids.shape[0]
+        up4 = lambda n: (n + 3) // 4 * 4
+        sizes = [_align_sizes(T, t.shape[1], e) for t, e in zip(self.tables, self.experts)]
+        buf = torch.empty((sum(up4(n) for s in sizes for n in s),), dtype=torch.int32, device=token_ids.device)
+        hip().call("spy_moe_align_tables", _ptr(buf), ctypes.c_int64(buf.shape[0]), _ptr(self._desc), ctypes.c_int(len(self.tables)),
+                   ctypes.c_int(max(self.experts)), ctypes.c_int(max(t.shape[1] for t in self.tables)), _ptr(token_ids), ctypes.c_int(T),
+                   ctypes.c_int(self.tables[0].shape[0]), _Hip.stream())
+        out, at = [], 0
+        for (rows, pairs, tiles), t, e in zip(sizes, self.tables, self.experts):
+            parts = []
+            for n in (rows, pairs, tiles):
+                parts.append(buf[at:at + n])
+                at += up4(n)
+            out.append(MoEAlignment(*parts, T, t.shape[1], e))
+        return out
+
+
+class ExpertRows:
+    """A mixture's result as its experts' unsummed rows: out[t] = add[t] + scale * sum_k weights[t, k] y[pair_row[t, k]] (no
+    weights: all one).  A kernel that reads the result next may sum it in its own pass (``result_norm``); ``combine`` makes
+    ordinary rows [T, H] of the activation dtype."""
+    __slots__ = ("y", "pair_row", "weights", "add", "top", "scale", "shape", "dtype")
+
+    def __init__(self, y, pair_row, weights, add, top, scale, T, dtype):
+        self.y, self.pair_row, self.weights, self.add, self.top, self.scale = y, pair_row, weights, add, top, float(scale)
+        self.shape, self.dtype = (T, y.shape[1]), dtype
+
+    def combine(self) -> torch.Tensor:
+        T, K = self.shape
+        out = torch.empty((T, K), dtype=self.dtype, device=self.y.device)
+        hip().call("spy_moe_combine", _ptr(out), _code(out, "out"), _ptr(self.y), _ptr(self.weights), _ptr(self.pair_row), ctypes.c_int(T),
+                   ctypes.c_int(self.top), ctypes.c_int(K), _ptr(self.add), ctypes.c_float(self.scale), _Hip.stream())
+        return out
+
+
+def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[torch.Tensor], w_gate_up: torch.Tensor, w_down: torch.Tensor,
+                activation: str = "silu", limit: float = 0.0, weight_input: bool = False, add: Optional[torch.Tensor] = None,
+                align: Optional[MoEAlignment] = None, scale: float = 1.0, unsummed: bool = False):
     """out[t] = sum_k weights[t, k] * down_e( silu(gate_e x[t]) * up_e x[t] ), e = ids[t, k]; ``w_gate_up [E, 2 F, K]`` =
     every expert's [gate rows | up rows], ``w_down [E, K, F]``.  The (token, choice) pairs are sorted by expert on the
     device and the experts' products run over the sorted rows; no size here depends on the choice.  ``activation``
     "clamped": g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) in place of silu(gate) up.
     ``weight_input``: the weight multiplies the expert's input, out[t] = sum_k expert_e(weights[t, k] x[t]) (the two
     products being linear, it is multiplied into their sums, ahead of the activation).  ``add [T, K]``: added to the result
-    in the pass that sums the choices (the result of a layer that every token uses)."""
+    in the pass that sums the choices (the result of a layer that every token uses).  ``align``: the pairs already sorted
+    (``ids`` is not read then, and ``weights`` may be None: all one).  ``scale``: a factor on the sum over the choices.
+    ``unsummed``: the result is ``ExpertRows`` instead of [T, K]."""
     _dev(add)
     _check(add is None or (add.shape == x.shape and add.dtype == x.dtype and add.is_contiguous()), "moe_experts: the addend must be like x")
     _check(activation in ("silu", "clamped") and (activation == "silu" or limit > 0.0), "moe_experts: activation silu, or clamped with a positive limit")
     act_kind = 1 if activation == "clamped" else 0
     _dev(x, ids, weights, w_gate_up, w_down)
     T, K = x.shape
-    top = ids.shape[1]
+    top = ids.shape[1] if align is None else align.top
     E, F2, _ = w_gate_up.shape
     F = F2 // 2
-    _check(x.dim() == 2 and ids.dtype == torch.int32 and ids.shape == (T, top) and weights.dtype == torch.float32 and weights.shape == (T, top),
+    _check(x.dim() == 2 and (align is not None or (ids.dtype == torch.int32 and ids.shape == (T, top) and weights is not None))
+           and (weights is None or (weights.dtype == torch.float32 and weights.shape == (T, top))),
            "moe_experts: experts int32 [T, top] and weights float32 [T, top] expected")
+    _check(align is None or (align.T == T and align.experts == E), "moe_experts: the alignment is of another step or mixture")
+    _check(weights is not None or not weight_input, "moe_experts: no weights for the experts' input")
     _check(w_gate_up.dim() == 3 and w_gate_up.shape == (E, 2 * F, K) and tuple(w_down.shape) == (E, K, F) and w_down.dtype == w_gate_up.dtype,
            "moe_experts: expert matrices [E, 2 F, K] and [E, K, F] of one dtype expected")
-    out = torch.empty((T, K), dtype=x.dtype, device=x.device)
     if not T:
-        return out
-    tm = hip().lib.spy_moe_tile_rows()
-    P = T * top
-    max_tiles = P // tm + min(E, P)
+        return torch.empty((T, K), dtype=x.dtype, device=x.device)
     dev = x.device
-    sorted_pair = torch.empty((max_tiles * tm,), dtype=torch.int32, device=dev)
-    pair_row = torch.empty((P,), dtype=torch.int32, device=dev)
-    tile_expert = torch.empty((max_tiles,), dtype=torch.int32, device=dev)
-    hip().call("spy_moe_align", _ptr(sorted_pair), _ptr(pair_row), _ptr(tile_expert), _ptr(ids), ctypes.c_int(P), ctypes.c_int(E),
-               ctypes.c_int(max_tiles), _Hip.stream())
+    rows, P, max_tiles = _align_sizes(T, top, E)
+    tm = rows // max_tiles
+    if align is None:
+        sorted_pair = torch.empty((rows,), dtype=torch.int32, device=dev)
+        pair_row = torch.empty((P,), dtype=torch.int32, device=dev)
+        tile_expert = torch.empty((max_tiles,), dtype=torch.int32, device=dev)
+        hip().call("spy_moe_align", _ptr(sorted_pair), _ptr(pair_row), _ptr(tile_expert), _ptr(ids), ctypes.c_int(P), ctypes.c_int(E),
+                   ctypes.c_int(max_tiles), _Hip.stream())
+    else:
+        sorted_pair, pair_row, tile_expert = align.sorted_pair, align.pair_row, align.tile_expert
+        _dev(sorted_pair, pair_row, tile_expert)
+        _check(sorted_pair.shape == (rows,) and pair_row.shape == (P,) and tile_expert.shape == (max_tiles,), "moe_experts: the alignment does not fit")
     # bfloat16: the matrix cores, a block taking one row tile of an expert when the experts have few rows (decoding:
     # blocks for the whole device), up to eight when they have many (an expert's matrices are read once per 128 rows)
     per_block = 0 if not MOE_MFMA or x.dtype != torch.bfloat16 or w_gate_up.dtype != torch.bfloat16 else (8 if P >= 16 * E else 1)
@@ -1551,9 +1721,8 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gat
     hip().call("spy_moe_gemm", _ptr(y), F32, _ptr(act), _code(act, "act"), _ptr(w_down), _code(w_down, "expert matrices"), _ptr(tile_expert),
                _ptr(sorted_pair), ctypes.c_int(0), ctypes.c_int(0), ctypes.c_int(max_tiles), ctypes.c_int(E), ctypes.c_int(K), ctypes.c_int(F),
                ctypes.c_int(per_block), ctypes.c_int(0), ctypes.c_float(0.0), _ptr(None), _Hip.stream())
-    hip().call("spy_moe_combine", _ptr(out), _code(out, "out"), _ptr(y), _ptr(None if weight_input else weights), _ptr(pair_row), ctypes.c_int(T), ctypes.c_int(top),
-               ctypes.c_int(K), _ptr(add), _Hip.stream())
-    return out
+    result = ExpertRows(y, pair_row, None if weight_input else weights, add, top, scale, T, x.dtype)
+    return result if unsummed else result.combine()
 
 
 # --------------------------------------------------------------------------

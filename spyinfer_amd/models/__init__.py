@@ -3,4 +3,5 @@ from . import sefevik  # registers "Sefevik"
 from . import sodedra  # registers "Sodedra"
 from . import meronex  # registers "Meronex"
 from . import tarunex  # registers "Tarunex"
+from . import balelorn  # registers "Balelorn"
 from .base import DecoderModel, LayerCall

@@ -7,7 +7,8 @@ of all tokens of the step written to their pages before any query reads
 through its request's block table with the causal mask ``key <= position``
 (:98-111), scale 1/sqrt(d) after the dot product (:59, :110), kv head
 ``h * n_kv / n_q`` (:96); output projection.  One meaning for whole prompts,
-portions and single tokens.  ``window`` keeps only the last ``window`` keys.
+portions and single tokens.  ``window`` keeps only the last ``window`` keys; ``chunk`` only those of the query's own chunk
+of that many positions, counted from the request's first token.
 
 Options beside the reference's arrangement: biases on the q, k and v projections; a value size other than the
 key size (the smaller of the two is padded with zero rows when the weights are bound, so that one head size runs
@@ -16,8 +17,9 @@ q, k and v; a rotation whose angles are formed in the kernel from the encoding's
 position limit: encodings with rescaled frequencies, with or without a factor on cos and sin); values divided by their
 root mean square per head before they are stored; scores capped by cap tanh(score / cap) after the scale; queries
 multiplied by a temperature that grows with the logarithm of the position; a penalty r1_h ln(1 + r2_h (i - j)) on the
-distance, taken off the (capped) score; a softmax whose denominator holds a one (a sink of score 0 without a value); the
-gate as one number per head instead of one per value.
+distance, taken off the (capped) score; a softmax whose denominator holds a one (a sink of score 0 without a value) or
+e^sink of a learned number per head; the gate as one number per head instead of one per value; values blended with those
+of an earlier layer of the same step before they are stored.
 """
 from __future__ import annotations
 
@@ -37,18 +39,24 @@ ROWS_PER_TILE = 16        # rows of (token, head-in-group) pairs in a small atte
 BIG_MIN_ROWS = 64         # entries with at least this many rows go to the prefill kernel
 
 
-def plan_attention_tiles(batch, group_size: int, big_rows: int = 0, key_parts: bool = True) -> None:
+def _tiles_name(group_size: int, big_rows: int, chunk: int) -> str:
+    return "%d_%d" % (group_size, big_rows) + ("_c%d" % chunk if chunk else "")
+
+
+def plan_attention_tiles(batch, group_size: int, big_rows: int = 0, key_parts: bool = True, chunk: int = 0) -> None:
     """Adds to the step's arrays the tiles over each entry's rows (token-major, head-in-group minor) for a query-head
     group of ``group_size``: entries with at least BIG_MIN_ROWS rows are cut into tiles of ``big_rows`` rows (the
     LDS-sharing prefill kernel; 0: never), the others into 16-row tiles (one block of waves each).  Once per step,
     group size and tile size.  ``key_parts``: the caller's launches take the number of key parts from the longest
-    request (False: its keys are cut another way, ``plan_decode_pieces``)."""
+    request (False: its keys are cut another way, ``plan_decode_pieces``).  ``chunk``: the layers read inside chunks of that
+    many positions, which the order of the large tiles goes by (0: no chunks)."""
     if key_parts:
         # the 16-row tiles' keys are split into a number of parts that follows the longest request: a launch shape
         batch.add_graph_key("attention_key_parts", ops.key_parts_for(batch.max_kv_len))
-    note = ("attention_tiles", group_size, big_rows)
+    note = ("attention_tiles", group_size, big_rows, chunk)
     if note in batch.shared:
         return
+    name = _tiles_name(group_size, big_rows, chunk)
     S, lens = batch.S, batch.lens
     rows = lens.astype(np.int64) * group_size
     big = (rows >= BIG_MIN_ROWS) & bool(big_rows)
@@ -63,11 +71,14 @@ def plan_attention_tiles(batch, group_size: int, big_rows: int = 0, key_parts: b
             # the prefill kernel gives a block the tiles b and n - 1 - b: sorted by the keys they read, blocks are even
             pos0 = batch.host_array("pos0")[tile_entry].astype(np.int64)
             last_tok = np.minimum(lens[tile_entry].astype(np.int64), (tile_row0.astype(np.int64) + size + group_size - 1) // group_size)
-            order = np.argsort(-(pos0 + last_tok), kind="stable")
+            keys = pos0 + last_tok
+            if chunk:
+                keys -= (pos0 + tile_row0 // group_size) // chunk * chunk        # the tile's first row has its first key
+            order = np.argsort(-keys, kind="stable")
             tile_entry, tile_row0 = tile_entry[order], tile_row0[order]
         counts[kind] = int(first[-1])
-        batch.add_array("tile_entry_%s_%d_%d" % (kind, group_size, big_rows), tile_entry)
-        batch.add_array("tile_row0_%s_%d_%d" % (kind, group_size, big_rows), tile_row0)
+        batch.add_array("tile_entry_%s_%s" % (kind, name), tile_entry)
+        batch.add_array("tile_row0_%s_%s" % (kind, name), tile_row0)
     batch.shared[note] = counts
 
 
@@ -81,17 +92,17 @@ def plan_decode_pieces(batch, n_kv: int, window: int, head_dim: int) -> None:
         batch.shared[note] = True
 
 
-def attention_meta(batch, group: int, group_size: int, big_rows: int = 0) -> ops.AttentionMeta:
+def attention_meta(batch, group: int, group_size: int, big_rows: int = 0, chunk: int = 0) -> ops.AttentionMeta:
     """The step's description for the attention kernels, from the batch's arrays on the device (one object per step,
-    cache group, group size and tile size)."""
-    note = ("attention_meta", group, group_size, big_rows)
+    cache group, group size, tile size and chunk length)."""
+    note = ("attention_meta", group, group_size, big_rows, chunk)
     meta = batch.shared.get(note)
     if meta is None:
         tiles = None
-        counts = batch.shared.get(("attention_tiles", group_size, big_rows))
+        counts = batch.shared.get(("attention_tiles", group_size, big_rows, chunk))
         if counts is not None:
-            tiles = {kind: (batch.array("tile_entry_%s_%d_%d" % (kind, group_size, big_rows)),
-                            batch.array("tile_row0_%s_%d_%d" % (kind, group_size, big_rows)), n) for kind, n in counts.items()}
+            name = _tiles_name(group_size, big_rows, chunk)
+            tiles = {kind: (batch.array("tile_entry_%s_%s" % (kind, name)), batch.array("tile_row0_%s_%s" % (kind, name)), n) for kind, n in counts.items()}
         pieces = {key[1:]: batch.array("decode_pieces_%d_%d_%d" % key[1:]).view(-1, key_pieces.PIECE_RECORD)
                   for key in batch.shared if isinstance(key, tuple) and key[0] == "decode_pieces"}
         meta = ops.AttentionMeta(batch.array("cu_q"), batch.array("pos0"), batch.array("kv_len"), batch.block_table(group),
@@ -108,7 +119,7 @@ class PagedAttention(Mixer):
                  window: Optional[int] = None, scale: Optional[float] = None, fold_rows: Optional[int] = None,
                  value_dim: Optional[int] = None, bias: bool = False, gate: bool = False, names: Optional[dict] = None,
                  softcap: float = 0.0, value_norm_eps: Optional[float] = None, query_temperature=None, distance_penalty: bool = False,
-                 zero_sink: bool = False):
+                 zero_sink: bool = False, chunk: Optional[int] = None, sink: bool = False, value_mix: Optional[str] = None):
         """``fold_rows``: most rows of a step whose products here run with the norms and the residual sum folded in
         (None: ``ops.default_fold_rows`` of this part's matrices).  ``value_dim``: size of a value head (None: ``head_dim``).
         ``bias``: q, k and v have biases.  ``gate``: the heads' results are multiplied by sigmoid(Wg x) before the output
@@ -118,7 +129,12 @@ class PagedAttention(Mixer):
         gate is one number per head (a matrix [heads, hidden]) instead of one per value.  ``query_temperature`` = (coef,
         every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).  ``distance_penalty``:
         two numbers per head (tensors ``r1``, ``r2`` [heads]); the score of a key x positions back is lowered by
-        r1 ln(1 + r2 x), after the cap.  ``zero_sink``: p_j = e^(s_j) / (1 + sum e^(s_j))."""
+        r1 ln(1 + r2 x), after the cap.  ``zero_sink``: p_j = e^(s_j) / (1 + sum e^(s_j)).  ``chunk`` (in place of a window): the
+        query at position p reads the keys of its own chunk only, from p - p mod chunk on.  ``sink``: a learned number per
+        head (tensor ``sink`` [heads]), p_j = e^(s_j) / (e^sink + sum e^(s_j)).  ``value_mix``: what is cached as values is
+        (1 - lam) v + lam v_first, lam one learned number (tensor ``vmix`` without dimensions) and v_first the same tokens'
+        values in the layer that says "first" (it caches its own; its tensor, if stored, is not read); the others, which run
+        later in the step and must have as many value heads of the same size, say "blend"."""
         if num_heads % num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
         self.hidden_size, self.num_heads, self.num_kv_heads = hidden_size, num_heads, num_kv_heads
@@ -130,8 +146,14 @@ class PagedAttention(Mixer):
         self.query_temperature = None if query_temperature is None else (float(query_temperature[0]), int(query_temperature[1]))
         self.has_distance, self.zero_sink = bool(distance_penalty), bool(zero_sink)
         self.distance = None
+        if chunk is not None and window is not None:
+            raise ValueError("a window or chunks, not both")
+        if value_mix not in (None, "first", "blend") or (zero_sink and sink):
+            raise ValueError("value_mix %r is not known, or two kinds of sink" % (value_mix,))
+        self.chunk, self.has_sink, self.value_mix = (None if chunk is None else int(chunk)), bool(sink), value_mix
+        self.sink, self.mix_lambda = None, 0.0
         self.names = dict(q=".q_proj.weight", k=".k_proj.weight", v=".v_proj.weight", o=".o_proj.weight", g=".g_proj.weight",
-                          q_norm=".q_norm.weight", k_norm=".k_norm.weight", bias=".bias", r1=".r1", r2=".r2")
+                          q_norm=".q_norm.weight", k_norm=".k_norm.weight", bias=".bias", r1=".r1", r2=".r2", sink=".sink", vmix=".vmix")
         self.names.update(names or {})
         self.b_qkv = None
         self.position = position
@@ -155,6 +177,10 @@ class PagedAttention(Mixer):
             specs.append(WeightSpec(prefix + n["g"], (nq if self.gate_per_head else nq * dv, H)))
         if self.has_distance:
             specs += [WeightSpec(prefix + n["r1"], (nq,), "bias"), WeightSpec(prefix + n["r2"], (nq,), "norm")]
+        if self.has_sink:
+            specs.append(WeightSpec(prefix + n["sink"], (nq,), "bias"))
+        if self.value_mix is not None:
+            specs.append(WeightSpec(prefix + n["vmix"], (), "bias", optional=self.value_mix == "first"))
         if self.qk_norm_eps is not None:
             specs += [WeightSpec(prefix + n["q_norm"], (dk,), "norm"), WeightSpec(prefix + n["k_norm"], (dk,), "norm")]
         return specs
@@ -198,6 +224,13 @@ class PagedAttention(Mixer):
         if self.has_distance:
             # the penalty's numbers enter the scores, which are float32: [2, heads]
             self.distance = torch.stack([weights[prefix + n["r1"]].float(), weights[prefix + n["r2"]].float()]).contiguous()
+        # the sinks enter the softmax, which is float32: [heads] (a zero sink is a sink of score 0)
+        if self.has_sink:
+            self.sink = weights[prefix + n["sink"]].float().contiguous()
+        elif self.zero_sink:
+            self.sink = torch.zeros((nq,), dtype=torch.float32, device=self.w_o.device)
+        if self.value_mix == "blend":
+            self.mix_lambda = float(weights[prefix + n["vmix"]])
         if self.qk_norm_eps is not None:
             if dk != self.head_dim:
                 raise ValueError("per-head norms of q and k with a value size other than the key size are not implemented")
@@ -209,18 +242,20 @@ class PagedAttention(Mixer):
 
     # ---- cache -----------------------------------------------------------
     def cache_spec(self):
-        return PagedKV(self.num_kv_heads, self.head_dim, self.window)
+        return PagedKV(self.num_kv_heads, self.head_dim, self.window, self.chunk)
 
     def plan(self, batch) -> None:
         # a step of single tokens that the fused kernel will take has its keys cut into even pieces on the host
         pieces = ops.decode_pieces_ok(batch.S, batch.T, batch.act_dtype, self.num_kv_heads, self.head_dim) and self._rotated_whole()
-        plan_attention_tiles(batch, self.num_heads // self.num_kv_heads, self._big_rows(batch, batch.page_size), key_parts=not pieces)
+        plan_attention_tiles(batch, self.num_heads // self.num_kv_heads, self._big_rows(batch, batch.page_size), key_parts=not pieces,
+                             chunk=self.chunk or 0)
         if pieces:
             plan_decode_pieces(batch, self.num_kv_heads, int(self.window or 0), self.head_dim)
 
     def plan_arrays(self, entries):
         G = self.num_heads // self.num_kv_heads
-        out = {"tile_entry_small_%d" % G: entries, "tile_row0_small_%d" % G: entries}
+        name = _tiles_name(G, 0, self.chunk or 0)
+        out = {"tile_entry_small_%s" % name: entries, "tile_row0_small_%s" % name: entries}
         if ops.decode_pieces_ok(entries, entries, torch.bfloat16, self.num_kv_heads, self.head_dim):
             out["decode_pieces_%d_%d_%d" % (self.num_kv_heads, int(self.window or 0), self.head_dim)] = \
                 key_pieces.decode_pieces_capacity(entries, self.num_kv_heads) * key_pieces.PIECE_RECORD
@@ -231,7 +266,8 @@ class PagedAttention(Mixer):
         Otherwise one kernel adds the biases, rotates by angles that it forms itself from the encoding's frequencies (an
         encoding with rescaled frequencies has no table) and stores."""
         return not (self.has_bias or self.has_gate or self.softcap or self.value_norm_eps is not None
-                    or self.query_temperature is not None or self.has_distance or self.zero_sink
+                    or self.query_temperature is not None or self.has_distance or self.zero_sink or self.has_sink
+                    or self.chunk is not None or self.value_mix is not None
                     or (self.position is not None and getattr(self.position, "scaling", None) is not None))
 
     def _rotated_whole(self) -> bool:
@@ -274,7 +310,7 @@ class PagedAttention(Mixer):
             qkv = ops.linear_few(x, self.w_qkv, self.w_qkv_tiled)       # (no folded path here: the decode products up to 64 rows)
         else:
             qkv = ops.linear(x, self.w_qkv, tiled=self.w_qkv_tiled)
-        meta = attention_meta(batch, cache.group, nq // nkv, self._big_rows(batch, cache.page_size))
+        meta = attention_meta(batch, cache.group, nq // nkv, self._big_rows(batch, cache.page_size), self.chunk or 0)
         if not self._plain_projections():
             # biases, rotation and store in one kernel that reads q, k and v out of the wider product; the gate's rows,
             # which lie behind them, are multiplied into the heads' results
@@ -285,15 +321,26 @@ class PagedAttention(Mixer):
                 freq, mag, rdim = self.position.frequencies()
             slots = batch.slot_mapping(cache.group) if store else None
             vnorm = None if self.value_norm_eps is None else (self.value_norm_eps, self.value_dim)
+            mix = None
+            if self.value_mix is not None:
+                v0 = (nq + nkv) * d
+                own = qkv[:, v0:v0 + nkv * d]
+                if self.value_mix == "first":
+                    batch.shared["first_values"] = (own, nkv, d, self.value_dim)
+                else:
+                    first, heads, size, n = batch.shared["first_values"]
+                    if (heads, n) != (nkv, self.value_dim):
+                        raise ValueError("%d value heads of %d cannot be blended with %d of %d" % (nkv, self.value_dim, heads, n))
+                    mix = (first, size, n, self.mix_lambda)
             q = ops.bias_rope_store(qkv, nq, nkv, d, self.b_qkv, freq, rdim, batch.positions, cache.k, cache.v, cache.page_size, slots,
-                                    mag=mag, value_norm=vnorm, query_temperature=self.query_temperature)
+                                    mag=mag, value_norm=vnorm, query_temperature=self.query_temperature, value_mix=mix)
+            g0 = (nq + 2 * nkv) * d
+            # (a gate per value is multiplied in where the attention kernels write their result)
+            gate = qkv[:, g0:] if self.has_gate and not self.gate_per_head else None
             out = ops.paged_attention(q, cache.k, cache.v, cache.page_size, meta, nq, nkv, d, self.scale, self.window, softcap=self.softcap,
-                                      distance=self.distance, zero_sink=self.zero_sink)
+                                      distance=self.distance, sink=self.sink, chunk=self.chunk, gate=gate)
             if self.has_gate and self.gate_per_head:
-                g0 = (nq + 2 * nkv) * d
                 ops.sigmoid_gate(out, qkv[:, g0:g0 + nq], per=d)
-            elif self.has_gate:
-                ops.sigmoid_gate(out, qkv[:, (nq + 2 * nkv) * d:])
             return out
         rot = self.position.rotary() if self.position is not None else None
         cos, sin, rdim = rot if rot is not None else (None, None, 0)

@@ -34,17 +34,47 @@ class ResultGate(Part):
         return ops.GatedAddend(y, ops.linear_few(n, self.w, self.w_tiled), self.bias, self.mult)
 
 
+class ResultNorm(Part):
+    """A sublayer's result is normed, and may be multiplied element by element by a learned vector (a layer scale), before it
+    meets the stream: y / sqrt(mean(y^2) + eps) * w * s.  The two vectors are multiplied once, in float32, when the weights
+    are bound.  ``names``: the tensors' names behind the prefix for the norm's weight and the scale (None: no scale)."""
+
+    takes_expert_rows = True       # a mixture may hand its experts' rows over unsummed (``ops.ExpertRows``)
+
+    def __init__(self, hidden_size: int, eps: float, names=("norm1b", "ls1")):
+        self.hidden_size, self.eps, self.names = hidden_size, float(eps), names
+        self.weight = None
+
+    def weight_specs(self, prefix):
+        return [WeightSpec(prefix + n, (self.hidden_size,), "norm") for n in self.names if n is not None]
+
+    def bind(self, prefix, weights):
+        parts = [weights[prefix + n].float() for n in self.names if n is not None]
+        self.weight = (parts[0] * parts[1] if len(parts) > 1 else parts[0]).contiguous()
+
+    def capturable(self, batch):
+        return True
+
+    def apply(self, y, n):
+        """The normed result as an addend that the next norm's kernel forms and sums (``ops.NormedAddend``)."""
+        return ops.NormedAddend(y, self.weight, self.eps)
+
+
 class PreNormBlock(Block):
     def __init__(self, norm1: Norm, mixer: Mixer, norm2: Norm = None, ffn: FeedForward = None,
-                 names=("input_layernorm", "self_attn", "post_attention_layernorm", "mlp"), gates=None, gate_names=("rg1", "rg2")):
-        """``ffn`` (with ``norm2``) may be absent.  ``gates``: None, or a pair of ``ResultGate`` (the second None without a
-        feed-forward) that multiply the two sublayers' results, each reading its sublayer's input."""
+                 names=("input_layernorm", "self_attn", "post_attention_layernorm", "mlp"), gates=None, gate_names=("rg1", "rg2"),
+                 unread=()):
+        """``ffn`` (with ``norm2``) may be absent.  ``gates``: None, or a pair of parts (the second None without a
+        feed-forward) through which the two sublayers' results go before they meet the stream: ``ResultGate``, which reads
+        its sublayer's input as well, or ``ResultNorm``.  ``gate_names``: their prefixes behind the block's.  ``unread``: ``WeightSpec``s
+        (names behind the block's prefix) of tensors that a checkpoint may hold and the block does not read."""
         if (ffn is None) != (norm2 is None):
             raise ValueError("a feed-forward and its norm come together")
         self.norm1, self.mixer, self.norm2, self.ffn = norm1, mixer, norm2, ffn
         self.names = names
         self.gate1, self.gate2 = gates if gates is not None else (None, None)
         self.gate_names = gate_names
+        self.unread = tuple(unread)
 
     def _parts(self, prefix):
         parts = list(zip((self.norm1, self.mixer, self.norm2, self.ffn), (prefix + "." + n for n in self.names)))
@@ -52,7 +82,8 @@ class PreNormBlock(Block):
         return [(part, p) for part, p in parts if part is not None]
 
     def weight_specs(self, prefix):
-        return [s for part, p in self._parts(prefix) for s in part.weight_specs(p)]
+        return [s for part, p in self._parts(prefix) for s in part.weight_specs(p)] \
+            + [WeightSpec(prefix + "." + u.name, u.shape, u.role, optional=True) for u in self.unread]
 
     def bind(self, prefix, weights):
         for part, p in self._parts(prefix):
@@ -92,7 +123,10 @@ class PreNormBlock(Block):
         if self.ffn is None:
             return resid, a
         n2 = self.norm2.add_norm(resid, a, act)
-        f = self.ffn.forward(n2, batch)
+        if getattr(self.gate2, "takes_expert_rows", False) and hasattr(self.ffn, "forward_unsummed"):
+            f = self.ffn.forward_unsummed(n2, batch)
+        else:
+            f = self.ffn.forward(n2, batch)
         return resid, (self.gate2.apply(f, n2) if self.gate2 is not None else f)
 
 
@@ -188,7 +222,7 @@ class OutputNormBlock(Block):
             pending = None
         if pending is not None and not isinstance(pending, ops.ScaledInput):
             for addend in (pending if isinstance(pending, (tuple, list)) else (pending,)):
-                resid.add_((addend.resolve() if isinstance(addend, ops.GatedAddend) else addend).float())         # a block of another arrangement left an addend (or a pair of them)
+                resid.add_((addend.resolve() if isinstance(addend, (ops.GatedAddend, ops.NormedAddend)) else addend).float())         # a block of another arrangement left an addend (or a pair of them)
         x = stream_copy(batch, resid)
         y = self.mixer.forward(x, batch, cache, store)
         out = self.depth.result_slot(batch, resid) if self.depth is not None else resid

@@ -11,29 +11,39 @@ from .base import Part
 
 
 class TokenEmbedding(Part):
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, suffix: str = ".weight"):
-        """``scale``: h[t] = E[id[t]] * scale (a tied head still reads the table as it is stored)."""
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, suffix: str = ".weight", norm_eps: float = None,
+                 norm_suffix: str = ".norm"):
+        """``scale``: h[t] = E[id[t]] * scale (a tied head still reads the table as it is stored).  ``norm_eps``: the rows are
+        RMS-normed before the first layer, with a weight of their own (tensor ``<prefix><norm_suffix>``), in float32."""
         self.vocab_size, self.hidden_size = vocab_size, hidden_size
         self.scale, self.suffix = float(scale), suffix
-        self.weight = None
+        self.norm_eps, self.norm_suffix = None if norm_eps is None else float(norm_eps), norm_suffix
+        self.weight = self.norm = None
 
     def weight_specs(self, prefix):
-        return [WeightSpec(prefix + self.suffix, (self.vocab_size, self.hidden_size))]
+        specs = [WeightSpec(prefix + self.suffix, (self.vocab_size, self.hidden_size))]
+        if self.norm_eps is not None:
+            specs.append(WeightSpec(prefix + self.norm_suffix, (self.hidden_size,), "norm"))
+        return specs
 
     def bind(self, prefix, weights):
         self.weight = weights[prefix + self.suffix]
+        if self.norm_eps is not None:
+            self.norm = (weights[prefix + self.norm_suffix].float().contiguous(), self.norm_eps)
 
     def capturable(self, batch):
         return True
 
     def forward(self, ids):
+        if self.norm is not None:
+            return ops.embedding(ids, self.weight, self.scale, norm=self.norm)
         return ops.embedding(ids, self.weight, self.scale)
 
     def forward_for(self, ids, norm, act_dtype):
         """(stream, pending) with the input of ``norm`` prepared where few rows and a foldable norm allow it."""
         fold = norm.foldable(act_dtype) if norm is not None else None
-        if fold is None or self.scale != 1.0 or not ops.fused_decode_ok(ids.shape[0], act_dtype):
-            return ops.embedding(ids, self.weight, self.scale), None
+        if fold is None or self.scale != 1.0 or self.norm is not None or not ops.fused_decode_ok(ids.shape[0], act_dtype):
+            return self.forward(ids), None
         return ops.embedding_scaled(ids, self.weight, fold[0], fold[1], norm)
 
 

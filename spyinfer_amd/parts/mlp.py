@@ -1,10 +1,12 @@
 """Gated feed-forward: down( silu(gate(x)) * up(x) ), no biases
 (src/models/qwen3.hpp:232-263; src/backends/cpu/x64/kernels.cpp:242-247).
-Gate and up run as one product with rows [gate | up].
+Gate and up run as one product with rows [gate | up].  The gate's activation may be the tanh form of gelu instead.
 
 ``MoEMLP``: a mixture of such gated layers.  A router (float32) scores all experts, s = softmax(W_r x); the choice goes
 by s plus a stored correction, among the experts of the best groups of neighbouring experts only; a token's result is
-the sum of its chosen experts' results, weighted with the chosen s over their sum, times a constant."""
+the sum of its chosen experts' results, weighted with the chosen s over their sum, times a constant.
+
+``TableMoEMLP``: a mixture without a router: a table of the token ids names each token's experts."""
 from __future__ import annotations
 
 import torch
@@ -19,9 +21,10 @@ class GatedMLP(FeedForward):
                  names=(".gate_proj.weight", ".up_proj.weight", ".down_proj.weight")):
         """``fold_rows``: most rows of a step whose products here run with the norms and the residual sum folded in
         (None: ``ops.default_fold_rows`` of this part's matrices).  ``names``: the tensors' names behind the prefix."""
-        if activation != "silu":
+        if activation not in ops.GATED_ACTIVATIONS:
             raise ValueError("GatedMLP: activation %r is not implemented" % activation)
         self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
+        self.activation = activation
         self.fold_rows = fold_rows
         self.names = names
         self.w_gate_up = self.w_down = self.w_gate_up_tiled = self.w_down_tiled = None
@@ -52,14 +55,14 @@ class GatedMLP(FeedForward):
 
     def forward(self, x, batch):
         if isinstance(x, ops.ScaledInput):
-            return ops.linear(ops.decode_linear_swiglu(x, self.w_gate_up_tiled), self.w_down, tiled=self.w_down_tiled)
-        return ops.linear_few(ops.linear_swiglu(x, self.w_gate_up, self.w_gate_up_tiled, few_rows=ops.DECODE_ROWS_PLAIN), self.w_down,
-                              self.w_down_tiled)
+            return ops.linear(ops.decode_linear_swiglu(x, self.w_gate_up_tiled, activation=self.activation), self.w_down, tiled=self.w_down_tiled)
+        return ops.linear_few(ops.linear_swiglu(x, self.w_gate_up, self.w_gate_up_tiled, few_rows=ops.DECODE_ROWS_PLAIN, activation=self.activation),
+                              self.w_down, self.w_down_tiled)
 
     def forward_into(self, x, batch, resid, next_norm):
         weight, eps = next_norm.foldable(batch.act_dtype)
-        return ops.decode_linear_residual(ops.decode_linear_swiglu(x, self.w_gate_up_tiled, for_product=True), self.w_down_tiled,
-                                          resid, weight, eps, next_norm)
+        act = ops.decode_linear_swiglu(x, self.w_gate_up_tiled, for_product=True, activation=self.activation)
+        return ops.decode_linear_residual(act, self.w_down_tiled, resid, weight, eps, next_norm)
 
 
 class DenseMLP(FeedForward):
@@ -88,6 +91,16 @@ class DenseMLP(FeedForward):
 
     def forward(self, x, batch):
         return ops.linear_few(ops.linear_xielu(x, self.w_up, self.act, tiled=self.w_up_tiled), self.w_down, self.w_down_tiled)
+
+
+def stacked_experts(weights, experts: int, gate: str, up: str, down: str):
+    """Takes the experts' matrices out of ``weights`` (names with a place for the expert's number): every expert's [gate rows |
+    up rows] and its down matrix, the experts one after the other."""
+    mats = [weights.pop(n % e) for e in range(experts) for n in (gate, up, down)]
+    if len({m.dtype for m in mats}) > 1:
+        mats = [m.float() for m in mats]
+    return (torch.stack([torch.cat([mats[3 * e], mats[3 * e + 1]], dim=0) for e in range(experts)]).contiguous(),
+            torch.stack([mats[3 * e + 2] for e in range(experts)]).contiguous())
 
 
 class MoEMLP(FeedForward):
@@ -143,13 +156,7 @@ class MoEMLP(FeedForward):
         self.router_bias = weights[prefix + "." + self.more_names[0]].float().contiguous() if self.has_router_bias else None
         if self.shared is not None:
             self.shared.bind(prefix + "." + self.more_names[1], weights)
-        E = self.experts
-        mats = [weights.pop(n % e) for e in range(E) for n in (gate, up, down)]
-        if len({m.dtype for m in mats}) > 1:
-            mats = [m.float() for m in mats]
-        # every expert's [gate rows | up rows] and its down matrix, the experts one after the other
-        self.w_gate_up = torch.stack([torch.cat([mats[3 * e], mats[3 * e + 1]], dim=0) for e in range(E)]).contiguous()
-        self.w_down = torch.stack([mats[3 * e + 2] for e in range(E)]).contiguous()
+        self.w_gate_up, self.w_down = stacked_experts(weights, self.experts, gate, up, down)
 
     def capturable(self, batch):
         return self.shared is None or self.shared.capturable(batch)
@@ -161,3 +168,57 @@ class MoEMLP(FeedForward):
         everyone = self.shared.forward(x, batch) if self.shared is not None else None
         return ops.moe_experts(x, ids, weights, self.w_gate_up, self.w_down, activation=self.activation, limit=self.limit,
                                weight_input=self.weight_on == "input", add=everyone)
+
+
+class TableMoEMLP(FeedForward):
+    """``experts`` gated feed-forwards of inner size ``expert_size`` without a router: row ``id`` of an integer table
+    [vocab, top] names the experts of a token with that id, each with the weight 1 / top.  ``routes``: the model's
+    ``ops.ExpertTables``, which all its mixtures of this kind share: the step's (token, choice) pairs of every mixture are
+    sorted by expert in one launch, when the first of them runs.  ``activation``, ``limit``: as ``MoEMLP``.  Tensors:
+    ``table``, ``e<i>.gate``, ``e<i>.up``, ``e<i>.down``."""
+
+    def __init__(self, hidden_size: int, expert_size: int, experts: int, top: int, vocab_size: int, routes, activation: str = "clamped",
+                 limit: float = 0.0, names=("table", "e%d.gate", "e%d.up", "e%d.down")):
+        if activation not in ("silu", "clamped") or (activation == "clamped" and not limit > 0.0):
+            raise ValueError("TableMoEMLP: activation silu, or clamped with a positive limit")
+        if experts <= 0 or not 0 < top <= experts:
+            raise ValueError("%d choices among %d experts cannot be made" % (top, experts))
+        self.hidden_size, self.expert_size, self.experts, self.top, self.vocab_size = hidden_size, expert_size, experts, top, vocab_size
+        self.routes, self.activation, self.limit, self.names = routes, activation, float(limit), names
+        self.number = None
+        self.w_gate_up = self.w_down = None
+
+    def weight_specs(self, prefix):
+        H, F, E = self.hidden_size, self.expert_size, self.experts
+        table, gate, up, down = (prefix + "." + n for n in self.names)
+        specs = [WeightSpec(table, (self.vocab_size, self.top), "table", below=E)]
+        for e in range(E):
+            specs += [WeightSpec(gate % e, (F, H)), WeightSpec(up % e, (F, H)), WeightSpec(down % e, (H, F))]
+        return specs
+
+    def bind(self, prefix, weights):
+        table, gate, up, down = (prefix + "." + n for n in self.names)
+        rows = weights.pop(table)
+        lo, hi = int(rows.min()), int(rows.max())
+        if lo < 0 or hi >= self.experts:
+            raise ValueError("%s names experts %d .. %d of %d" % (table, lo, hi, self.experts))
+        self.number = self.routes.add(rows.contiguous(), self.experts, self.number)
+        self.routes.prepare()
+        self.w_gate_up, self.w_down = stacked_experts(weights, self.experts, gate, up, down)
+
+    def capturable(self, batch):
+        return True                    # the choices are read from the tables by the step's token ids, on the device
+
+    def forward(self, x, batch):
+        return self._run(x, batch, False)
+
+    def forward_unsummed(self, x, batch):
+        """The result as ``ops.ExpertRows``, for a reader that sums it in its own pass."""
+        return self._run(x, batch, True)
+
+    def _run(self, x, batch, unsummed):
+        note = ("expert_tables", id(self.routes))
+        if note not in batch.shared:
+            batch.shared[note] = self.routes.align(batch.token_ids)
+        return ops.moe_experts(x, None, None, self.w_gate_up, self.w_down, activation=self.activation, limit=self.limit,
+                               align=batch.shared[note][self.number], scale=1.0 / self.top, unsummed=unsummed)

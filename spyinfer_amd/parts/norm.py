@@ -43,15 +43,23 @@ class RMSNorm(Norm):
         return True
 
     def add_norm(self, resid, delta, out_dtype, rows=None, second=None):
-        """``delta``: None, one addend, a pair of addends (the results of two sublayers that read the same norm), or an
+        """``delta``: None, one addend, a pair of addends (the results of two sublayers that read the same norm), an
+        ``ops.GatedAddend`` or ``ops.NormedAddend`` (a result behind a gate or a norm of its own), or an
         ``ops.EntryAddends`` (any of these plus an earlier state of the stream and a vector for every row).  ``second``:
         another norm of this kind that reads the same sum: the result is the pair of both outputs, from one pass."""
+        if isinstance(delta, ops.NormedAddend):
+            # a sublayer's result behind a norm of its own: both norms and the sum in one pass
+            if second is None and self.groups == 1:
+                return ops.result_norm(resid, delta.y, delta.weight, delta.eps, self.weight, self.eps, out_dtype, rows)
+            delta = delta.resolve().to(out_dtype)
         more = {}
         if isinstance(delta, ops.EntryAddends):
             more = dict(base=delta.base, vec=delta.vec)
             delta = None if isinstance(delta.pending, ops.ScaledInput) else delta.pending
             if isinstance(delta, ops.GatedAddend):
                 delta = delta.resolve()
+            elif isinstance(delta, ops.NormedAddend):
+                delta = delta.resolve().to(out_dtype)
         if second is not None:
             if (second.size, second.eps, second.groups) != (self.size, self.eps, self.groups) or second.weight.dtype != self.weight.dtype:
                 raise ValueError("two norms of one sum must have one size, eps, grouping and weight dtype")

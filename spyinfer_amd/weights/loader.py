@@ -31,6 +31,9 @@ class WeightSpec:
     role: str = "matrix"
     #: names whose presence is tolerated but not read (a tied head stored again)
     optional: bool = False
+    #: role "table": the entries lie in 0 .. below - 1 and those of a row differ (None: random tables are drawn from the
+    #: range that the caller gives)
+    below: Optional[int] = None
 
 
 class WeightError(ValueError):

@@ -30,6 +30,12 @@ def _stream(seed: int, name: str) -> torch.Generator:
     return g
 
 
+def _distinct_rows(spec: WeightSpec, g: torch.Generator, device="cpu") -> torch.Tensor:
+    """Every row of the table: its entries drawn from 0 .. below - 1 without repeats."""
+    order = torch.rand(spec.shape[:-1] + (spec.below,), generator=g, device=device).argsort(dim=-1)
+    return order[..., :spec.shape[-1]].to(torch.int32).contiguous()
+
+
 def random_tensors(specs: Iterable[WeightSpec], seed: int, dtype: torch.dtype = torch.bfloat16,
                    matrix_std: float = 0.02, norm_mean: float = 1.0, norm_std: float = 0.01,
                    table_range: int = 2, bias_std: float = 0.02) -> Dict[str, torch.Tensor]:
@@ -42,7 +48,9 @@ def random_tensors(specs: Iterable[WeightSpec], seed: int, dtype: torch.dtype = 
         if any(n < 0 for n in s.shape):
             raise ValueError("tensor %s has a size that only a stored tensor decides; random weights need it in the configuration" % s.name)
         g = _stream(seed, s.name)
-        if s.role == "table":
+        if s.role == "table" and s.below is not None:
+            out[s.name] = _distinct_rows(s, g)
+        elif s.role == "table":
             out[s.name] = torch.randint(0, table_range, s.shape, generator=g, dtype=torch.int32)
         elif s.role == "norm":
             out[s.name] = (norm_mean + norm_std * torch.randn(s.shape, generator=g, dtype=torch.float32)).to(dtype)
@@ -74,7 +82,9 @@ def random_tensors_on_device(specs: Iterable[WeightSpec], seed: int, dtype: torc
     for s in specs:
         if s.optional:
             continue
-        if s.role == "table":
+        if s.role == "table" and s.below is not None:
+            out[s.name] = _distinct_rows(s, g, device)
+        elif s.role == "table":
             out[s.name] = torch.randint(0, 2, s.shape, generator=g, dtype=torch.int32, device=device)
         elif s.role == "norm":
             out[s.name] = (norm_mean + norm_std * torch.randn(s.shape, generator=g, dtype=torch.float32, device=device)).to(dtype)

@@ -8,8 +8,18 @@ import torch
 
 
 class EmuOps:
-    def embedding(self, ids, table, scale=1.0):
-        return table[ids.long()].float() * scale
+    def embedding(self, ids, table, scale=1.0, norm=None):
+        x = table[ids.long()].float() * scale
+        return x if norm is None else x * torch.rsqrt((x * x).mean(-1, keepdim=True) + norm[1]) * norm[0]
+
+    def result_norm(self, resid, y, result_weight, result_eps, weight, eps, out_dtype, rows=None):
+        yf = y.float()
+        x = resid + yf * torch.rsqrt((yf * yf).mean(-1, keepdim=True) + result_eps) * result_weight
+        if rows is None:
+            resid.copy_(x)
+        else:
+            x = x[rows.long()]
+        return (x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * weight.float()).to(out_dtype)
 
     def add_rms_norm(self, resid, delta, weight, eps, out_dtype, rows=None, delta2=None, groups=1, gate=None, base=None, vec=None,
                      weight2=None):
@@ -80,7 +90,7 @@ class EmuOps:
         return q.reshape(T, n_q * d).to(qkv.dtype)
 
     def paged_attention(self, q, k_cache, v_cache, page_size, meta, n_q, n_kv, d, scale, window, softcap=0.0, distance=None,
-                        zero_sink=False):
+                        sink=None, chunk=None, gate=None):
         T = meta.T
         out = torch.zeros((T, n_q, d), dtype=torch.float32)
         qf = q.float().reshape(T, n_q, d)
@@ -88,7 +98,7 @@ class EmuOps:
         for t in range(T):
             s = int(meta.token_entry[t])
             p = int(meta.positions[t])
-            lo = 0 if not window else max(0, p - window + 1)
+            lo = p - p % chunk if chunk else (0 if not window else max(0, p - window + 1))
             keys = list(range(lo, p + 1))
             pages = [int(bt[s, c // page_size]) for c in keys]
             assert all(pg >= 0 for pg in pages), "attention reads a page that is not held"
@@ -103,16 +113,19 @@ class EmuOps:
                 if distance is not None:
                     back = torch.tensor([p - c for c in keys], dtype=torch.float32)
                     sc = sc - distance[0, h] * torch.log1p(distance[1, h] * back)
-                if zero_sink:
-                    pr = torch.softmax(torch.cat([sc, torch.zeros(1)]), dim=0)[:-1]
+                if sink is not None:
+                    pr = torch.softmax(torch.cat([sc, sink[h:h + 1]]), dim=0)[:-1]
                 else:
                     pr = torch.softmax(sc, dim=0)
                 out[t, h] = pr @ V[:, g, :]
-        return out.reshape(T, n_q * d).to(q.dtype)
+        out = out.reshape(T, n_q * d)
+        return (out if gate is None else out * torch.sigmoid(gate.float())).to(q.dtype)
 
-    def swiglu(self, gate_up):
+    def swiglu(self, gate_up, activation="silu"):
         I = gate_up.shape[1] // 2
         g, u = gate_up[:, :I].float(), gate_up[:, I:].float()
+        if activation == "gelu_tanh":
+            return (torch.nn.functional.gelu(g, approximate="tanh") * u).to(gate_up.dtype)
         return (g / (1.0 + torch.exp(-g)) * u).to(gate_up.dtype)
 
     def sample(self, logits, temperature, u):
@@ -249,7 +262,7 @@ class EmuOps:
 
     # ---- attention with biases, angles formed per call, an output gate ----
     def bias_rope_store(self, x, n_q, n_kv, d, bias, freq, rotary_dim, positions, k_cache, v_cache, page_size, slots, mag=1.0,
-                        value_norm=None, query_temperature=None):
+                        value_norm=None, query_temperature=None, value_mix=None):
         T = x.shape[0]
         n = (n_q + 2 * n_kv) * d
         f = x[:, :n].float()
@@ -263,6 +276,11 @@ class EmuOps:
         if value_norm is not None:
             eps, n = value_norm
             v = v * torch.rsqrt((v[..., :n] ** 2).mean(-1, keepdim=True) + eps)
+        if value_mix is not None:
+            other, size, nv, lam = value_mix
+            first = torch.stack([other[:, g * size:g * size + nv] for g in range(n_kv)], dim=1).float()
+            v = v.clone()
+            v[..., :nv] = (1.0 - lam) * v[..., :nv] + lam * first
         if query_temperature is not None:
             coef, every = query_temperature
             steps = torch.div(positions.long() + 1, int(every), rounding_mode="floor").float()
@@ -414,8 +432,13 @@ class EmuOps:
                 ids[t, j], w[t, j] = e, float(s[e]) / tot * scale
         return ids, w
 
-    def moe_experts(self, x, ids, weights, w_gate_up, w_down, activation="silu", limit=0.0, weight_input=False, add=None):
+    def moe_experts(self, x, ids, weights, w_gate_up, w_down, activation="silu", limit=0.0, weight_input=False, add=None,
+                    align=None, scale=1.0, unsummed=False):
         T, K = x.shape
+        if align is not None:                  # (the stand-in's alignment is the choices themselves; unsummed rows come summed)
+            ids = align
+        if weights is None:
+            weights = torch.ones(ids.shape)
         F = w_gate_up.shape[1] // 2
         out = torch.zeros((T, K), dtype=torch.float32)
         xf = x.float()
@@ -432,6 +455,10 @@ class EmuOps:
                     act = g * torch.sigmoid(1.702 * g) * (u + 1.0)
                 act = act.to(x.dtype).float()
                 out[t] += (1.0 if weight_input else weights[t, j]) * (w_down[e].float() @ act)
+        out *= scale
         if add is not None:
             out += add.float()
         return out.to(x.dtype)
+
+    def align_tables(self, tables, token_ids):
+        return [t[token_ids.long()] for t in tables.tables]
