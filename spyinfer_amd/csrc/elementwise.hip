@@ -20,8 +20,10 @@ __global__ void embedding_kernel(float* __restrict__ out, const TW* __restrict__
 }
 
 // out[t, :] = row / sqrt(mean(row^2) + eps) * w, row = table[ids[t], :] * scale: an embedding that is normed before the first
-// layer.  The row is read twice, the second time from the caches.
-template <typename TW>
+// layer.  VEC (H % 4 == 0, 16-byte aligned rows of the stream and 8-byte pieces of the table, at most EN_PASSES pieces of four
+// a thread): the row is read once, in pieces asked for together and ahead of the sum that they wait for; else it is read twice.
+#define EN_PASSES 4
+template <typename TW, bool VEC>
 __global__ void embedding_norm_kernel(float* __restrict__ out, const TW* __restrict__ table, const int* __restrict__ ids, int H, int V,
                                       float scale, const float* __restrict__ w, float eps) {
     __shared__ float red[16];
@@ -34,11 +36,37 @@ __global__ void embedding_norm_kernel(float* __restrict__ out, const TW* __restr
     }
     const TW* row = table + (size_t)id * H;
     float ss = 0.f;
-#pragma unroll 4
+    if (VEC) {
+        float v[EN_PASSES][4], g[EN_PASSES][4];
+#pragma unroll
+        for (int p = 0; p < EN_PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < H) { Vec4<TW>::load(row + i, v[p]); Vec4<float>::load(w + i, g[p]); }
+        }
+#pragma unroll
+        for (int p = 0; p < EN_PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < H) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { v[p][e] *= scale; ss = fmaf(v[p][e], v[p][e], ss); }
+            }
+        }
+        ss = block_sum(ss, red);
+        const float r = 1.0f / sqrtf(ss / (float)H + eps);
+#pragma unroll
+        for (int p = 0; p < EN_PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < H) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[p][e] = (r * v[p][e]) * g[p][e];
+                Vec4<float>::store(o + i, v[p]);
+            }
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < H; i += blockDim.x) { const float v = to_f32<TW>(row[i]) * scale; ss = fmaf(v, v, ss); }
     ss = block_sum(ss, red);
     const float r = 1.0f / sqrtf(ss / (float)H + eps);
-#pragma unroll 4
     for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = (r * (to_f32<TW>(row[i]) * scale)) * w[i];
 }
 
@@ -47,7 +75,12 @@ extern "C" int spy_embedding(float* out, const void* table, int table_dtype, con
                              const float* norm_w, float eps, hipStream_t st) {
     SPY_REQUIRE(T > 0 && H > 0 && V > 0, "spy_embedding: empty operand");
     if (norm_w) {
-        SPY_DISPATCH(table_dtype, TW, (embedding_norm_kernel<TW><<<T, H >= 1024 ? 256 : 64, 0, st>>>(out, (const TW*)table, ids, H, V, scale, norm_w, eps)));
+        const int threads = H >= 4096 ? 512 : (H >= 1024 ? 256 : 64);
+        const bool vec = H % 4 == 0 && H <= threads * 4 * EN_PASSES && (((uintptr_t)out | (uintptr_t)norm_w | (uintptr_t)table) % 16) == 0;
+        SPY_DISPATCH(table_dtype, TW, {
+            if (vec) embedding_norm_kernel<TW, true><<<T, threads, 0, st>>>(out, (const TW*)table, ids, H, V, scale, norm_w, eps);
+            else embedding_norm_kernel<TW, false><<<T, threads, 0, st>>>(out, (const TW*)table, ids, H, V, scale, norm_w, eps);
+        });
         SPY_CHECK_LAUNCH("spy_embedding");
         return 0;
     }

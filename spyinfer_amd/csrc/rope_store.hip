@@ -73,6 +73,130 @@ __global__ __launch_bounds__(RS_WAVES * 64) void bias_rope_store_kernel(
     for (int j = rot + lane; j < d; j += 64) dst[j] = from_f32<TA>((to_f32<TA>(row[j]) + (b ? to_f32<TW>(b[j]) : 0.f)) * qt);
 }
 
+// The same for many bfloat16 tokens, in 16-byte pieces (d % 8 == 0, rot % 16 == 0, P % 8 == 0, no value norm).  The first T blocks
+// have a token's q and k heads each: the token's cosines and sines are formed once and lie in LDS for all its heads.  The
+// others have 16 tokens of one value head each, which go through LDS, so that a dim's 8 tokens, which lie side by side in a
+// page, leave in one store.
+typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t rs_u32x4;
+__device__ __forceinline__ void rs_widen(const rs_u32x4& r, float (&v)[8]) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { v[2 * i] = __uint_as_float(r[i] << 16); v[2 * i + 1] = __uint_as_float(r[i] & 0xffff0000u); }
+}
+__device__ __forceinline__ rs_u32x4 rs_narrow(const float (&v)[8]) {
+    return rs_u32x4{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7])};
+}
+template <typename TW>
+__global__ __launch_bounds__(256) void bias_rope_store_many_kernel(
+    const bf16_t* __restrict__ x, long long xs, bf16_t* __restrict__ q_out, int T, int n_q, int n_kv, int d, const TW* __restrict__ bias,
+    const float* __restrict__ freq, int rot, const int* __restrict__ positions, bf16_t* __restrict__ kc, bf16_t* __restrict__ vc, int P,
+    int num_pages, const int* __restrict__ slots, float mag, float qt_coef, int qt_every, const bf16_t* __restrict__ v1, long long v1s, int v1d,
+    float lam, int dv) {
+    __shared__ __align__(16) bf16_t tile[16 * (RS_MAX_D + 8)];
+    __shared__ float cs[RS_MAX_D / 2], sn[RS_MAX_D / 2];
+    const int qk_heads = n_q + n_kv, d8 = d >> 3;
+    if ((int)blockIdx.x < T) {
+        const int t = blockIdx.x, half = rot >> 1, h8 = half >> 3;
+        const int pos = positions[t];
+        const float p = (float)pos;
+        const float qt = qt_every > 0 ? 1.0f + qt_coef * logf((float)((pos + 1) / qt_every) + 1.0f) : 1.0f;
+        for (int j = threadIdx.x; j < half; j += 256) {
+            const float ang = p * freq[j];
+            cs[j] = cosf(ang) * mag;
+            sn[j] = sinf(ang) * mag;
+        }
+        __syncthreads();
+        const int slot = slots ? slots[t] : -1;
+        const bool stored = slot >= 0 && slot < num_pages * P;
+        const int page = stored ? slot / P : 0, off = stored ? slot - page * P : 0;
+        // units of a head: its rotated pairs of pieces, then the pieces that pass unchanged
+        const int per = d8 - h8;
+        for (int u = threadIdx.x; u < qk_heads * per; u += 256) {
+            const int h = u / per, c = u - h * per;
+            const bool is_q = h < n_q;
+            if (!is_q && !stored) continue;
+            const bf16_t* row = x + (size_t)t * xs + (size_t)h * d;
+            const TW* b = bias ? bias + (size_t)h * d : nullptr;
+            bf16_t* dst = is_q ? q_out + ((size_t)t * n_q + h) * d : kc + (((size_t)page * n_kv + (h - n_q)) * P + off) * d;
+            const float f = is_q ? qt : 1.0f;
+            const int ja = c < h8 ? 8 * c : rot + 8 * (c - h8);
+            float a[8], y[8];
+            rs_widen(*reinterpret_cast<const rs_u32x4*>(row + ja), a);
+            if (b) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) a[e] += to_f32<TW>(b[ja + e]);
+            }
+            if (c < h8) {
+                float o[8], z[8];
+                rs_widen(*reinterpret_cast<const rs_u32x4*>(row + ja + half), o);
+                if (b) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) o[e] += to_f32<TW>(b[ja + half + e]);
+                }
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float c_ = cs[ja + e], s_ = sn[ja + e];
+                    y[e] = (a[e] * c_ - o[e] * s_) * f;
+                    z[e] = (o[e] * c_ + a[e] * s_) * f;
+                }
+                *reinterpret_cast<rs_u32x4*>(dst + ja + half) = rs_narrow(z);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) y[e] = a[e] * f;
+            }
+            *reinterpret_cast<rs_u32x4*>(dst + ja) = rs_narrow(y);
+        }
+        return;
+    }
+    // ---- values: 16 tokens of one kv head (blocks of this kind exist only with slots) -----------------------------
+    const int vb = blockIdx.x - T;
+    const int t0 = (vb / n_kv) * 16, hv = vb % n_kv, ld = d + 8;
+    const TW* b = bias ? bias + (size_t)(qk_heads + hv) * d : nullptr;
+    for (int i = threadIdx.x; i < 16 * d8; i += 256) {
+        const int tt = i / d8, j0 = 8 * (i - tt * d8);
+        if (t0 + tt >= T) continue;
+        float v[8];
+        rs_widen(*reinterpret_cast<const rs_u32x4*>(x + (size_t)(t0 + tt) * xs + (size_t)(qk_heads + hv) * d + j0), v);
+        if (b) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] += to_f32<TW>(b[j0 + e]);
+        }
+        if (v1) {
+            const bf16_t* o = v1 + (size_t)(t0 + tt) * v1s + (size_t)hv * v1d + j0;
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                if (j0 + e < dv) v[e] = (1.0f - lam) * v[e] + lam * bf16_to_f32(o[e]);
+        }
+        *reinterpret_cast<rs_u32x4*>(tile + tt * ld + j0) = rs_narrow(v);
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < 2 * d; i += 256) {
+        const int tg = i / d, j = i - tg * d;                 // dim j of tokens t0 + 8 tg .. + 7
+        const int tb = t0 + 8 * tg;
+        if (tb >= T) continue;
+        const int s0 = slots[tb];
+        bool run = tb + 8 <= T && s0 >= 0 && s0 % 8 == 0 && s0 + 8 <= num_pages * P;
+        if (run) {
+#pragma unroll
+            for (int e = 1; e < 8; ++e) run = run && slots[tb + e] == s0 + e;
+        }
+        const bf16_t* col = tile + 8 * tg * ld + j;
+        if (run) {                                            // P is a multiple of 8: the 8 slots lie in one page
+            rs_u32x4 w;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) w[e] = (uint32_t)col[2 * e * ld] | ((uint32_t)col[(2 * e + 1) * ld] << 16);
+            const int page = s0 / P, off = s0 - page * P;
+            *reinterpret_cast<rs_u32x4*>(vc + (((size_t)page * n_kv + hv) * d + j) * P + off) = w;
+        } else {
+            for (int e = 0; e < 8 && tb + e < T; ++e) {
+                const int slot = slots[tb + e];
+                if (slot < 0 || slot >= num_pages * P) continue;
+                const int page = slot / P, off = slot - page * P;
+                vc[(((size_t)page * n_kv + hv) * d + j) * P + off] = col[e * ld];
+            }
+        }
+    }
+}
+
 extern "C" int spy_bias_rope_store(const void* x, long long xs, int dtype, void* q_out, int T, int n_q, int n_kv, int d,
                                    const void* bias, int b_dtype, const float* freq, int rot, const int* positions, void* kc,
                                    void* vc, int P, int num_pages, const int* slots, float mag, float v_eps, int v_n, float qt_coef, int qt_every,
@@ -84,6 +208,16 @@ extern "C" int spy_bias_rope_store(const void* x, long long xs, int dtype, void*
     SPY_REQUIRE(n_q + 2 * n_kv <= 65535 * RS_WAVES, "spy_bias_rope_store: too many heads");
     SPY_REQUIRE(v_n >= 0 && v_n <= d, "spy_bias_rope_store: a value norm over %d of %d values", v_n, d);
     SPY_REQUIRE(!v1 || (dv > 0 && dv <= d && v1d >= dv && v1s >= (long long)(n_kv - 1) * v1d + dv), "spy_bias_rope_store: the other layer's values do not fit");
+    const uintptr_t bits = (uintptr_t)x | (uintptr_t)q_out | (uintptr_t)kc | (uintptr_t)vc;
+    if (dtype == SPY_BF16 && T >= 64 && d % 8 == 0 && rot % 16 == 0 && xs % 8 == 0 && v_n == 0 && (!slots || P % 8 == 0) && bits % 16 == 0) {
+        const long long blocks = (long long)T + (slots ? (long long)((T + 15) / 16) * n_kv : 0);
+        SPY_REQUIRE(blocks < (1ll << 31), "spy_bias_rope_store: too many tokens");
+        SPY_DISPATCH(b_dtype, TW, (bias_rope_store_many_kernel<TW><<<(unsigned)blocks, 256, 0, st>>>(
+            (const bf16_t*)x, xs, (bf16_t*)q_out, T, n_q, n_kv, d, (const TW*)bias, freq, rot, positions, (bf16_t*)kc, (bf16_t*)vc, P, num_pages, slots,
+            mag, qt_coef, qt_every, (const bf16_t*)v1, v1s, v1d, lam, dv)));
+        SPY_CHECK_LAUNCH("spy_bias_rope_store");
+        return 0;
+    }
     const dim3 grid(T, (n_q + 2 * n_kv + RS_WAVES - 1) / RS_WAVES);
     SPY_DISPATCH(dtype, TA, SPY_DISPATCH(b_dtype, TW, (bias_rope_store_kernel<TA, TW><<<grid, RS_WAVES * 64, 0, st>>>(
         (const TA*)x, xs, (TA*)q_out, n_q, n_kv, d, (const TW*)bias, freq, rot, positions, (TA*)kc, (TA*)vc, P, num_pages, slots, mag, v_eps, v_n,
