@@ -741,3 +741,136 @@ class BalelornConfig(ModelConfig):
                 raise ConfigError("%s.mlp: the inner size must be positive" % where)
             if f and f["kind"] == "moe" and (not f["limit"] > 0.0 or f["experts"] <= 0 or not 0 < f["top"] <= f["experts"]):
                 raise ConfigError("%s.mlp: a positive limit and 1 to %d choices" % (where, max(f["experts"], 1)))
+
+
+@dataclasses.dataclass
+class NolatarConfig(ModelConfig):
+    """Nolatar: layers whose sublayers read the stream itself and add a layer norm (with a bias) of their result to it; token
+    mixers 'mamba2' (a state-space recurrence behind a short convolution, gated ahead of a norm in groups), 'attention'
+    (differential: two normed and rotated maps a head over the same values; a layer may read an earlier one's keys and
+    values) and 'parallel' (an attention in chunks with normed heads beside a retention, weighted by two constants); the
+    feed-forward a mixture of experts without gates plus an expert that every token uses, or none.  The configuration is
+    nested; ``layers`` lists every layer's type and sizes, and nothing is assumed equal between layers, except that a layer
+    that reads another's cache has its head counts, sizes and rotation."""
+
+    architecture: str = ""
+    vocab: int = -1
+    width: int = -1
+    norm_eps: float = 0.0
+    #: one dict per layer: type, mixer (sizes and constants of that mixer), mlp (None or {kind: moe, ff, experts, top, shared_ff})
+    layers: List[Dict[str, Any]] = dataclasses.field(default_factory=list)
+
+    MIXERS: ClassVar[tuple] = ("mamba2", "attention", "parallel")
+
+    @classmethod
+    def from_dict(cls, raw: Dict[str, Any]) -> "NolatarConfig":
+        cfg = cls(architecture=str(raw.get("architecture") or (raw.get("architectures") or [""])[0]),
+                  vocab=_need(raw, "vocab", int), width=_need(raw, "width", int), norm_eps=float(_need(raw, "norm.eps", (int, float))))
+        cfg.layers = [cls._layer(i, l) for i, l in enumerate(_need(raw, "layers", list))]
+        cfg._raw = dict(raw)
+        cfg.validate()
+        return cfg
+
+    @staticmethod
+    def _rotation(m: Dict[str, Any], dim: int, at: str) -> Optional[Dict[str, Any]]:
+        rot = m.get("rot")
+        if not rot:
+            return None
+        return {"base": float(_need(rot, "base", (int, float), at + ".rot")),
+                "dims": _need(rot, "dims", int, at + ".rot") if rot.get("dims") is not None else dim}
+
+    @classmethod
+    def _attention(cls, m: Dict[str, Any], at: str) -> Dict[str, Any]:
+        mix = {k: _need(m, k, int, at) for k in ("heads", "dim")}
+        mix["vdim"] = _need(m, "vdim", int, at) if m.get("vdim") is not None else mix["dim"]
+        mix["kv_heads"] = _need(m, "kv_heads", int, at) if m.get("kv_heads") is not None else mix["heads"]
+        mix["scale"] = float(_need(m, "scale", (int, float), at))
+        mix["rot"] = cls._rotation(m, mix["dim"], at)
+        return mix
+
+    @classmethod
+    def _layer(cls, i: int, raw: Dict[str, Any]) -> Dict[str, Any]:
+        where = "config.json layers[%d]" % i
+        if not isinstance(raw, dict):
+            raise ConfigError("%s is no object" % where)
+        kind = _need(raw, "type", str, where)
+        if kind not in cls.MIXERS:
+            raise ConfigError("%s: mixer type %r is not known (%s)" % (where, kind, ", ".join(cls.MIXERS)))
+        m = _need(raw, "mixer", dict, where)
+        at = where + ".mixer"
+        if kind == "mamba2":
+            mix = {k: _need(m, k, int, at) for k in ("heads", "vdim", "state", "conv")}
+            for k in ("groups", "norm_groups"):
+                mix[k] = _need(m, k, int, at) if m.get(k) is not None else 1
+        elif kind == "attention":
+            mix = cls._attention(m, at)
+            mix["diff"] = float(_need(m, "diff", (int, float), at))
+            mix["kv_from"] = _need(m, "kv_from", int, at) if m.get("kv_from") is not None else None
+        else:
+            l, r = _need(m, "left", dict, at), _need(m, "right", dict, at)
+            left = cls._attention(l, at + ".left")
+            left["chunk"] = _need(l, "mask.size", int, at + ".left") if l.get("mask") else None
+            right = {k: _need(r, k, int, at + ".right") for k in ("heads", "dim")}
+            right["vdim"] = _need(r, "vdim", int, at + ".right") if r.get("vdim") is not None else right["dim"]
+            right["rot"] = cls._rotation(r, right["dim"], at + ".right")
+            decay = _need(r, "decay", list, at + ".right")
+            if any(isinstance(x, bool) or not isinstance(x, (int, float)) for x in decay):
+                raise ConfigError("%s.right.decay must be a list of numbers" % at)
+            right["decay"] = [float(x) for x in decay]
+            mix = {"left": left, "right": right}
+            for k in ("left_scale", "right_scale"):
+                mix[k] = float(_need(m, k, (int, float), at))
+        out = {"type": kind, "mixer": mix, "mlp": None}
+        mlp = raw.get("mlp")
+        if mlp is not None:
+            at = where + ".mlp"
+            fk = _need(mlp, "kind", str, at)
+            if fk != "moe":
+                raise ConfigError("%s: kind %r is not known (moe)" % (at, fk))
+            out["mlp"] = {"kind": fk, "ff": _need(mlp, "expert.ff", int, at), "experts": _need(mlp, "router.experts", int, at),
+                          "top": _need(mlp, "router.top", int, at),
+                          "shared_ff": _need(mlp, "shared.ff", int, at) if mlp.get("shared") else None}
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        return dict(getattr(self, "_raw", {}))
+
+    def validate(self) -> None:
+        if self.vocab <= 0 or self.width <= 0:
+            raise ConfigError("config.json: vocab and width must be positive")
+        if not (self.norm_eps > 0.0):
+            raise ConfigError("config.json: norm.eps must be positive")
+        if not self.layers:
+            raise ConfigError("config.json: no layers")
+        for i, layer in enumerate(self.layers):
+            where = "config.json layers[%d]" % i
+            sides = [("", layer["mixer"])] if layer["type"] != "parallel" else [(".left", layer["mixer"]["left"]), (".right", layer["mixer"]["right"])]
+            for side, m in sides:
+                if any(isinstance(v, int) and not isinstance(v, bool) and v <= 0 for k, v in m.items() if k != "kv_from"):
+                    raise ConfigError("%s.mixer%s: sizes must be positive" % (where, side))
+                if "kv_heads" in m and m["heads"] % m["kv_heads"]:
+                    raise ConfigError("%s.mixer%s: heads (%d) is not a multiple of kv_heads (%d)" % (where, side, m["heads"], m["kv_heads"]))
+                rot = m.get("rot")
+                if rot and (rot["dims"] % 2 or not (0 < rot["dims"] <= m["dim"]) or not rot["base"] > 0.0):
+                    raise ConfigError("%s.mixer%s.rot: dims must be even and at most dim, base positive" % (where, side))
+            m = layer["mixer"]
+            if layer["type"] == "mamba2":
+                if m["heads"] % m["groups"] or (m["heads"] * m["vdim"]) % m["norm_groups"]:
+                    raise ConfigError("%s.mixer: groups must divide the heads, norm_groups the heads' values together" % where)
+                if m["conv"] > 8:
+                    raise ConfigError("%s.mixer.conv: at most 8 taps" % where)
+            elif layer["type"] == "attention":
+                src = m["kv_from"]
+                if src is not None:
+                    if not (0 <= src < i) or self.layers[src]["type"] != "attention" or self.layers[src]["mixer"]["kv_from"] is not None:
+                        raise ConfigError("%s.mixer.kv_from = %r must name an earlier attention layer with projections of its own" % (where, src))
+                    other = self.layers[src]["mixer"]
+                    if any(other[k] != m[k] for k in ("kv_heads", "dim", "vdim", "rot")):
+                        raise ConfigError("%s.mixer: kv_heads, dim, vdim and rot must equal those of layer %d, whose cache it reads" % (where, src))
+            else:
+                right = m["right"]
+                if len(right["decay"]) != right["heads"] or not all(0.0 < x <= 1.0 for x in right["decay"]):
+                    raise ConfigError("%s.mixer.right.decay: one number above 0 and up to 1 per head" % where)
+            f = layer["mlp"]
+            if f and (f["ff"] <= 0 or f["experts"] <= 0 or not 0 < f["top"] <= f["experts"] or (f["shared_ff"] is not None and f["shared_ff"] <= 0)):
+                raise ConfigError("%s.mlp: inner sizes positive, 1 to %d choices" % (where, max(f["experts"], 1)))

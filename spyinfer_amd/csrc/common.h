@@ -108,12 +108,15 @@ __device__ __forceinline__ float xielu_f(float z, float ap, float aq) {
     return z > 0.f ? fmaf(ap * z, z, 0.5f * z) : fmaf(aq, expm1f(z) - z, 0.5f * z);
 }
 
+__device__ __forceinline__ float gelu_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)); }
+
 // The activation of a gated feed-forward, z sigmoid(z (c1 + c3 z^2)) of the gate's value z:  silu with (1, 0), and the tanh
 // form of gelu, z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), with twice the tanh's two factors, 1 + tanh(y) being
 // 2 sigmoid(2 y).  The kernels take the two numbers and have no branch.
 struct GateAct { float c1, c3; };
 #define SPY_ACT_SILU 0
 #define SPY_ACT_GELU_TANH 1
+#define SPY_ACT_GELU 2           // the exact gelu, z/2 (1 + erf(z / sqrt 2)): products without a gate only
 inline bool gate_act_of(int code, GateAct* a) {
     if (code == SPY_ACT_SILU) { *a = {1.0f, 0.0f}; return true; }
     if (code == SPY_ACT_GELU_TANH) { *a = {1.5957691216057308f, 0.07135481282553525f}; return true; }

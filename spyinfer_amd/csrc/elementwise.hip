@@ -440,6 +440,34 @@ extern "C" int spy_swiglu(const void* in, void* out, int dtype, int T, int I, in
 }
 
 // ---------------------------------------------------------------------------------------------
+// In place: x = gelu(x), the exact form (a feed-forward without a gate, for products that have no epilogue of ours)
+template <typename TA, int N>
+__global__ void gelu_kernel(TA* __restrict__ x, size_t n) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+        if constexpr (N == 4) {
+            float v[4];
+            Vec4<TA>::load(x + 4 * i, v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = gelu_f(v[e]);
+            Vec4<TA>::store(x + 4 * i, v);
+        } else {
+            x[i] = from_f32<TA>(gelu_f(to_f32<TA>(x[i])));
+        }
+    }
+}
+
+extern "C" int spy_gelu(void* x, int dtype, int64_t n, hipStream_t st) {
+    SPY_REQUIRE(n > 0, "spy_gelu: empty operand");
+    const bool vec = n % 4 == 0 && ((uintptr_t)x % 16) == 0;
+    const size_t work = vec ? n / 4 : n;
+    const unsigned blocks = (unsigned)((work + 255) / 256 > 65536 ? 65536 : (work + 255) / 256);
+    if (vec) { SPY_DISPATCH(dtype, TA, (gelu_kernel<TA, 4><<<blocks, 256, 0, st>>>((TA*)x, work))); }
+    else { SPY_DISPATCH(dtype, TA, (gelu_kernel<TA, 1><<<blocks, 256, 0, st>>>((TA*)x, work))); }
+    SPY_CHECK_LAUNCH("spy_gelu");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------------------------
 // A matrix [N, K] back from the order the decode products read it ([K/128 chunks][N/16 tiles][4 steps][g = 4][r = 16][8])
 // into rows, for the library's products of many rows when only that copy of the matrix is kept.  A block moves
 // UNTILE_TILES tiles of 16 rows x 128 columns (4 KiB each, one piece of the source); thread (r, step, g) of a tile

@@ -58,6 +58,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_kernel(
     const bool act = EPI == EPI_STORE && w_next != nullptr;
     uint32_t act_raw = 0;
     if (act) act_raw = *reinterpret_cast<const uint32_t*>(w_next);
+    const bool gelu = EPI == EPI_STORE && gact.c1 == 0.f;      // (the stored product has no use for the two numbers of a gate: a first one of 0 says gelu)
 
     // Loads whose values are needed only after the product are issued now, so that they are on their way while
     // the matrix streams: every thread's share of the parts of sum(h^2) of row r (the first 256 parts; more are
@@ -182,7 +183,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_kernel(
             if (!mine) continue;
             TC* out = C + (size_t)m * N + n + 16 * nt;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) out[i] = from_f32<TC>(act ? xielu_f(acc[nt][i], act_p, act_q) : acc[nt][i]);
+            for (int i = 0; i < 4; ++i) out[i] = from_f32<TC>(act ? xielu_f(acc[nt][i], act_p, act_q) : (gelu ? gelu_f(acc[nt][i]) : acc[nt][i]));
         }
         return;
     }
@@ -192,6 +193,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_kernel(
         float v = acc[0][i];
         if (EPI == EPI_GATED) v = gated_value(gact, v, acc[NT - 1][i]);
         if (act) v = xielu_f(v, act_p, act_q);
+        if (gelu) v = gelu_f(v);
         out[i] = from_f32<TC>(v);
     }
 }
@@ -223,6 +225,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_rows_kernel(
     const bool act = EPI == EPI_STORE && w_next != nullptr;          // the stored product with an activation: see gemm_decode_kernel
     uint32_t act_raw = 0;
     if (act) act_raw = *reinterpret_cast<const uint32_t*>(w_next);
+    const bool gelu = EPI == EPI_STORE && gact.c1 == 0.f;
     f32x4_t h_old = {0.f, 0.f, 0.f, 0.f};
     uint2 wn = {0u, 0u};
     if (EPI == EPI_RESID && wave < MT && 16 * wave + r < M) {
@@ -376,6 +379,7 @@ __global__ __launch_bounds__(GD_WAVES * 64) void gemm_decode_rows_kernel(
                 float v = acc[ct][mt][i];
                 if (EPI == EPI_GATED) v = gated_value(gact, v, acc[CT + ct][mt][i]);
                 if (act) v = xielu_f(v, act_p, act_q);
+                if (gelu) v = gelu_f(v);
                 out[i] = from_f32<TC>(v);
             }
         }
@@ -482,7 +486,7 @@ extern "C" int64_t spy_gemm_decode_workspace() { return gd_splitk_workspace_byte
 // x: bfloat16 [M, K], M <= 128; MP = 16 times the row tiles the kernel is built with (M rounded up to 16 up to 64 rows, 96
 // or 128 beyond).  scaled != 0: x = bf16(h * w_norm) and ss_in
 // [n_parts, MP] holds the parts of sum(h^2); the result is multiplied by rsqrt(sum / K + eps).
-// epi 0: C [M, N] (c_dtype), with w_next = two bfloat16 numbers (p, q): xIELU of the result;  epi 1: W = [gate | up], C [M, N] = act(gate) * up (act: SPY_ACT_*);  epi 2: resid [M, N] += result,
+// epi 0: C [M, N] (c_dtype), with w_next = two bfloat16 numbers (p, q): xIELU of the result, with act SPY_ACT_GELU: its gelu;  epi 1: W = [gate | up], C [M, N] = act(gate) * up (act: SPY_ACT_*);  epi 2: resid [M, N] += result,
 // xw_out [M, N] = bf16(resid * w_next), ss_out [N / 16, MP] = every block's part of the rows' sums of squares.
 // x_tiled / out_tiled: X / the bfloat16 output for the next product (xw_out of epi 2, C of epi 1) are in operand order.
 extern "C" int spy_gemm_decode(const void* X, int scaled, const float* ss_in, int n_parts, float eps, const void* Wt, int epi,
@@ -502,12 +506,13 @@ extern "C" int spy_gemm_decode(const void* X, int scaled, const float* ss_in, in
     SPY_REQUIRE(!out_tiled || (N % 32 == 0 && (epi == EPI_RESID || (epi == EPI_GATED && c_dtype == SPY_BF16))),
                 "spy_gemm_decode: operand order is for the bfloat16 output of the gated and the residual epilogue, N a multiple of 32");
     GateAct gact;
-    SPY_REQUIRE(gate_act_of(act, &gact), "spy_gemm_decode: unknown activation %d of the gated epilogue", act);
+    if (epi == EPI_STORE && act == SPY_ACT_GELU) gact = {0.f, 0.f};
+    else SPY_REQUIRE(gate_act_of(act, &gact), "spy_gemm_decode: unknown activation %d of the gated epilogue", act);
     GdArgs a = {(const bf16_t*)X, (const bf16_t*)Wt, C, resid, (bf16_t*)xw_out, (const bf16_t*)w_next, ss_out, ss_in, n_parts, eps, M, N, K,
                 x_tiled != 0, out_tiled != 0, st, gact, ws, (long long)ws_bytes};
     const bool f32 = c_dtype == SPY_F32;
     // (a stored product with an activation is built in this file's kernels only)
-    const bool store_act = epi == EPI_STORE && w_next != nullptr;
+    const bool store_act = epi == EPI_STORE && (w_next != nullptr || act == SPY_ACT_GELU);
     if (!store_act && (gd_splitk_try(a, epi, scaled != 0, f32) || gd_wide_try(a, epi, scaled != 0, f32))) {
         SPY_CHECK_LAUNCH("spy_gemm_decode");
         return 0;

@@ -391,10 +391,11 @@ extern "C" int spy_mlstm(void* out, float* o_tmp, float* state, const void* x, l
 }
 
 // ---- short causal convolution + silu -----------------------------------------------------------------------------------
-// y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c]); inputs before the entry's first token come from the request's
-// kept inputs keep[slot][n - 1][C] (index n - 2 the newest), which are zero for a new request.
+// y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c] + bias[c]); inputs before the entry's first token come from the
+// request's kept inputs keep[slot][n - 1][C] (index n - 2 the newest), which are zero for a new request; bias may be null.
+// The plain form: any number of taps, a thread per value.
 template <typename TA, typename TW>
-__global__ void causal_conv_silu_kernel(TA* __restrict__ y, const TA* __restrict__ x, long long xs, const TW* __restrict__ taps,
+__global__ void causal_conv_silu_kernel(TA* __restrict__ y, const TA* __restrict__ x, long long xs, const TW* __restrict__ taps, const TW* __restrict__ bias,
                                         const float* __restrict__ keep, long long keep_stride, const int* __restrict__ token_entry,
                                         const int* __restrict__ cu_q, const int* __restrict__ slot_ids, int num_slots, int T, int C,
                                         int n) {
@@ -405,7 +406,7 @@ __global__ void causal_conv_silu_kernel(TA* __restrict__ y, const TA* __restrict
         const int t0 = cu_q[e];
         const int slot = slot_ids[e];
         const bool ok = slot >= 0 && slot < num_slots;
-        float acc = 0.f;
+        float acc = bias ? to_f32<TW>(bias[c]) : 0.f;
         for (int j = 0; j < n; ++j) {
             const int src = t - (n - 1) + j;
             float v;
@@ -417,8 +418,90 @@ __global__ void causal_conv_silu_kernel(TA* __restrict__ y, const TA* __restrict
     }
 }
 
-// after the convolution has read them: the kept inputs move on by the entry's tokens
+// Steps of single tokens (entry e is token e): a thread has a channel of an entry, reads its kept inputs once and leaves
+// them moved on by the token, so the second kernel falls away.
 #define CONV_MAX_TAPS 8
+template <typename TA, typename TW>
+__global__ void causal_conv_silu_step_kernel(TA* __restrict__ y, const TA* __restrict__ x, long long xs, const TW* __restrict__ taps,
+                                             const TW* __restrict__ bias, float* __restrict__ keep, long long keep_stride,
+                                             const int* __restrict__ slot_ids, int num_slots, int C, int n) {
+    const int t = blockIdx.y, c = blockIdx.x * blockDim.x + threadIdx.x;
+    if (c >= C) return;
+    const int slot = slot_ids[t];
+    const bool ok = slot >= 0 && slot < num_slots;
+    float* kp = keep + (size_t)(ok ? slot : 0) * keep_stride + c;
+    float v[CONV_MAX_TAPS];
+    const float now = to_f32<TA>(x[(size_t)t * xs + c]);
+    float acc = bias ? to_f32<TW>(bias[c]) : 0.f;
+#pragma unroll
+    for (int j = 0; j < CONV_MAX_TAPS; ++j) v[j] = j < n - 1 ? (ok ? kp[(size_t)j * C] : 0.f) : now;
+#pragma unroll
+    for (int j = 0; j < CONV_MAX_TAPS; ++j)
+        if (j < n) acc = fmaf(to_f32<TW>(taps[(size_t)c * n + j]), v[j], acc);
+    y[(size_t)t * C + c] = from_f32<TA>(acc * mm_sigmoid(acc));
+#pragma unroll
+    for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+        if (ok && j < n - 1) kp[(size_t)j * C] = v[j + 1];                   // (v[n - 1] is the token's own input)
+}
+
+// Many tokens, up to four taps: a thread has eight neighbouring channels of a run of CONV_RUN tokens, whose inputs it reads
+// once each, in 16-byte pieces, and keeps the last NT of; where an entry begins, or the run, the inputs before are fetched.
+#define CONV_RUN 16
+template <typename TW, int NT>
+__global__ __launch_bounds__(256) void causal_conv_silu_run_kernel(bf16_t* __restrict__ y, const bf16_t* __restrict__ x, long long xs,
+                                                                   const TW* __restrict__ taps, const TW* __restrict__ bias,
+                                                                   const float* __restrict__ keep, long long keep_stride,
+                                                                   const int* __restrict__ token_entry, const int* __restrict__ cu_q,
+                                                                   const int* __restrict__ slot_ids, int num_slots, int T, int C) {
+    typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4_t;
+    const int c8 = blockIdx.x * blockDim.x + threadIdx.x, c = 8 * c8;
+    if (c >= C) return;
+    auto widen = [](const u32x4_t& r, float (&v)[8]) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { v[2 * i] = __uint_as_float(r[i] << 16); v[2 * i + 1] = __uint_as_float(r[i] & 0xffff0000u); }
+    };
+    float w[NT][8], b[8], win[NT][8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        b[e] = bias ? to_f32<TW>(bias[c + e]) : 0.f;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) w[j][e] = to_f32<TW>(taps[(size_t)(c + e) * NT + j]);
+    }
+    const int ta = blockIdx.y * CONV_RUN, tb = min(ta + CONV_RUN, T);
+    for (int t = ta; t < tb; ++t) {
+        const int entry = token_entry[t], t0 = cu_q[entry];
+        if (t == ta || t == t0) {
+            const int slot = slot_ids[entry];
+            const bool ok = slot >= 0 && slot < num_slots;
+#pragma unroll
+            for (int j = 0; j < NT - 1; ++j) {
+                const int src = t - (NT - 1) + j;
+                if (src >= t0) widen(*reinterpret_cast<const u32x4_t*>(x + (size_t)src * xs + c), win[j]);
+                else {
+                    const float* kp = keep + (size_t)(ok ? slot : 0) * keep_stride + (size_t)((NT - 1) + (src - t0)) * C + c;
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) win[j][e] = ok ? kp[e] : 0.f;
+                }
+            }
+        }
+        widen(*reinterpret_cast<const u32x4_t*>(x + (size_t)t * xs + c), win[NT - 1]);
+        float o[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            float acc = b[e];
+#pragma unroll
+            for (int j = 0; j < NT; ++j) acc = fmaf(w[j][e], win[j][e], acc);
+            o[e] = acc * mm_sigmoid(acc);
+        }
+        *reinterpret_cast<u32x4_t*>(y + (size_t)t * C + c) = u32x4_t{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]), pack_bf16x2(o[4], o[5]), pack_bf16x2(o[6], o[7])};
+#pragma unroll
+        for (int j = 0; j + 1 < NT; ++j)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) win[j][e] = win[j + 1][e];
+    }
+}
+
+// after the convolution has read them: the kept inputs move on by the entry's tokens
 template <typename TA>
 __global__ void conv_keep_kernel(float* __restrict__ keep, long long keep_stride, const TA* __restrict__ x, long long xs,
                                  const int* __restrict__ cu_q, const int* __restrict__ slot_ids, int num_slots, int C, int n) {
@@ -442,15 +525,37 @@ __global__ void conv_keep_kernel(float* __restrict__ keep, long long keep_stride
         if (i < n - 1) kp[(size_t)i * C + c] = v[i];
 }
 
-extern "C" int spy_causal_conv_silu(void* y, const void* x, long long xs, int dtype, const void* taps, int w_dtype, float* keep,
+// single != 0: every entry is one token (entry e is token e).
+extern "C" int spy_causal_conv_silu(void* y, const void* x, long long xs, int dtype, const void* taps, const void* bias, int w_dtype, float* keep,
                                     long long keep_stride, const int* token_entry, const int* cu_q, const int* slot_ids,
-                                    int num_slots, int S, int T, int C, int n, hipStream_t st) {
+                                    int num_slots, int S, int T, int C, int n, int single, hipStream_t st) {
     SPY_REQUIRE(S > 0 && T > 0 && C > 0 && num_slots > 0 && xs >= C, "spy_causal_conv_silu: empty operand");
     SPY_REQUIRE(n >= 1 && n <= CONV_MAX_TAPS && keep_stride >= (long long)(n - 1) * C && S <= 65535, "spy_causal_conv_silu: %d taps (1..%d)", n, CONV_MAX_TAPS);
-    const size_t total = (size_t)T * C;
-    const unsigned blocks = (unsigned)((total + 255) / 256 > 65536 ? 65536 : (total + 255) / 256);
-    SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (causal_conv_silu_kernel<TA, TW><<<blocks, 256, 0, st>>>(
-        (TA*)y, (const TA*)x, xs, (const TW*)taps, keep, keep_stride, token_entry, cu_q, slot_ids, num_slots, T, C, n))));
+    if (single) {
+        SPY_REQUIRE(S == T, "spy_causal_conv_silu: %d tokens of %d entries", T, S);
+        const dim3 grid((C + 255) / 256, T);
+        SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (causal_conv_silu_step_kernel<TA, TW><<<grid, 256, 0, st>>>(
+            (TA*)y, (const TA*)x, xs, (const TW*)taps, (const TW*)bias, keep, keep_stride, slot_ids, num_slots, C, n))));
+        SPY_CHECK_LAUNCH("spy_causal_conv_silu (single tokens)");
+        return 0;
+    }
+    const bool pieces = dtype == SPY_BF16 && T >= 64 && C % 8 == 0 && xs % 8 == 0 && n >= 2 && n <= 4 && (((uintptr_t)x | (uintptr_t)y) % 16) == 0 &&
+                        (T + CONV_RUN - 1) / CONV_RUN <= 65535;
+    if (pieces) {
+        const dim3 grid((C / 8 + 255) / 256, (T + CONV_RUN - 1) / CONV_RUN);
+#define CONV_ARGS (bf16_t*)y, (const bf16_t*)x, xs, (const TW*)taps, (const TW*)bias, keep, keep_stride, token_entry, cu_q, slot_ids, num_slots, T, C
+        SPY_DISPATCH(w_dtype, TW, {
+            if (n == 2) causal_conv_silu_run_kernel<TW, 2><<<grid, 256, 0, st>>>(CONV_ARGS);
+            else if (n == 3) causal_conv_silu_run_kernel<TW, 3><<<grid, 256, 0, st>>>(CONV_ARGS);
+            else causal_conv_silu_run_kernel<TW, 4><<<grid, 256, 0, st>>>(CONV_ARGS);
+        });
+#undef CONV_ARGS
+    } else {
+        const size_t total = (size_t)T * C;
+        const unsigned blocks = (unsigned)((total + 255) / 256 > 65536 ? 65536 : (total + 255) / 256);
+        SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (causal_conv_silu_kernel<TA, TW><<<blocks, 256, 0, st>>>(
+            (TA*)y, (const TA*)x, xs, (const TW*)taps, (const TW*)bias, keep, keep_stride, token_entry, cu_q, slot_ids, num_slots, T, C, n))));
+    }
     SPY_CHECK_LAUNCH("spy_causal_conv_silu");
     if (n > 1) {
         const dim3 grid((C + 255) / 256, S);

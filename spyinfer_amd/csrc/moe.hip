@@ -10,6 +10,7 @@
 //   gemm:    C[row] = A[source of row] . W[expert of the row's tile]^T, float32 products and sums; optionally gated:
 //            W = [gate rows | up rows], C = silu(gate) * up; or (MoeAct kind 1) with the row's weight w multiplied into both
 //            sums first, g = min(w gate, limit), u = clamp(w up, -limit, limit), C = g sigmoid(1.702 g) (u + 1).
+//            Experts without a gate: W = [up rows], C = gelu(up).
 //            Where tables name the experts by token id, the align step of all mixtures is one launch ahead of the layers.
 //   combine: out[t] = scale * sum_k weight[t, k] * Y[row of pair (t, k)].
 #include "common.h"
@@ -18,7 +19,8 @@
 #define MOE_TM 16
 #define MOE_MAX_EXPERTS 1024
 
-// What a gated product does with its two sums (see the top).  pair_w: the weight of every (token, choice) pair, or null.
+// What a gated product does with its two sums (see the top), and one without a gate with its sum: kind 2: gelu (exact); else
+// nothing.  pair_w: the weight of every (token, choice) pair, or null.
 struct MoeAct {
     int kind;
     float limit;
@@ -30,6 +32,7 @@ __device__ __forceinline__ float moe_gated(float g, float u, const MoeAct& a, fl
     u = fminf(fmaxf(u * w, -a.limit), a.limit);
     return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
 }
+__device__ __forceinline__ float moe_ungated(float v, const MoeAct& a) { return a.kind == 2 ? gelu_f(v) : v; }
 
 // one wave per token
 __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ z,
@@ -285,6 +288,8 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(TC* __restrict__ C, const
         float v = acc[i];
         if (GATED) {
             v = moe_gated(acc[i], acc2[i], act, rw);
+        } else {
+            v = moe_ungated(v, act);
         }
         C[row * N + n] = from_f32<TC>(v);
     }
@@ -417,7 +422,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(TC* __restrict__ C, 
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         const int col = n0 + nt * 16 + 4 * g + i;
-                        if (col < N) C[row * N + col] = from_f32<TC>(acc[nt][mt][i]);
+                        if (col < N) C[row * N + col] = from_f32<TC>(moe_ungated(acc[nt][mt][i], act));
                     }
             }
         }
@@ -536,7 +541,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_lds_kernel(TC* __restrict__
 #pragma unroll
                         for (int i = 0; i < 4; ++i) {
                             const int col = n0 + nt * 16 + 4 * g + i;
-                            if (col < N) C[row * N + col] = from_f32<TC>(acc[nt][mt][i]);
+                            if (col < N) C[row * N + col] = from_f32<TC>(moe_ungated(acc[nt][mt][i], act));
                         }
                 }
             }
@@ -574,7 +579,7 @@ extern "C" int spy_moe_gemm(void* C, int c_dtype, const void* A, int a_dtype, co
                             const int* sorted_pair, int gather, int gated, int max_tiles, int E, int N, int K, int tiles_per_block,
                             int act_kind, float limit, const float* pair_w, hipStream_t st) {
     SPY_REQUIRE(max_tiles > 0 && E > 0 && N > 0 && K > 0 && gather >= 0, "spy_moe_gemm: bad sizes (%d tiles)", max_tiles);
-    SPY_REQUIRE((act_kind == 0 && !pair_w) || (act_kind == 1 && gated && limit > 0.f), "spy_moe_gemm: activation %d with limit %g", act_kind, (double)limit);
+    SPY_REQUIRE((act_kind == 0 && !pair_w) || (act_kind == 1 && gated && limit > 0.f) || (act_kind == 2 && !gated && !pair_w), "spy_moe_gemm: activation %d with limit %g", act_kind, (double)limit);
     const MoeAct act = {act_kind, limit, pair_w};
     // bfloat16 operands in 16-byte pieces: the matrix cores; tiles_per_block: 0 = the plain float32 kernel
     if (tiles_per_block > 0 && a_dtype == SPY_BF16 && w_dtype == SPY_BF16 && K % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0) {

@@ -6,16 +6,8 @@
 // sum_k weight[t, k] * Y[pair_row[t top + k]] (no weights: all one; no add: nothing), so that neither the mixture's sum nor
 // its rounding to the activation dtype is a pass of its own.  All arithmetic is float32.
 #include "common.h"
+#include "result_rows.h"
 #include <math.h>
-
-struct ExpertSum {
-    const float* y;             // [sorted rows, H]; null: the result comes as ordinary rows
-    const int* pair_row;        // [T, top]
-    const float* weights;       // [T, top] or null
-    const void* add;            // [T, H] of the activation dtype, or null
-    int top;
-    float scale;
-};
 
 // One block per row.  PASSES > 0: the row (H % 4 == 0, 16-byte aligned, at most 4 PASSES values a thread) is read once and
 // kept in registers; 0: any row, read again for every pass.

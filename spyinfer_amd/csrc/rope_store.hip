@@ -1,7 +1,8 @@
 // Projection biases, rotation by angles formed in the kernel, and the store of keys and values into their pages, for
 // attention layers whose heads are rotated in part and whose frequencies are rescaled (no table: the angle of pair j at
-// position p is float(p) * freq[j], float32, and its cosine and sine come from the full-range functions).  And the
-// sigmoid gate that such a layer multiplies into its result.
+// position p is float(p) * freq[j], float32, and its cosine and sine come from the full-range functions).  The same for
+// layers that norm every query and key head, with one map a head or several.  And what such layers do with the heads'
+// results: a sigmoid gate, the difference of two maps.
 //
 // The projections come as rows of a wider product: [q heads | k heads | v heads] of `d` values each, `xs` values from
 // one token's row to the next.  One wave per (token, head).  q -> q_out[t, h, :]; k -> K[page, h, off, :];
@@ -223,6 +224,131 @@ extern "C" int spy_bias_rope_store(const void* x, long long xs, int dtype, void*
         (const TA*)x, xs, (TA*)q_out, n_q, n_kv, d, (const TW*)bias, freq, rot, positions, (TA*)kc, (TA*)vc, P, num_pages, slots, mag, v_eps, v_n,
         qt_coef, qt_every, (const TA*)v1, v1s, v1d, lam, dv))));
     SPY_CHECK_LAUNCH("spy_bias_rope_store");
+    return 0;
+}
+
+// ---- per-head norms, rotation and store, from heads as the projections give them (no padding) ---------------------------
+// For layers that norm every query and key head (root mean square over its own `dim` values, one weight for all heads)
+// ahead of the rotation, and for layers with several maps a head (differential attention): a map is a head of its own in
+// the projection, normed and rotated by itself, while in the cache a kv head's maps lie one behind the other in ONE row of
+// d >= maps dim values, so that a map's score is the product of that row with a query that is zero in the other maps'
+// places.  One wave per (token, unit): n_q maps query units, n_kv maps key units, n_kv value units of dv values; units lie
+// `hs` (values: `hv`) values apart from their first column on.  q -> q_out[t, unit, d]; k -> K[page, g, off, :]; v ->
+// V[page, g, :, off], each filled up with zeros to d.  inter: pair j is dims (2 j, 2 j + 1) instead of (j, j + rot / 2).
+struct NormRope {
+    int n_q, n_kv, maps, dim, dv, d;
+    long long q_off, k_off, v_off;
+    int hs, hv, rot, inter, P, num_pages;
+    float eps;
+};
+template <typename TA, typename TW>
+__global__ __launch_bounds__(RS_WAVES * 64) void norm_rope_store_kernel(
+    const TA* __restrict__ x, long long xs, TA* __restrict__ q_out, NormRope a, const TW* __restrict__ qw, const TW* __restrict__ kw,
+    const float* __restrict__ freq, const int* __restrict__ positions, TA* __restrict__ kc, TA* __restrict__ vc, const int* __restrict__ slots) {
+    const int t = blockIdx.x, lane = threadIdx.x & 63;
+    int u = blockIdx.y * RS_WAVES + (threadIdx.x >> 6);
+    const int nq = a.n_q * a.maps, nk = slots ? a.n_kv * a.maps : 0, nv = slots ? a.n_kv : 0;
+    if (u >= nq + nk + nv) return;
+    const TA* row = x + (size_t)t * xs;
+    int page = 0, off = 0;
+    if (u >= nq) {
+        const int slot = slots[t];
+        if (slot < 0 || slot >= a.num_pages * a.P) return;
+        page = slot / a.P;
+        off = slot - page * a.P;
+    }
+    if (u >= nq + nk) {
+        const int g = u - nq - nk;
+        const TA* src = row + a.v_off + (size_t)g * a.hv;
+        TA* dst = vc + ((size_t)page * a.n_kv + g) * a.d * a.P + off;
+        for (int j = lane; j < a.d; j += 64) dst[(size_t)j * a.P] = j < a.dv ? src[j] : from_f32<TA>(0.f);
+        return;
+    }
+    const bool is_q = u < nq;
+    if (!is_q) u -= nq;
+    const int map = u % a.maps;
+    const TA* src = row + (is_q ? a.q_off : a.k_off) + (size_t)u * a.hs;
+    const TW* w = is_q ? qw : kw;
+    TA* dst = is_q ? q_out + ((size_t)t * nq + u) * a.d : kc + (((size_t)page * a.n_kv + u / a.maps) * a.P + off) * a.d;
+    float ss = 0.f;
+    for (int j = lane; j < a.dim; j += 64) { const float v = to_f32<TA>(src[j]); ss = fmaf(v, v, ss); }
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+    TA* at = dst + map * a.dim;
+    const int half = a.rot >> 1;
+    const float p = (float)positions[t];
+    for (int j = lane; j < half; j += 64) {
+        const int ja = a.inter ? 2 * j : j, jb = a.inter ? 2 * j + 1 : j + half;
+        const float v = (to_f32<TA>(src[ja]) * r) * to_f32<TW>(w[ja]), z = (to_f32<TA>(src[jb]) * r) * to_f32<TW>(w[jb]);
+        const float ang = p * freq[j];
+        const float cs = cosf(ang), sn = sinf(ang);
+        at[ja] = from_f32<TA>(v * cs - z * sn);
+        at[jb] = from_f32<TA>(z * cs + v * sn);
+    }
+    for (int j = a.rot + lane; j < a.dim; j += 64) at[j] = from_f32<TA>((to_f32<TA>(src[j]) * r) * to_f32<TW>(w[j]));
+    // zeros: a query's other maps and its padding; a key's padding (by the wave of its last map)
+    if (is_q) {
+        for (int j = lane; j < a.d; j += 64)
+            if (j < map * a.dim || j >= (map + 1) * a.dim) dst[j] = from_f32<TA>(0.f);
+    } else if (map == a.maps - 1) {
+        for (int j = a.maps * a.dim + lane; j < a.d; j += 64) dst[j] = from_f32<TA>(0.f);
+    }
+}
+
+extern "C" int spy_norm_rope_store(const void* x, long long xs, int dtype, void* q_out, int T, int n_q, int n_kv, int maps, int dim, int dv,
+                                   int d, long long q_off, long long k_off, long long v_off, int hs, int hv, const void* qw, const void* kw,
+                                   int w_dtype, float eps, const float* freq, int rot, int inter, const int* positions, void* kc, void* vc,
+                                   int P, int num_pages, const int* slots, hipStream_t st) {
+    SPY_REQUIRE(T > 0 && n_q > 0 && n_kv > 0 && maps > 0 && dim > 0 && dv > 0 && d >= maps * dim && d >= dv && hs >= dim, "spy_norm_rope_store: bad sizes");
+    SPY_REQUIRE(rot >= 0 && rot <= dim && rot % 2 == 0 && (rot == 0 || freq), "spy_norm_rope_store: %d rotated dims do not fit a head of %d", rot, dim);
+    SPY_REQUIRE(qw && (!slots || kw), "spy_norm_rope_store: no norm weights");
+    SPY_REQUIRE(q_off >= 0 && q_off + (long long)(n_q * maps - 1) * hs + dim <= xs, "spy_norm_rope_store: the queries' columns reach beyond the rows");
+    SPY_REQUIRE(!slots || (kc && vc && P > 0 && num_pages > 0 && hv >= dv && k_off >= 0 && v_off >= 0 &&
+                           k_off + (long long)(n_kv * maps - 1) * hs + dim <= xs && v_off + (long long)(n_kv - 1) * hv + dv <= xs),
+                "spy_norm_rope_store: slots without a cache, or the keys' or values' columns reach beyond the rows");
+    const int units = (n_q + (slots ? n_kv : 0)) * maps + (slots ? n_kv : 0);
+    SPY_REQUIRE(units <= 65535 * RS_WAVES, "spy_norm_rope_store: too many heads");
+    const NormRope a = {n_q, n_kv, maps, dim, dv, d, q_off, k_off, v_off, hs, hv, rot, inter, P, num_pages, eps};
+    const dim3 grid(T, (units + RS_WAVES - 1) / RS_WAVES);
+    SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (norm_rope_store_kernel<TA, TW><<<grid, RS_WAVES * 64, 0, st>>>(
+        (const TA*)x, xs, (TA*)q_out, a, (const TW*)qw, (const TW*)kw, freq, positions, (TA*)kc, (TA*)vc, slots))));
+    SPY_CHECK_LAUNCH("spy_norm_rope_store");
+    return 0;
+}
+
+// ---- two maps of a head into one -----------------------------------------------------------------------------------------
+// x [T, H, 2, d] (only the first dv values of a map's result count) -> out [T, H dv]: o = x1 - lam x2, over its root mean
+// square (mean over the dv values, no weight), times `mult`.  One wave per (token, head).
+template <typename TA, typename TO>
+__global__ __launch_bounds__(RS_WAVES * 64) void map_difference_kernel(TO* __restrict__ out, const TA* __restrict__ x, int heads, int dv, int d,
+                                                                       float lam, float eps, float mult) {
+    const int i = blockIdx.x * RS_WAVES + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (i >= heads) return;
+    const TA* a = x + (size_t)i * 2 * d;
+    TO* o = out + (size_t)i * dv;
+    float v[RS_MAX_D / 64];
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < RS_MAX_D / 64; ++e) {
+        const int j = lane + 64 * e;
+        v[e] = j < dv ? to_f32<TA>(a[j]) - lam * to_f32<TA>(a[d + j]) : 0.f;
+        ss = fmaf(v[e], v[e], ss);
+    }
+    const float r = mult / sqrtf(wave_sum(ss) / (float)dv + eps);
+#pragma unroll
+    for (int e = 0; e < RS_MAX_D / 64; ++e) {
+        const int j = lane + 64 * e;
+        if (j < dv) o[j] = from_f32<TO>(v[e] * r);
+    }
+}
+
+extern "C" int spy_map_difference(void* out, int out_dtype, const void* x, int dtype, int T, int H, int dv, int d, float lam, float eps,
+                                  float mult, hipStream_t st) {
+    SPY_REQUIRE(T > 0 && H > 0 && dv > 0 && d >= dv && d <= RS_MAX_D, "spy_map_difference: heads of %d in rows of %d (up to %d)", dv, d, RS_MAX_D);
+    SPY_REQUIRE((long long)T * H < (1ll << 31) - RS_WAVES, "spy_map_difference: too many heads");
+    const int heads = T * H;
+    SPY_DISPATCH(dtype, TA, SPY_DISPATCH(out_dtype, TO, (map_difference_kernel<TA, TO><<<(heads + RS_WAVES - 1) / RS_WAVES, RS_WAVES * 64, 0, st>>>(
+        (TO*)out, (const TA*)x, heads, dv, d, lam, eps, mult))));
+    SPY_CHECK_LAUNCH("spy_map_difference");
     return 0;
 }
 

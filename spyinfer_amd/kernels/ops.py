@@ -79,7 +79,8 @@ class _Hip:
                      "spy_gemm_strided", "spy_latent_attention", "spy_latent_attention_mfma", "spy_latent_attention_mfma_workspace", "spy_head_products",
                      "spy_bias_rope_store", "spy_sigmoid_gate", "spy_mlstm", "spy_causal_conv_silu", "spy_delta_rule", "spy_moe_route",
                      "spy_moe_align", "spy_moe_gemm", "spy_moe_combine", "spy_moe_tile_rows", "spy_token_shift", "spy_tanh", "spy_time_mix",
-                     "spy_norm_pair_mean", "spy_scale_cap", "spy_result_norm", "spy_moe_align_tables"):
+                     "spy_norm_pair_mean", "spy_scale_cap", "spy_result_norm", "spy_moe_align_tables", "spy_layer_norm", "spy_layer_norm_residual",
+                     "spy_gelu", "spy_norm_rope_store", "spy_map_difference", "spy_rotation_angles", "spy_decay_memory", "spy_group_norm"):
             if not hasattr(self.lib, name):
                 raise KernelError("the kernel library %s lacks %s: it is older than its sources; build it again "
                                   "(spyinfer_amd.kernels.build.build())" % (self.lib._name, name))
@@ -211,6 +212,73 @@ def result_norm(resid: torch.Tensor, y, result_weight: torch.Tensor, result_eps:
                    ctypes.c_int(ex[4]), ctypes.c_float(ex[5]), _ptr(result_weight), ctypes.c_float(result_eps), _ptr(weight),
                    _code(weight, "norm weight"), ctypes.c_float(eps), _ptr(out), _ptr(rows), ctypes.c_int(n_out), ctypes.c_int(T), ctypes.c_int(H),
                    _Hip.stream())
+    return out
+
+
+class WeightedPair:
+    """Two sublayers' results that meet weighted: the addend is ``sa * a + sb * b`` (rows of the activation dtype).  The norm
+    that reads it forms it in its own pass (``layer_norm_residual``); whoever cannot calls ``resolve``."""
+    __slots__ = ("a", "b", "sa", "sb")
+
+    def __init__(self, a, b, sa, sb):
+        self.a, self.b, self.sa, self.sb = a, b, float(sa), float(sb)
+
+    def resolve(self):
+        return (self.a.float() * self.sa + self.b.float() * self.sb).to(self.a.dtype)
+
+
+def layer_norm_residual(base: torch.Tensor, y, weight: torch.Tensor, bias: torch.Tensor, eps: float, out: Optional[torch.Tensor] = None,
+                        copy_dtype: Optional[torch.dtype] = None):
+    """out = base + (y - mean) / sqrt(mean squared deviation + eps) * weight + bias, float32 (``out`` may be ``base``; a new
+    tensor if None).  ``y``: rows [T, H] of the activation dtype, a ``WeightedPair``, or ``ExpertRows`` (a mixture's unsummed
+    rows); the latter two are summed here.  Returns (out, copy of out in ``copy_dtype`` or None)."""
+    experts = y if isinstance(y, ExpertRows) else None
+    pair = y if isinstance(y, WeightedPair) else None
+    rows = y if experts is None and pair is None else None
+    _dev(base, rows, weight, bias, out)
+    _check(base.dtype == torch.float32 and base.dim() == 2, "layer_norm_residual: the stream must be float32 [T, H]")
+    T, H = base.shape
+    _check(weight.shape == (H,) and bias.shape == (H,) and weight.dtype == bias.dtype, "layer_norm_residual: weight and bias [H] of one dtype expected")
+    if out is None:
+        out = torch.empty_like(base)
+    _check(out.dtype == torch.float32 and tuple(out.shape) == (T, H), "layer_norm_residual: out must be float32 [T, H]")
+    if experts is not None:
+        _check(tuple(experts.shape) == (T, H), "layer_norm_residual: the experts' rows must be those of the step's tokens")
+        _dev(experts.y, experts.pair_row, experts.weights, experts.add)
+        dtype = experts.dtype
+        ex = (experts.y, experts.pair_row, experts.weights, experts.add, experts.top, experts.scale)
+    else:
+        ex = (None, None, None, None, 0, 1.0)
+        if pair is not None:
+            _dev(pair.a, pair.b)
+            _check(tuple(pair.a.shape) == (T, H) and pair.b.shape == pair.a.shape and pair.a.dtype == pair.b.dtype, "layer_norm_residual: a pair of rows [T, H] of one dtype expected")
+        else:
+            _check(tuple(y.shape) == (T, H), "layer_norm_residual: rows [T, H] expected")
+        dtype = pair.a.dtype if pair is not None else y.dtype
+    _check(dtype in _CODES and (copy_dtype in (None, torch.float32, dtype)), "layer_norm_residual: the copy has the result's dtype")
+    copy = _copy_of(out, copy_dtype)
+    if T:
+        hip().call("spy_layer_norm_residual", _ptr(out), _ptr(copy), _ptr(base), ctypes.c_int(_CODES[dtype]), _ptr(rows),
+                   _ptr(pair.a if pair is not None else None), _ptr(pair.b if pair is not None else None),
+                   ctypes.c_float(pair.sa if pair is not None else 0.0), ctypes.c_float(pair.sb if pair is not None else 0.0),
+                   _ptr(ex[0]), _ptr(ex[1]), _ptr(ex[2]), _ptr(ex[3]), ctypes.c_int(ex[4]), ctypes.c_float(ex[5]), _ptr(weight), _ptr(bias),
+                   _code(weight, "norm weight"), ctypes.c_float(eps), ctypes.c_int(T), ctypes.c_int(H), _Hip.stream())
+    return out, copy
+
+
+def layer_norm(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float, out_dtype: torch.dtype,
+               rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The layer norm of float32 rows ``x [T, H]``, in ``out_dtype``; ``rows`` (int32 [R]): of those rows only -> [R, H]."""
+    _dev(x, weight, bias, rows)
+    _check(x.dtype == torch.float32 and x.dim() == 2, "layer_norm: float32 rows [T, H] expected")
+    T, H = x.shape
+    _check(weight.shape == (H,) and bias.shape == (H,) and weight.dtype == bias.dtype, "layer_norm: weight and bias [H] of one dtype expected")
+    _check(rows is None or (rows.dtype == torch.int32 and rows.dim() == 1), "layer_norm: rows must be int32 [R]")
+    n = T if rows is None else rows.shape[0]
+    out = torch.empty((n, H), dtype=out_dtype, device=x.device)
+    if n:
+        hip().call("spy_layer_norm", _ptr(out), _code(out, "out"), _ptr(x), _ptr(weight), _ptr(bias), _code(weight, "norm weight"),
+                   ctypes.c_float(eps), _ptr(rows), ctypes.c_int(n), ctypes.c_int(T), ctypes.c_int(H), _Hip.stream())
     return out
 
 
@@ -412,6 +480,8 @@ def linear_few(x: torch.Tensor, w: torch.Tensor, tiled: Optional[torch.Tensor] =
 
 #: activations of a gated feed-forward: "silu", or the tanh form of gelu, z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
 GATED_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+#: code of the exact gelu, the activation of products without a gate
+ACT_GELU = 2
 
 
 def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, tiled: Optional[torch.Tensor] = None, few_rows: int = 0,
@@ -1123,6 +1193,23 @@ def linear_xielu(x: torch.Tensor, w: torch.Tensor, pq: torch.Tensor, tiled: Opti
     return xielu(linear_few(x, w, tiled), pq)
 
 
+def gelu(x: torch.Tensor) -> torch.Tensor:
+    """In place: x/2 (1 + erf(x / sqrt 2)), float32 arithmetic."""
+    _dev(x)
+    if x.numel():
+        hip().call("spy_gelu", _ptr(x), ctypes.c_int(_code(x, "x")), ctypes.c_int64(x.numel()), _Hip.stream())
+    return x
+
+
+def linear_gelu(x: torch.Tensor, w: torch.Tensor, tiled: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """gelu(x . w^T), the exact form; for few bfloat16 rows in the product's store epilogue."""
+    if tiled is not None and x.dtype == torch.bfloat16 and x.dim() == 2 and 0 < x.shape[0] <= DECODE_ROWS_PLAIN and x.is_contiguous():
+        out = torch.empty((x.shape[0], tiled.shape[0]), dtype=torch.bfloat16, device=x.device)
+        _gemm_decode(x, tiled, 0, tiled.shape[0], out, None, None, None, None, ACT_GELU)
+        return out
+    return gelu(linear_few(x, w, tiled))
+
+
 # --------------------------------------------------------------------------
 def mingru(zxg: torch.Tensor, bz: torch.Tensor, bx: torch.Tensor, state: torch.Tensor, pieces: torch.Tensor, n_pieces: int,
            multi: bool, slot_ids: torch.Tensor) -> torch.Tensor:
@@ -1347,6 +1434,65 @@ def bias_rope_store(x: torch.Tensor, n_q: int, n_kv: int, d: int, bias: Optional
     return q
 
 
+def norm_rope_store(x: torch.Tensor, n_q: int, n_kv: int, dim: int, value_dim: int, d: int, q_norm_w: torch.Tensor,
+                    k_norm_w: Optional[torch.Tensor], eps: float, freq: Optional[torch.Tensor], rotary_dim: int, positions: torch.Tensor,
+                    k_cache, v_cache, page_size: int, slots: Optional[torch.Tensor], maps: int = 1, interleaved: bool = False,
+                    columns=None) -> torch.Tensor:
+    """From rows ``x`` (a view into a wider product may be given) with n_q query heads, n_kv key heads and n_kv value heads:
+    every query and key head over its root mean square times its weight ``[dim]``, the first ``rotary_dim`` dims of it
+    rotated (angle float32(position) * freq[j]; pair j is (j, j + rotary_dim / 2), ``interleaved``: (2 j, 2 j + 1)); q written
+    to the result [T, n_q maps, d], k and v into the cache pages at ``slots`` (None: the layer reads another's cache; x then
+    has queries only).  ``maps``: maps of a head, each a head of ``dim`` values of its own in x; a kv head's cache row holds
+    them one behind the other, and a query's row is zero outside its own map's place.  All rows are filled up with zeros to
+    ``d``.  ``columns`` = (first column of q, of k, of v, values from one q or k head to the next, from one value head to the
+    next); None: [q heads | k heads | v heads] without gaps."""
+    xs = _row_view(x, "norm_rope_store")
+    T = x.shape[0]
+    if columns is None:
+        columns = (0, n_q * maps * dim, (n_q + n_kv) * maps * dim, dim, value_dim)
+    q0, k0, v0, hs, hv = (int(c) for c in columns)
+    _dev(q_norm_w, k_norm_w, freq, positions, k_cache, v_cache, slots)
+    _check(d >= maps * dim and d >= value_dim and hs >= dim, "norm_rope_store: %d maps of %d or values of %d in rows of %d", maps, dim, value_dim, d)
+    _check(q_norm_w.shape == (dim,) and (k_norm_w is None or (k_norm_w.shape == (dim,) and k_norm_w.dtype == q_norm_w.dtype)),
+           "norm_rope_store: norm weights must be [dim] of one dtype")
+    _check(0 <= q0 and q0 + (n_q * maps - 1) * hs + dim <= x.shape[1], "norm_rope_store: the queries' columns reach beyond the rows")
+    _check(positions.dtype == torch.int32 and positions.shape == (T,), "norm_rope_store: positions must be int32 [T]")
+    _check(rotary_dim == 0 or (freq is not None and freq.dtype == torch.float32 and freq.shape == (rotary_dim // 2,) and rotary_dim % 2 == 0
+                               and rotary_dim <= dim), "norm_rope_store: one float32 frequency per rotated pair expected")
+    num_pages = 0
+    if slots is not None:
+        _check(slots.dtype == torch.int32 and slots.shape == (T,) and k_norm_w is not None, "norm_rope_store: slots must be int32 [T], and keys have a norm")
+        _check(0 <= k0 and k0 + (n_kv * maps - 1) * hs + dim <= x.shape[1] and 0 <= v0 and v0 + (n_kv - 1) * hv + value_dim <= x.shape[1] and hv >= value_dim,
+               "norm_rope_store: the keys' or values' columns reach beyond the rows")
+        num_pages = k_cache.shape[0]
+        _check(k_cache.dtype == x.dtype and v_cache.dtype == x.dtype and tuple(k_cache.shape) == (num_pages, n_kv, page_size, d)
+               and tuple(v_cache.shape) == (num_pages, n_kv, d, page_size),
+               "norm_rope_store: cache pages must be K [pages, n_kv, page, d] and V [pages, n_kv, d, page] of the activation dtype")
+    q = torch.empty((T, n_q * maps * d), dtype=x.dtype, device=x.device)
+    if T:
+        L, I = ctypes.c_longlong, ctypes.c_int
+        hip().call("spy_norm_rope_store", ctypes.c_void_p(x.data_ptr()), L(xs), _code(x, "x"), _ptr(q), I(T), I(n_q), I(n_kv), I(maps), I(dim),
+                   I(value_dim), I(d), L(q0), L(k0), L(v0), I(hs), I(hv), _ptr(q_norm_w), _ptr(k_norm_w), _code(q_norm_w, "head norm weight"),
+                   ctypes.c_float(eps), _ptr(freq), I(rotary_dim), I(1 if interleaved else 0), _ptr(positions),
+                   _ptr(k_cache if slots is not None else None), _ptr(v_cache if slots is not None else None), I(page_size), I(num_pages),
+                   _ptr(slots), _Hip.stream())
+    return q
+
+
+def map_difference(x: torch.Tensor, heads: int, value_dim: int, d: int, lam: float, eps: float, mult: float,
+                   out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+    """``x [T, heads * 2 * d]``: two maps' results of every head, ``value_dim`` values in rows of d.  o = x1 - lam x2 over its root
+    mean square, times ``mult`` -> [T, heads * value_dim]."""
+    _dev(x)
+    T = x.shape[0]
+    _check(x.dim() == 2 and x.shape[1] == heads * 2 * d and 0 < value_dim <= d, "map_difference: rows of two maps of %d per head expected", d)
+    out = torch.empty((T, heads * value_dim), dtype=out_dtype or x.dtype, device=x.device)
+    if T:
+        hip().call("spy_map_difference", _ptr(out), _code(out, "out"), _ptr(x), _code(x, "x"), ctypes.c_int(T), ctypes.c_int(heads),
+                   ctypes.c_int(value_dim), ctypes.c_int(d), ctypes.c_float(lam), ctypes.c_float(eps), ctypes.c_float(mult), _Hip.stream())
+    return out
+
+
 def sigmoid_gate(y: torch.Tensor, gate: torch.Tensor, bias: Optional[torch.Tensor] = None, mult: float = 1.0, per: int = 1) -> torch.Tensor:
     """In place: y[t, j] *= mult * sigmoid(gate[t, j / per] + bias[j / per]); ``gate`` may be a view into a wider product.
     ``per``: columns of y that share one gate value (a head's size: one number per head)."""
@@ -1425,14 +1571,15 @@ def mlstm(x: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: int, gates
 
 
 def causal_conv_silu(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, keep_off: int, token_entry: torch.Tensor,
-                     cu_q: torch.Tensor, slot_ids: torch.Tensor) -> torch.Tensor:
-    """y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c]) per request (``x [T, C]`` may be a view into a wider
+                     cu_q: torch.Tensor, slot_ids: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """y[t, c] = silu(sum_j taps[c, j] x[t - (n - 1) + j, c] + bias[c]) per request (``x [T, C]`` may be a view into a wider
     product); inputs before an entry's first token are the request's kept inputs ``state[slot, keep_off + i C + c]``
     (i = 0 .. n - 2, the newest last; float32), which afterwards hold the entry's last n - 1 inputs."""
     xs = _row_view(x, "causal_conv_silu")
     T, C = x.shape
-    _dev(taps, state, token_entry, cu_q, slot_ids)
+    _dev(taps, state, token_entry, cu_q, slot_ids, bias)
     S = _entries(cu_q, slot_ids, "causal_conv_silu")
+    _check(bias is None or (bias.shape == (C,) and bias.dtype == taps.dtype), "causal_conv_silu: one bias per channel, of the taps' dtype, expected")
     _check(taps.dim() == 2 and taps.shape[0] == C and 1 <= taps.shape[1] <= 8, "causal_conv_silu: taps [C, 1..8] expected")
     n = taps.shape[1]
     _check(token_entry.dtype == torch.int32 and token_entry.shape == (T,), "causal_conv_silu: token_entry must be int32 [T]")
@@ -1440,10 +1587,10 @@ def causal_conv_silu(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, k
            "causal_conv_silu: the kept inputs reach beyond the float32 state")
     y = torch.empty((T, C), dtype=x.dtype, device=x.device)
     if T:
-        hip().call("spy_causal_conv_silu", _ptr(y), ctypes.c_void_p(x.data_ptr()), ctypes.c_longlong(xs), _code(x, "x"), _ptr(taps),
+        hip().call("spy_causal_conv_silu", _ptr(y), ctypes.c_void_p(x.data_ptr()), ctypes.c_longlong(xs), _code(x, "x"), _ptr(taps), _ptr(bias),
                    _code(taps, "taps"), ctypes.c_void_p(state.data_ptr() + 4 * keep_off), ctypes.c_longlong(state.shape[1]), _ptr(token_entry),
                    _ptr(cu_q), _ptr(slot_ids), ctypes.c_int(state.shape[0]), ctypes.c_int(S), ctypes.c_int(T), ctypes.c_int(C), ctypes.c_int(n),
-                   _Hip.stream())
+                   ctypes.c_int(1 if S == T else 0), _Hip.stream())      # (as many entries as tokens: every entry is one token)
     return y
 
 
@@ -1551,6 +1698,109 @@ def norm_pair_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch
         hip().call("spy_norm_pair_mean", _ptr(out), _ptr(a), _ptr(b), _code(a, "rows"), _ptr(wa), _ptr(wb), _code(wa, "norm weight"),
                    ctypes.c_float(eps), ctypes.c_int(T), ctypes.c_int(W), _Hip.stream())
     return out
+
+
+DECAY_PIECE = 64                  # most tokens of a piece of ``decay_memory``
+DECAY_NORM_MAX_VDIM = 128         # largest value head whose norm and gate ride in the recurrence's kernels
+
+
+def rotation_angles(positions: torch.Tensor, freq: torch.Tensor) -> torch.Tensor:
+    """[T, pairs, 2] float32: cosine and sine of float32(position) * freq[j]."""
+    _dev(positions, freq)
+    _check(positions.dtype == torch.int32 and positions.dim() == 1 and freq.dtype == torch.float32 and freq.dim() == 1 and freq.shape[0] > 0,
+           "rotation_angles: positions int32 [T] and float32 frequencies expected")
+    T, half = positions.shape[0], freq.shape[0]
+    out = torch.empty((T, half, 2), dtype=torch.float32, device=positions.device)
+    if T:
+        hip().call("spy_rotation_angles", _ptr(out), _ptr(positions), _ptr(freq), ctypes.c_int(T), ctypes.c_int(half), _Hip.stream())
+    return out
+
+
+def group_norm(o: torch.Tensor, weight: Optional[torch.Tensor], eps: float, groups: int, out_dtype: torch.dtype,
+               gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Float32 rows [T, N], each of ``groups`` equal runs over its own root mean square, times ``weight [N]`` (None: nothing),
+    times silu(``gate``) (rows [T, N] of ``out_dtype``, a view into a wider product may be given)."""
+    _dev(o, weight)
+    _check(o.dtype == torch.float32 and o.dim() == 2 and groups > 0 and o.shape[1] % groups == 0, "group_norm: float32 rows in %d groups expected", groups)
+    T, N = o.shape
+    _check(weight is None or weight.shape == (N,), "group_norm: a weight [N] expected")
+    gs = 0
+    if gate is not None:
+        gs = _row_view(gate, "group_norm")
+        _check(gate.dtype == out_dtype and gate.shape == (T, N) and gate.device == o.device, "group_norm: gate rows [T, N] of the result's dtype expected")
+    out = torch.empty((T, N), dtype=out_dtype, device=o.device)
+    if T:
+        hip().call("spy_group_norm", _ptr(out), _code(out, "out"), _ptr(o), _ptr(weight), _code(weight, "norm weight") if weight is not None else F32,
+                   ctypes.c_void_p(0 if gate is None else gate.data_ptr()), ctypes.c_longlong(gs), ctypes.c_float(eps), ctypes.c_int(T), ctypes.c_int(groups), ctypes.c_int(N), _Hip.stream())
+    return out
+
+
+def decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, H: int, G: int, d: int, dv: int, state: torch.Tensor, cu_q: torch.Tensor,
+                 slot_ids: torch.Tensor, pieces, kscale: float = 1.0, log_decay: Optional[torch.Tensor] = None, steps=None,
+                 angles: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, norm_eps: Optional[float] = None,
+                 skip: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per head a state S [d, dv] (``state[slot, h d dv ..]`` float32, row = key channel), read at an entry's start and left at
+    its end:  S = a S + b (kscale k) v^T,  o = S^T q.  ``q``, ``k``: rows of G heads of d (head h of H reads head h // (H / G)),
+    ``v``: rows of H heads of dv; all may be views into wider products.  Decay: ``log_decay`` float32 [H] (a constant per
+    head, b = 1), or ``steps`` = (raw step sizes float32 [T, H], bias float32 [H], rate float32 [H]): dt = softplus(raw + bias),
+    a = exp(-rate dt), b = dt.  ``angles`` (``rotation_angles``): q and k are rotated first, pairs (j, j + pairs).  ``pieces`` =
+    (int32 [4 n], n, whether there are several per entry) of at most DECAY_PIECE tokens.
+    The result: o [T, H dv] float32; with ``norm_eps``: every head's o over its root mean square, times silu(``gate``), in the
+    operands' dtype; with ``skip`` (float32 [H]): (o + skip_h v) silu(``gate``), float32."""
+    qs, ks, vs = (_row_view(t, "decay_memory") for t in (q, k, v))
+    T = q.shape[0]
+    S = _entries(cu_q, slot_ids, "decay_memory")
+    _dev(state, cu_q, slot_ids, log_decay, angles, skip)
+    _check(q.dtype == k.dtype == v.dtype and k.shape[0] == T and v.shape[0] == T and q.device == k.device == v.device == state.device,
+           "decay_memory: q, k and v rows of one dtype expected")
+    _check(H % G == 0 and min(q.shape[1], k.shape[1]) >= G * d and v.shape[1] >= H * dv, "decay_memory: rows are too short for %d / %d heads of %d x %d", G, H, d, dv)
+    _check(0 < d <= MATRIX_MEMORY_MAX_DIM and 0 < dv <= MATRIX_MEMORY_MAX_VDIM, "decay_memory: heads of %d x %d (up to %d x %d)", d, dv,
+           MATRIX_MEMORY_MAX_DIM, MATRIX_MEMORY_MAX_VDIM)
+    _check(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] >= H * d * dv, "decay_memory: state must be float32 [slots, >= H d dv]")
+    _check((log_decay is None) != (steps is None), "decay_memory: a constant decay or step sizes")
+    _check(log_decay is None or (log_decay.dtype == torch.float32 and log_decay.shape == (H,)), "decay_memory: log decays float32 [H] expected")
+    dt = dt_bias = rate = None
+    dts = 0
+    if steps is not None:
+        dt, dt_bias, rate = steps
+        dts = _row_view(dt, "decay_memory")
+        _dev(dt_bias, rate)
+        _check(dt.dtype == torch.float32 and dt.shape == (T, H) and all(t.dtype == torch.float32 and t.shape == (H,) for t in (dt_bias, rate)),
+               "decay_memory: step sizes [T, H], their bias and rate [H], all float32, expected")
+    half = 0
+    if angles is not None:
+        half = angles.shape[1]
+        _check(angles.dtype == torch.float32 and angles.shape == (T, half, 2) and 2 * half <= d, "decay_memory: angles float32 [T, pairs, 2] expected")
+    gs = 0
+    if gate is not None:
+        gs = _row_view(gate, "decay_memory")
+        _check(gate.dtype == q.dtype and gate.shape == (T, H * dv) and gate.device == q.device, "decay_memory: gate rows [T, H dv] like q expected")
+    _check((norm_eps is None or skip is None) and (gate is not None) == (norm_eps is not None or skip is not None), "decay_memory: a gate comes with a norm or with a skip")
+    _check(skip is None or (skip.dtype == torch.float32 and skip.shape == (H,)), "decay_memory: skip float32 [H] expected")
+    # the head's norm rides in the recurrence's kernel where a block has the whole head
+    quads = dv % 4 == 0 and state.shape[1] % 4 == 0 and state.data_ptr() % 16 == 0
+    fused = norm_eps is not None and dv <= DECAY_NORM_MAX_VDIM and quads
+    epi = 1 if fused else (2 if skip is not None else 0)
+    out = torch.empty((T, H * dv), dtype=q.dtype if fused else torch.float32, device=q.device)
+    if T:
+        single = S == T                                    # as many entries as tokens: every entry is one token
+        parr = work = decay = None
+        n = 0
+        if not single:
+            parr, n, _ = pieces
+            _dev(parr)
+            _check(parr.dtype == torch.int32 and parr.shape == (4 * n,) and n > 0, "decay_memory: pieces must be int32 [4 n]")
+            work = torch.empty((n, H, d * dv), dtype=torch.float32, device=q.device)
+            decay = torch.empty((n, H), dtype=torch.float32, device=q.device)
+        L, I = ctypes.c_longlong, ctypes.c_int
+        at = lambda t: ctypes.c_void_p(0 if t is None else t.data_ptr())
+        hip().call("spy_decay_memory", _ptr(out), at(q), L(qs), at(k), L(ks), at(v), L(vs), at(gate), L(gs), _code(q, "q"), I(H), I(H // G), I(d),
+                   I(dv), ctypes.c_float(kscale), _ptr(log_decay), at(dt), L(dts), _ptr(dt_bias), _ptr(rate), _ptr(angles), I(half), _ptr(skip),
+                   ctypes.c_float(norm_eps or 0.0), I(epi), _ptr(state), L(state.shape[1]), _ptr(slot_ids), I(state.shape[0]), I(S), I(T),
+                   I(1 if single else 0), _ptr(parr), I(n), _ptr(work), _ptr(decay), _Hip.stream())
+    if norm_eps is None or fused:
+        return out
+    return group_norm(out, None, norm_eps, H, q.dtype, gate)
 
 
 # --------------------------------------------------------------------------
@@ -1678,22 +1928,25 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
     products being linear, it is multiplied into their sums, ahead of the activation).  ``add [T, K]``: added to the result
     in the pass that sums the choices (the result of a layer that every token uses).  ``align``: the pairs already sorted
     (``ids`` is not read then, and ``weights`` may be None: all one).  ``scale``: a factor on the sum over the choices.
-    ``unsummed``: the result is ``ExpertRows`` instead of [T, K]."""
+    ``unsummed``: the result is ``ExpertRows`` instead of [T, K].  ``activation`` "gelu": experts without a gate, ``w_gate_up
+    [E, F, K]`` = every expert's up rows, down_e(gelu(up_e x)), the exact gelu."""
     _dev(add)
     _check(add is None or (add.shape == x.shape and add.dtype == x.dtype and add.is_contiguous()), "moe_experts: the addend must be like x")
-    _check(activation in ("silu", "clamped") and (activation == "silu" or limit > 0.0), "moe_experts: activation silu, or clamped with a positive limit")
-    act_kind = 1 if activation == "clamped" else 0
+    _check(activation in ("silu", "clamped", "gelu") and (activation != "clamped" or limit > 0.0), "moe_experts: activation silu, gelu, or clamped with a positive limit")
+    act_kind = {"silu": 0, "clamped": 1, "gelu": ACT_GELU}[activation]
+    gated = activation != "gelu"
+    _check(gated or not weight_input, "moe_experts: experts without a gate take their weights at the output")
     _dev(x, ids, weights, w_gate_up, w_down)
     T, K = x.shape
     top = ids.shape[1] if align is None else align.top
     E, F2, _ = w_gate_up.shape
-    F = F2 // 2
+    F = F2 // 2 if gated else F2
     _check(x.dim() == 2 and (align is not None or (ids.dtype == torch.int32 and ids.shape == (T, top) and weights is not None))
            and (weights is None or (weights.dtype == torch.float32 and weights.shape == (T, top))),
            "moe_experts: experts int32 [T, top] and weights float32 [T, top] expected")
     _check(align is None or (align.T == T and align.experts == E), "moe_experts: the alignment is of another step or mixture")
     _check(weights is not None or not weight_input, "moe_experts: no weights for the experts' input")
-    _check(w_gate_up.dim() == 3 and w_gate_up.shape == (E, 2 * F, K) and tuple(w_down.shape) == (E, K, F) and w_down.dtype == w_gate_up.dtype,
+    _check(w_gate_up.dim() == 3 and w_gate_up.shape == (E, (2 if gated else 1) * F, K) and tuple(w_down.shape) == (E, K, F) and w_down.dtype == w_gate_up.dtype,
            "moe_experts: expert matrices [E, 2 F, K] and [E, K, F] of one dtype expected")
     if not T:
         return torch.empty((T, K), dtype=x.dtype, device=x.device)
@@ -1715,7 +1968,7 @@ def moe_experts(x: torch.Tensor, ids: Optional[torch.Tensor], weights: Optional[
     per_block = 0 if not MOE_MFMA or x.dtype != torch.bfloat16 or w_gate_up.dtype != torch.bfloat16 else (8 if P >= 16 * E else 1)
     act = torch.empty((max_tiles * tm, F), dtype=x.dtype, device=dev)
     hip().call("spy_moe_gemm", _ptr(act), _code(act, "act"), _ptr(x), _code(x, "x"), _ptr(w_gate_up), _code(w_gate_up, "expert matrices"),
-               _ptr(tile_expert), _ptr(sorted_pair), ctypes.c_int(top), ctypes.c_int(1), ctypes.c_int(max_tiles), ctypes.c_int(E), ctypes.c_int(F),
+               _ptr(tile_expert), _ptr(sorted_pair), ctypes.c_int(top), ctypes.c_int(1 if gated else 0), ctypes.c_int(max_tiles), ctypes.c_int(E), ctypes.c_int(F),
                ctypes.c_int(K), ctypes.c_int(per_block), ctypes.c_int(act_kind), ctypes.c_float(limit), _ptr(weights if weight_input else None), _Hip.stream())
     y = torch.empty((max_tiles * tm, K), dtype=torch.float32, device=dev)
     hip().call("spy_moe_gemm", _ptr(y), F32, _ptr(act), _code(act, "act"), _ptr(w_down), _code(w_down, "expert matrices"), _ptr(tile_expert),

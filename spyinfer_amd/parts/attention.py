@@ -19,7 +19,8 @@ root mean square per head before they are stored; scores capped by cap tanh(scor
 multiplied by a temperature that grows with the logarithm of the position; a penalty r1_h ln(1 + r2_h (i - j)) on the
 distance, taken off the (capped) score; a softmax whose denominator holds a one (a sink of score 0 without a value) or
 e^sink of a learned number per head; the gate as one number per head instead of one per value; values blended with those
-of an earlier layer of the same step before they are stored.
+of an earlier layer of the same step before they are stored; q and k normed per head beside angles formed in the kernel,
+chunks or a value size of its own (then without biases, gates and whatever else touches q, k and v on their way).
 """
 from __future__ import annotations
 
@@ -119,7 +120,8 @@ class PagedAttention(Mixer):
                  window: Optional[int] = None, scale: Optional[float] = None, fold_rows: Optional[int] = None,
                  value_dim: Optional[int] = None, bias: bool = False, gate: bool = False, names: Optional[dict] = None,
                  softcap: float = 0.0, value_norm_eps: Optional[float] = None, query_temperature=None, distance_penalty: bool = False,
-                 zero_sink: bool = False, chunk: Optional[int] = None, sink: bool = False, value_mix: Optional[str] = None):
+                 zero_sink: bool = False, chunk: Optional[int] = None, sink: bool = False, value_mix: Optional[str] = None,
+                 formed_angles: bool = False):
         """``fold_rows``: most rows of a step whose products here run with the norms and the residual sum folded in
         (None: ``ops.default_fold_rows`` of this part's matrices).  ``value_dim``: size of a value head (None: ``head_dim``).
         ``bias``: q, k and v have biases.  ``gate``: the heads' results are multiplied by sigmoid(Wg x) before the output
@@ -134,7 +136,10 @@ class PagedAttention(Mixer):
         head (tensor ``sink`` [heads]), p_j = e^(s_j) / (e^sink + sum e^(s_j)).  ``value_mix``: what is cached as values is
         (1 - lam) v + lam v_first, lam one learned number (tensor ``vmix`` without dimensions) and v_first the same tokens'
         values in the layer that says "first" (it caches its own; its tensor, if stored, is not read); the others, which run
-        later in the step and must have as many value heads of the same size, say "blend"."""
+        later in the step and must have as many value heads of the same size, say "blend".  ``formed_angles``: the rotation's
+        angles are formed in the kernel from the encoding's frequencies even where a table would do (an encoding of the
+        layer's own, no limit on positions)."""
+        self.formed_angles = bool(formed_angles)
         if num_heads % num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
         self.hidden_size, self.num_heads, self.num_kv_heads = hidden_size, num_heads, num_kv_heads
@@ -198,6 +203,9 @@ class PagedAttention(Mixer):
         # the matrices leave the caller's dictionary here, so that they are freed once they are fused: binding a
         # model never holds the separate matrices, the fused one and its tiled copy of all layers at once
         n, nq, nkv, dk, dv = self.names, self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
+        if self._head_norms():
+            if self.has_bias or self.has_gate or self.value_norm_eps is not None or self.query_temperature is not None or self.value_mix is not None:
+                raise ValueError("per-head norms of q and k beside biases, a gate, normed or blended values or a temperature are not implemented")
         mats = [weights.pop(prefix + n[c]) for c in "qkv"] + ([weights.pop(prefix + n["g"])] if self.has_gate else [])
         if len({m.dtype for m in mats}) > 1:
             mats = [m.float() for m in mats]
@@ -207,7 +215,9 @@ class PagedAttention(Mixer):
             gate_rows = torch.cat([mats[3], torch.zeros((fill, mats[3].shape[1]), dtype=mats[3].dtype, device=mats[3].device)]) if fill else mats[3]
             mats = [self._padded(m, heads, size) for m, heads, size in zip(mats[:3], (nq, nkv, nkv), (dk, dk, dv))] + [gate_rows]
         else:
-            mats = [self._padded(m, heads, size) for m, heads, size in zip(mats, (nq, nkv, nkv, nq), (dk, dk, dv, dv))]
+            # (heads that are normed by themselves are read as they are and padded where they are stored)
+            if not self._head_norms():
+                mats = [self._padded(m, heads, size) for m, heads, size in zip(mats, (nq, nkv, nkv, nq), (dk, dk, dv, dv))]
         # one product for q, k and v (and the gate): rows [q heads | k heads | v heads | gate]
         self.w_qkv = torch.cat(mats, dim=0).contiguous()
         del mats
@@ -232,8 +242,8 @@ class PagedAttention(Mixer):
         if self.value_mix == "blend":
             self.mix_lambda = float(weights[prefix + n["vmix"]])
         if self.qk_norm_eps is not None:
-            if dk != self.head_dim:
-                raise ValueError("per-head norms of q and k with a value size other than the key size are not implemented")
+            if dk != self.head_dim and not self._head_norms():
+                raise ValueError("per-head norms of q and k with a value size other than the key size need angles formed in the kernel")
             self.q_norm, self.k_norm = weights[prefix + n["q_norm"]], weights[prefix + n["k_norm"]]
             if self.q_norm.dtype != self.k_norm.dtype:
                 self.q_norm, self.k_norm = self.q_norm.float(), self.k_norm.float()
@@ -267,8 +277,12 @@ class PagedAttention(Mixer):
         encoding with rescaled frequencies has no table) and stores."""
         return not (self.has_bias or self.has_gate or self.softcap or self.value_norm_eps is not None
                     or self.query_temperature is not None or self.has_distance or self.zero_sink or self.has_sink
-                    or self.chunk is not None or self.value_mix is not None
+                    or self.chunk is not None or self.value_mix is not None or self.formed_angles
                     or (self.position is not None and getattr(self.position, "scaling", None) is not None))
+
+    def _head_norms(self) -> bool:
+        """q and k are normed per head in the kernel that forms the angles (not by the plain arrangement's)."""
+        return self.qk_norm_eps is not None and not self._plain_projections()
 
     def _rotated_whole(self) -> bool:
         """The head is rotated whole or not at all, and the group is one tile: what the fused kernel takes."""
@@ -276,6 +290,9 @@ class PagedAttention(Mixer):
             return False
         rot = self.position.rotary() if self.position is not None else None
         return (rot is None or rot[2] in (0, self.head_dim)) and self.num_heads // self.num_kv_heads <= 16
+
+    def _pairs_interleaved(self) -> bool:
+        return self.position is not None and getattr(self.position, "interleaved", False)
 
     def _big_rows(self, batch, page_size: int) -> int:
         """Rows of the tiles for this step's entries with many rows; 0 if the prefill kernel does not take this head
@@ -314,12 +331,17 @@ class PagedAttention(Mixer):
         if not self._plain_projections():
             # biases, rotation and store in one kernel that reads q, k and v out of the wider product; the gate's rows,
             # which lie behind them, are multiplied into the heads' results
-            if self.qk_norm_eps is not None:
-                raise ValueError("per-head norms of q and k beside biases, a gate or rescaled frequencies are not implemented")
             freq, mag, rdim = None, 1.0, 0
             if self.position is not None:
                 freq, mag, rdim = self.position.frequencies()
             slots = batch.slot_mapping(cache.group) if store else None
+            if self._head_norms():
+                if mag != 1.0:
+                    raise ValueError("per-head norms of q and k beside a rotation with a factor on cos and sin are not implemented")
+                q = ops.norm_rope_store(qkv, nq, nkv, self.key_dim, self.value_dim, d, self.q_norm, self.k_norm, self.qk_norm_eps, freq, rdim,
+                                        batch.positions, cache.k, cache.v, cache.page_size, slots, interleaved=self._pairs_interleaved())
+                return ops.paged_attention(q, cache.k, cache.v, cache.page_size, meta, nq, nkv, d, self.scale, self.window, softcap=self.softcap,
+                                           distance=self.distance, sink=self.sink, chunk=self.chunk)
             vnorm = None if self.value_norm_eps is None else (self.value_norm_eps, self.value_dim)
             mix = None
             if self.value_mix is not None:

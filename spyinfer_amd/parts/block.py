@@ -192,21 +192,25 @@ class DepthMix(Part):
 
 class OutputNormBlock(Block):
     """h += norm1(mixer(h)); h += norm2(ffn(h)): the norm sits on a sublayer's OUTPUT, the sublayers read the stream
-    itself.  ``ffn`` (with ``norm2``) may be absent.  ``depth``: a ``DepthMix`` after the layer."""
+    itself.  ``ffn`` (with ``norm2``) may be absent.  ``depth``: a ``DepthMix`` after the layer.  A norm that says
+    ``takes_unsummed`` gets the results of parts that can hand them over so (``forward_unsummed``: a mixture's experts, two
+    mixers side by side) as they are and sums them in its pass.  ``unread``: as ``PreNormBlock``."""
 
     def __init__(self, mixer: Mixer, norm1: Norm, ffn: FeedForward = None, norm2: Norm = None, depth: "DepthMix" = None,
-                 names=("mix", "norm1", "mlp", "norm2", "dwa")):
+                 names=("mix", "norm1", "mlp", "norm2", "dwa"), unread=()):
         if (ffn is None) != (norm2 is None):
             raise ValueError("a feed-forward and its norm come together")
         self.mixer, self.norm1, self.ffn, self.norm2, self.depth = mixer, norm1, ffn, norm2, depth
         self.names = names
+        self.unread = tuple(unread)
 
     def _parts(self, prefix):
         parts = zip((self.mixer, self.norm1, self.ffn, self.norm2, self.depth), (prefix + "." + n for n in self.names))
         return [(part, p) for part, p in parts if part is not None]
 
     def weight_specs(self, prefix):
-        return [s for part, p in self._parts(prefix) for s in part.weight_specs(p)]
+        return [s for part, p in self._parts(prefix) for s in part.weight_specs(p)] \
+            + [WeightSpec(prefix + "." + u.name, u.shape, u.role, optional=True) for u in self.unread]
 
     def bind(self, prefix, weights):
         for part, p in self._parts(prefix):
@@ -214,6 +218,12 @@ class OutputNormBlock(Block):
 
     def capturable(self, batch):
         return all(part.capturable(batch) for part, _ in self._parts(""))
+
+    @staticmethod
+    def _run(part, norm):
+        """The part's ``forward``, or the one that leaves the sum of its results to the norm."""
+        unsummed = getattr(norm, "takes_unsummed", False) and hasattr(part, "forward_unsummed")
+        return part.forward_unsummed if unsummed else part.forward
 
     def forward(self, resid, pending, batch, cache, store=True, next_norm=None):
         act = batch.act_dtype
@@ -224,14 +234,14 @@ class OutputNormBlock(Block):
             for addend in (pending if isinstance(pending, (tuple, list)) else (pending,)):
                 resid.add_((addend.resolve() if isinstance(addend, (ops.GatedAddend, ops.NormedAddend)) else addend).float())         # a block of another arrangement left an addend (or a pair of them)
         x = stream_copy(batch, resid)
-        y = self.mixer.forward(x, batch, cache, store)
+        y = self._run(self.mixer, self.norm1)(x, batch, cache, store)
         out = self.depth.result_slot(batch, resid) if self.depth is not None else resid
         mix = self.depth.operands(batch) if self.depth is not None else None       # formed by the layer's last norm kernel
         last = self.ffn is None
         out, copy = self.norm1.add_normed(resid, y, out, act, mix if last else None)
         if not last:
             x = stream_copy(batch, out, copy)
-            f = self.ffn.forward(x, batch)
+            f = self._run(self.ffn, self.norm2)(x, batch)
             out, copy = self.norm2.add_normed(out, f, out, act, mix)
         stream_copy(batch, out, copy)
         return out, None

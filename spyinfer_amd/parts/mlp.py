@@ -66,36 +66,45 @@ class GatedMLP(FeedForward):
 
 
 class DenseMLP(FeedForward):
-    """down( act(up(x)) ), no gate and no biases.  ``activation`` "xielu": a piecewise activation with two learned
+    """down( act(up(x)) ), no gate and no biases.  ``activation`` "gelu": the exact form, z/2 (1 + erf(z / sqrt 2)).  "xielu": a piecewise activation with two learned
     numbers (p, q) in a tensor of its own: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z/2."""
 
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "xielu", names=("up", "down", "act")):
-        if activation != "xielu":
+        if activation not in ("xielu", "gelu"):
             raise ValueError("DenseMLP: activation %r is not implemented" % activation)
+        self.activation = activation
         self.hidden_size, self.intermediate_size, self.names = hidden_size, intermediate_size, names
         self.w_up = self.w_up_tiled = self.w_down = self.w_down_tiled = self.act = None
 
     def weight_specs(self, prefix):
         H, I = self.hidden_size, self.intermediate_size
-        up, down, act = (prefix + "." + n for n in self.names)
-        return [WeightSpec(up, (I, H)), WeightSpec(down, (H, I)), WeightSpec(act, (2,), "bias")]
+        up, down = (prefix + "." + n for n in self.names[:2])
+        return [WeightSpec(up, (I, H)), WeightSpec(down, (H, I))] \
+            + ([WeightSpec(prefix + "." + self.names[2], (2,), "bias")] if self.activation == "xielu" else [])
 
     def bind(self, prefix, weights):
-        up, down, act = (prefix + "." + n for n in self.names)
+        up, down = (prefix + "." + n for n in self.names[:2])
         self.w_up, self.w_up_tiled = ops.weight_forms(weights.pop(up))
         self.w_down, self.w_down_tiled = ops.weight_forms(weights.pop(down))
-        self.act = weights[act]
+        self.act = weights[prefix + "." + self.names[2]] if self.activation == "xielu" else None
 
     def capturable(self, batch):
         return True
 
     def forward(self, x, batch):
+        if self.activation == "gelu":
+            return ops.linear_few(ops.linear_gelu(x, self.w_up, tiled=self.w_up_tiled), self.w_down, self.w_down_tiled)
         return ops.linear_few(ops.linear_xielu(x, self.w_up, self.act, tiled=self.w_up_tiled), self.w_down, self.w_down_tiled)
 
 
 def stacked_experts(weights, experts: int, gate: str, up: str, down: str):
     """Takes the experts' matrices out of ``weights`` (names with a place for the expert's number): every expert's [gate rows |
-    up rows] and its down matrix, the experts one after the other."""
+    up rows] (``gate`` None: up rows alone) and its down matrix, the experts one after the other."""
+    if gate is None:
+        mats = [weights.pop(n % e) for e in range(experts) for n in (up, down)]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        return torch.stack(mats[0::2]).contiguous(), torch.stack(mats[1::2]).contiguous()
     mats = [weights.pop(n % e) for e in range(experts) for n in (gate, up, down)]
     if len({m.dtype for m in mats}) > 1:
         mats = [m.float() for m in mats]
@@ -117,13 +126,13 @@ class MoEMLP(FeedForward):
         """``score``: "softmax" over all experts or "sigmoid" of each logit.  ``renormalize``: the chosen scores over their
         sum (else as they are), times ``scale``.  ``correction``: a stored vector is added to the scores for the choice.
         ``weight_on``: "output": out = sum w expert(x); "input": out = sum expert(w x).  ``activation``: "silu":
-        silu(gate) * up; "clamped": g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+        silu(gate) * up; "gelu": experts without a gate (no tensors ``e<i>.gate``), gelu(up), the exact form; "clamped": g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
         ``router_bias``: the logits are W_r x + b (tensor ``router.b``); with softmax scores, renormalised, the weights are
         then the softmax over the chosen biased logits alone.  ``shared``: a feed-forward that every token uses (tensors
         under ``shared``), added to the experts' sum in the pass that forms it."""
         self.has_router_bias, self.shared, self.more_names = bool(router_bias), shared, more_names
         self.router_bias = None
-        if score not in ("softmax", "sigmoid") or weight_on not in ("output", "input") or activation not in ("silu", "clamped"):
+        if score not in ("softmax", "sigmoid") or weight_on not in ("output", "input") or activation not in ("silu", "clamped", "gelu"):
             raise ValueError("MoEMLP: score %r, weight_on %r or activation %r is not implemented" % (score, weight_on, activation))
         if activation == "clamped" and not limit > 0.0:
             raise ValueError("MoEMLP: the clamped activation needs a positive limit")
@@ -140,7 +149,7 @@ class MoEMLP(FeedForward):
         router, corr, gate, up, down = (prefix + "." + n for n in self.names)
         specs = [WeightSpec(router, (E, H))] + ([WeightSpec(corr, (E,), "bias")] if self.has_correction else [])
         for e in range(E):
-            specs += [WeightSpec(gate % e, (F, H)), WeightSpec(up % e, (F, H)), WeightSpec(down % e, (H, F))]
+            specs += ([WeightSpec(gate % e, (F, H))] if self.activation != "gelu" else []) + [WeightSpec(up % e, (F, H)), WeightSpec(down % e, (H, F))]
         if self.has_router_bias:
             specs.append(WeightSpec(prefix + "." + self.more_names[0], (E,), "bias"))
         if self.shared is not None:
@@ -156,18 +165,25 @@ class MoEMLP(FeedForward):
         self.router_bias = weights[prefix + "." + self.more_names[0]].float().contiguous() if self.has_router_bias else None
         if self.shared is not None:
             self.shared.bind(prefix + "." + self.more_names[1], weights)
-        self.w_gate_up, self.w_down = stacked_experts(weights, self.experts, gate, up, down)
+        self.w_gate_up, self.w_down = stacked_experts(weights, self.experts, gate if self.activation != "gelu" else None, up, down)
 
     def capturable(self, batch):
         return self.shared is None or self.shared.capturable(batch)
 
     def forward(self, x, batch):
+        return self._run(x, batch, {})
+
+    def forward_unsummed(self, x, batch):
+        """The result as ``ops.ExpertRows``, for a reader that sums it in its own pass."""
+        return self._run(x, batch, dict(unsummed=True))
+
+    def _run(self, x, batch, how):
         z = ops.linear(x, self.w_router, torch.float32)
         ids, weights = ops.moe_route(z, self.correction, self.top, self.groups, self.groups_kept, self.scale, score=self.score,
                                      renormalize=self.renormalize, logit_bias=self.router_bias)
         everyone = self.shared.forward(x, batch) if self.shared is not None else None
         return ops.moe_experts(x, ids, weights, self.w_gate_up, self.w_down, activation=self.activation, limit=self.limit,
-                               weight_input=self.weight_on == "input", add=everyone)
+                               weight_input=self.weight_on == "input", add=everyone, **how)
 
 
 class TableMoEMLP(FeedForward):

@@ -1,6 +1,6 @@
-"""RMS norm.  y = x / sqrt(mean(x^2) + eps) * w, sums and scale in float32, eps inside the
+"""RMS norm and layer norm.  RMS norm: y = x / sqrt(mean(x^2) + eps) * w, sums and scale in float32, eps inside the
 root, the weight multiplies as it is (src/backends/cpu/x64/kernels.cpp:168-180;
-src/backends/cuda/native/common.cuh:57-188)."""
+src/backends/cuda/native/common.cuh:57-188).  Layer norm (the reference has none): y = (x - mean) / sqrt(var + eps) * w + b."""
 from __future__ import annotations
 
 import torch
@@ -96,3 +96,46 @@ class RMSNorm(Norm):
         if self.groups == 1 and not self.scalar and out_dtype == torch.bfloat16 and self.weight is not None and self.weight.dtype == torch.bfloat16:
             return self.weight, self.eps
         return None
+
+
+class LayerNorm(Norm):
+    """y = (x - mean) / sqrt(var + eps) * w + b, var the mean of the squared deviations; float32 inside.  Tensors: the weight
+    under the prefix (and ``suffix``), the bias under the same name with ``bias_suffix`` behind it."""
+
+    takes_unsummed = True          # ``add_normed`` sums a mixture's experts or a weighted pair of results in its own pass
+
+    def __init__(self, size: int, eps: float, suffix: str = "", bias_suffix: str = ".b"):
+        self.size, self.eps, self.suffix, self.bias_suffix = size, float(eps), suffix, bias_suffix
+        self.weight = self.bias = None
+
+    def weight_specs(self, prefix):
+        name = prefix + self.suffix
+        return [WeightSpec(name, (self.size,), "norm"), WeightSpec(name + self.bias_suffix, (self.size,), "bias")]
+
+    def bind(self, prefix, weights):
+        name = prefix + self.suffix
+        self.weight, self.bias = weights[name], weights[name + self.bias_suffix]
+        if self.weight.dtype != self.bias.dtype:
+            self.weight, self.bias = self.weight.float(), self.bias.float()
+
+    def capturable(self, batch):
+        return True
+
+    def add_norm(self, resid, delta, out_dtype, rows=None):
+        """The norm of the stream (at ``rows`` only, if given); ``delta`` (whatever a block may leave pending) is summed into
+        it first."""
+        if delta is not None and not isinstance(delta, ops.ScaledInput):
+            if rows is not None:
+                resid = resid.clone()                     # (picked rows: the stream stays as it is)
+            if isinstance(delta, ops.EntryAddends):
+                delta.resolve(resid)
+            else:
+                for d in (delta if isinstance(delta, (tuple, list)) else (delta,)):
+                    resid.add_((d.resolve() if hasattr(d, "resolve") else d).float())
+        return ops.layer_norm(resid, self.weight, self.bias, self.eps, out_dtype, rows)
+
+    def add_normed(self, base, y, out=None, copy_dtype=None, mix=None):
+        """out = base + norm(y) in float32; ``y``: rows, ``ops.ExpertRows`` or ``ops.WeightedPair``.  Returns (out, copy)."""
+        if mix is not None:
+            raise ValueError("a layer norm whose result is mixed with kept layer results is not implemented")
+        return ops.layer_norm_residual(base, y, self.weight, self.bias, self.eps, out, copy_dtype)

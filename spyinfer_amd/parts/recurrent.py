@@ -24,6 +24,14 @@ S = diag(w) S + k v^T.  Every projection reads its own blend of the token's inpu
 x + (x' - x) mu (x' = 0 for a request's first token); w = exp(-exp(W2 tanh(W1 blend_w) + w0)); each head's o over its
 root mean square, times a weight, times silu(Wg blend_g), then the output projection.  The input of a request's last
 token is state of the request too.
+
+``Retention`` and ``StateSpace`` have one decay per head and token: S = a S + b k v^T, o = S^T q.  ``Retention``: a is a
+constant of the head and b = 1; q and k are rotated by their position, k times 1/sqrt(key size); each head's o over its root
+mean square (no weight), times silu(Wg x), then the output projection.  ``StateSpace``: v, k and q (x, B and C of a
+state-space model) pass a short causal convolution per channel with a bias and silu, k and q shared by the heads of a group;
+dt = softplus(Wdt x + bias_h), a = exp(-exp(A_h) dt), b = dt; (o + D_h v) silu(z), z projected too, over its root mean square
+in equal groups of channels, times a weight, then the output projection.  The convolution's last inputs are state of the
+request.  Entries of several tokens run in pieces, whose products go through the matrix cores in float32.
 """
 from __future__ import annotations
 
@@ -374,3 +382,148 @@ class TimeMix(Mixer):
         dec_pre = ops.linear(inner, self.w_2, torch.float32)
         y = ops.time_mix(r, k, v, dec_pre, self.w0, self.u, g, self.norm, self.norm_eps, cache.state, cu_q, slots, H, d)
         return ops.linear_few(y, self.w_o[0], self.w_o[1])
+
+
+def _whole_quads(n: int) -> int:
+    return -(-n // 4) * 4          # a slot's values in whole 16-byte pieces
+
+
+def plan_decay_pieces(batch) -> None:
+    """The pieces of a step's entries for ``ops.decay_memory``, where there is an entry of more than one token."""
+    if batch.T != batch.S:
+        plan_scan_pieces(batch, ops.DECAY_PIECE)
+
+
+def decay_pieces(batch):
+    if batch.T == batch.S:
+        return None
+    name = scan_pieces_name(ops.DECAY_PIECE)
+    return (batch.array(name),) + batch.shared[name]
+
+
+def step_angles(batch, position):
+    """Cosines and sines of the step's positions for an encoding's frequencies, once for all layers of that rotation."""
+    freq, mag, dims = position.frequencies()
+    if mag != 1.0:
+        raise ValueError("a rotation with a factor on cos and sin is not implemented here")
+    note = ("rotation_angles", position.theta, dims, id(position) if position.scaling is not None else 0)
+    if note not in batch.shared:
+        batch.shared[note] = ops.rotation_angles(batch.positions, freq)
+    return batch.shared[note]
+
+
+class Retention(Mixer):
+    """Tensors: ``q``, ``k`` [heads dim, H], ``v``, ``g`` [heads vdim, H], ``o`` [H, heads vdim].  ``decay``: one number per head.
+    ``position``: a rotary encoding with pairs (i, i + dims / 2) (None: no rotation)."""
+
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, decay, position, norm_eps: float, names=("q", "k", "v", "g", "o")):
+        if len(decay) != heads or not all(0.0 < float(x) <= 1.0 for x in decay):
+            raise ValueError("one decay above 0 and up to 1 per head")
+        if position is not None and position.interleaved:
+            raise ValueError("interleaved pairs are not implemented here")
+        self.hidden_size, self.heads, self.dim, self.vdim, self.norm_eps, self.names = hidden_size, heads, dim, vdim, float(norm_eps), names
+        self.decay, self.position = [float(x) for x in decay], position
+        self.w_in = self.w_in_tiled = self.w_o = self.w_o_tiled = self.log_decay = None
+
+    def weight_specs(self, prefix):
+        W, H, d, dv = self.hidden_size, self.heads, self.dim, self.vdim
+        q, k, v, g, o = (prefix + "." + n for n in self.names)
+        return [WeightSpec(q, (H * d, W)), WeightSpec(k, (H * d, W)), WeightSpec(v, (H * dv, W)), WeightSpec(g, (H * dv, W)), WeightSpec(o, (W, H * dv))]
+
+    def bind(self, prefix, weights):
+        q, k, v, g, o = (prefix + "." + n for n in self.names)
+        mats = [weights.pop(n) for n in (q, k, v, g)]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        # one product for the four projections: rows [q | k | v | g]
+        self.w_in, self.w_in_tiled = ops.weight_forms(torch.cat(mats, dim=0).contiguous())
+        del mats
+        self.w_o, self.w_o_tiled = ops.weight_forms(weights.pop(o))
+        self.log_decay = torch.log(torch.tensor(self.decay, dtype=torch.float64)).to(torch.float32).to(self.w_o.device)
+        if self.position is not None:
+            self.position.prepare(self.w_o.device, 0)
+
+    def cache_spec(self):
+        return FixedState((_whole_quads(self.heads * self.dim * self.vdim),), "float32")
+
+    def plan(self, batch) -> None:
+        plan_decay_pieces(batch)
+
+    def capturable(self, batch):
+        return True
+
+    def forward(self, x, batch, cache, store=True):
+        if not store:
+            raise ValueError("a recurrence cannot run on another layer's state without writing it")
+        H, d, dv = self.heads, self.dim, self.vdim
+        proj = ops.linear_few(x, self.w_in, self.w_in_tiled)
+        n, m = H * d, H * dv
+        y = ops.decay_memory(proj[:, :n], proj[:, n:2 * n], proj[:, 2 * n:2 * n + m], H, H, d, dv, cache.state, batch.array("cu_q"),
+                             batch.array("slot_ids"), decay_pieces(batch), kscale=d ** -0.5, log_decay=self.log_decay,
+                             angles=step_angles(batch, self.position) if self.position is not None else None,
+                             gate=proj[:, 2 * n + m:], norm_eps=self.norm_eps)
+        return ops.linear_few(y, self.w_o, self.w_o_tiled)
+
+
+class StateSpace(Mixer):
+    """Tensors: ``in`` [2 heads vdim + 2 groups state + heads, H] with rows [z | x | B | C | dt], ``conv`` [channels, taps] and
+    ``conv.b`` over the channels [x | B | C], ``dt_bias``, ``A_log``, ``D`` [heads], ``norm`` [heads vdim], ``o``."""
+
+    def __init__(self, hidden_size: int, heads: int, vdim: int, state: int, groups: int, conv: int, norm_groups: int, norm_eps: float,
+                 names=("in", "conv", "conv.b", "dt_bias", "A_log", "D", "norm", "o")):
+        if heads % groups or (heads * vdim) % norm_groups:
+            raise ValueError("groups must divide the heads, norm_groups the heads' values together")
+        if not 1 <= conv <= 8:
+            raise ValueError("the short convolution has 1 to 8 taps")
+        self.hidden_size, self.heads, self.vdim, self.state, self.groups, self.conv = hidden_size, heads, vdim, state, groups, conv
+        self.norm_groups, self.norm_eps, self.names = norm_groups, float(norm_eps), names
+        self.w_in = self.w_in_tiled = self.w_dt = self.w_o = self.w_o_tiled = None
+        self.taps = self.conv_bias = self.dt_bias = self.rate = self.skip = self.norm = None
+
+    def _channels(self):
+        return self.heads * self.vdim + 2 * self.groups * self.state
+
+    def weight_specs(self, prefix):
+        W, H, inner, C = self.hidden_size, self.heads, self.heads * self.vdim, self._channels()
+        win, conv, convb, dtb, alog, D, norm, o = (prefix + "." + n for n in self.names)
+        return [WeightSpec(win, (inner + C + H, W)), WeightSpec(conv, (C, self.conv), "bias"), WeightSpec(convb, (C,), "bias"), WeightSpec(dtb, (H,), "bias"),
+                WeightSpec(alog, (H,), "bias"), WeightSpec(D, (H,), "norm"), WeightSpec(norm, (inner,), "norm"), WeightSpec(o, (W, inner))]
+
+    def bind(self, prefix, weights):
+        inner, C = self.heads * self.vdim, self._channels()
+        win, conv, convb, dtb, alog, D, norm, o = (prefix + "." + n for n in self.names)
+        w = weights.pop(win)
+        # rows [z | x | B | C] in one product; the step sizes, which enter the recurrence's exponentials, come from a second,
+        # small product that stays float32
+        self.w_in, self.w_in_tiled = ops.weight_forms(w[:inner + C].contiguous())
+        self.w_dt = w[inner + C:].contiguous()
+        del w
+        self.w_o, self.w_o_tiled = ops.weight_forms(weights.pop(o))
+        self.taps, self.conv_bias = weights[conv], weights[convb]
+        if self.taps.dtype != self.conv_bias.dtype:
+            self.taps, self.conv_bias = self.taps.float(), self.conv_bias.float()
+        self.norm = weights[norm]
+        self.dt_bias, self.skip = weights[dtb].float().contiguous(), weights[D].float().contiguous()
+        self.rate = torch.exp(weights[alog].float()).contiguous()
+
+    def cache_spec(self):
+        return FixedState((_whole_quads(self.heads * self.state * self.vdim + (self.conv - 1) * self._channels()),), "float32")
+
+    def plan(self, batch) -> None:
+        plan_decay_pieces(batch)
+
+    def capturable(self, batch):
+        return True
+
+    def forward(self, x, batch, cache, store=True):
+        if not store:
+            raise ValueError("a recurrence cannot run on another layer's state without writing it")
+        H, G, N, dv = self.heads, self.groups, self.state, self.vdim
+        inner = H * dv
+        proj = ops.linear_few(x, self.w_in, self.w_in_tiled)
+        dt = ops.linear(x, self.w_dt, torch.float32)
+        cu_q, slots = batch.array("cu_q"), batch.array("slot_ids")
+        xbc = ops.causal_conv_silu(proj[:, inner:], self.taps, cache.state, H * N * dv, batch.array("token_entry"), cu_q, slots, bias=self.conv_bias)
+        o = ops.decay_memory(xbc[:, inner + G * N:], xbc[:, inner:inner + G * N], xbc[:, :inner], H, G, N, dv, cache.state, cu_q, slots,
+                             decay_pieces(batch), steps=(dt, self.dt_bias, self.rate), gate=proj[:, :inner], skip=self.skip)
+        return ops.linear_few(ops.group_norm(o, self.norm, self.norm_eps, self.norm_groups, x.dtype), self.w_o, self.w_o_tiled)

@@ -24,7 +24,7 @@ def emu_ops(monkeypatch):
     for name in ("embedding", "add_rms_norm", "rms_norm", "qk_norm_rope_store", "swiglu", "sample", "pair_embedding", "norm_residual",
                  "depth_mix", "xielu", "mingru", "gemm_strided", "latent_prepare", "latent_attention", "bias_rope_store", "sigmoid_gate",
                  "mlstm", "causal_conv_silu", "delta_rule", "moe_route", "moe_experts", "token_shift", "tanh_cast", "time_mix", "norm_pair_mean", "scale_cap",
-                 "result_norm"):
+                 "result_norm", "layer_norm", "layer_norm_residual", "norm_rope_store", "map_difference", "rotation_angles", "group_norm", "decay_memory"):
         monkeypatch.setattr(ops, name, getattr(emu, name))
 
     def linear(x, w, out_dtype=None, tiled=None, out=None):
@@ -33,6 +33,7 @@ def emu_ops(monkeypatch):
     monkeypatch.setattr(ops, "linear", linear)
     monkeypatch.setattr(ops, "linear_few", lambda x, w, tiled=None, out_dtype=None, out=None: linear(x, w, out_dtype, out=out))
     monkeypatch.setattr(ops, "linear_xielu", lambda x, w, pq, tiled=None: emu.xielu(emu.linear(x, w), pq))
+    monkeypatch.setattr(ops, "linear_gelu", lambda x, w, tiled=None: torch.nn.functional.gelu(emu.linear(x, w)))
     monkeypatch.setattr(ops, "linear_swiglu", lambda x, w, tiled=None, few_rows=0, activation="silu": emu.swiglu(emu.linear(x, w), activation))
     monkeypatch.setattr(ops.ExpertTables, "align", lambda self, token_ids: emu.align_tables(self, token_ids))
     monkeypatch.setattr(ops, "paged_attention", lambda q, k_cache, v_cache, page_size, meta, n_q, n_kv, d, scale, window, raw=None,

@@ -330,7 +330,7 @@ class EmuOps:
         g = f[:, g_off:g_off + H * dv]
         return (out.reshape(T, H * dv) * norm_w.float() * torch.sigmoid(g)).to(x.dtype)
 
-    def causal_conv_silu(self, x, taps, state, keep_off, token_entry, cu_q, slot_ids):
+    def causal_conv_silu(self, x, taps, state, keep_off, token_entry, cu_q, slot_ids, bias=None):
         T, C = x.shape
         n = taps.shape[1]
         f = x.float()
@@ -341,6 +341,8 @@ class EmuOps:
             rows = torch.cat([keep.clone(), f[t0:t1]], dim=0)
             for t in range(t1 - t0):
                 acc = (rows[t:t + n] * taps.float().T).sum(0)
+                if bias is not None:
+                    acc = acc + bias.float()
                 y[t0 + t] = acc * torch.sigmoid(acc)
             if n > 1:
                 keep.copy_(rows[rows.shape[0] - (n - 1):])
@@ -442,13 +444,17 @@ class EmuOps:
         F = w_gate_up.shape[1] // 2
         out = torch.zeros((T, K), dtype=torch.float32)
         xf = x.float()
+        if activation == "gelu":
+            assert not weight_input
         for t in range(T):
             for j in range(ids.shape[1]):
                 e = int(ids[t, j])
                 gu = w_gate_up[e].float() @ xf[t]
                 if weight_input:
                     gu = gu * weights[t, j]
-                if activation == "silu":
+                if activation == "gelu":
+                    act = torch.nn.functional.gelu(gu)
+                elif activation == "silu":
                     act = gu[:F] * torch.sigmoid(gu[:F]) * gu[F:]
                 else:
                     g, u = torch.clamp(gu[:F], max=limit), torch.clamp(gu[F:], -limit, limit)
@@ -462,3 +468,91 @@ class EmuOps:
 
     def align_tables(self, tables, token_ids):
         return [t[token_ids.long()] for t in tables.tables]
+
+    # ---- layer norms, heads normed ahead of the rotation, differences of maps, states with one decay per head ----
+    def layer_norm_residual(self, base, y, weight, bias, eps, out=None, copy_dtype=None):
+        yf = (y.resolve() if hasattr(y, "resolve") else y).float()
+        c = yf - yf.mean(-1, keepdim=True)
+        r = base + c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * weight.float() + bias.float()
+        out = r if out is None else out.copy_(r)
+        return out, self._copy(out, copy_dtype)
+
+    def layer_norm(self, x, weight, bias, eps, out_dtype, rows=None):
+        x = x if rows is None else x[rows.long()]
+        c = x - x.mean(-1, keepdim=True)
+        return (c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * weight.float() + bias.float()).to(out_dtype)
+
+    def norm_rope_store(self, x, n_q, n_kv, dim, value_dim, d, q_norm_w, k_norm_w, eps, freq, rotary_dim, positions, k_cache, v_cache, page_size,
+                        slots, maps=1, interleaved=False, columns=None):
+        T = x.shape[0]
+        assert columns is None
+        f = x.float()
+
+        def heads(first, n, w):
+            h = f[:, first:first + n * maps * dim].reshape(T, n, maps, dim)
+            h = h * torch.rsqrt((h * h).mean(-1, keepdim=True) + eps) * w.float()
+            return self._rotate(h, positions, freq, 1.0, rotary_dim, interleaved)
+        q = torch.zeros((T, n_q, maps, d))
+        qh = heads(0, n_q, q_norm_w)
+        for m in range(maps):
+            q[:, :, m, m * dim:(m + 1) * dim] = qh[:, :, m]
+        if slots is not None:
+            k, v = torch.zeros((T, n_kv, d)), torch.zeros((T, n_kv, d))
+            k[:, :, :maps * dim] = heads(n_q * maps * dim, n_kv, k_norm_w).reshape(T, n_kv, maps * dim)
+            first = (n_q + n_kv) * maps * dim
+            v[:, :, :value_dim] = f[:, first:first + n_kv * value_dim].reshape(T, n_kv, value_dim)
+            for t in range(T):
+                sl = int(slots[t])
+                k_cache[sl // page_size, :, sl % page_size, :] = k[t].to(k_cache.dtype)
+                v_cache[sl // page_size, :, :, sl % page_size] = v[t].to(v_cache.dtype)
+        return q.reshape(T, n_q * maps * d).to(x.dtype)
+
+    def map_difference(self, x, heads, value_dim, d, lam, eps, mult, out_dtype=None):
+        a = x.float().reshape(x.shape[0], heads, 2, d)[..., :value_dim]
+        o = a[:, :, 0] - lam * a[:, :, 1]
+        o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps) * mult
+        return o.reshape(x.shape[0], heads * value_dim).to(out_dtype or x.dtype)
+
+    def rotation_angles(self, positions, freq):
+        ang = positions.float()[:, None] * freq[None, :]
+        return torch.stack([torch.cos(ang), torch.sin(ang)], dim=-1)
+
+    def group_norm(self, o, weight, eps, groups, out_dtype, gate=None):
+        y = o.reshape(o.shape[0], groups, -1)
+        y = (y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps)).reshape(o.shape)
+        if weight is not None:
+            y = y * weight.float()
+        return (y if gate is None else y * torch.nn.functional.silu(gate.float())).to(out_dtype)
+
+    def decay_memory(self, q, k, v, H, G, d, dv, state, cu_q, slot_ids, pieces, kscale=1.0, log_decay=None, steps=None, angles=None, gate=None,
+                     norm_eps=None, skip=None):
+        T = q.shape[0]
+        qf, kf = (t[:, :G * d].float().reshape(T, G, d) for t in (q, k))
+        vf = v[:, :H * dv].float().reshape(T, H, dv)
+        if angles is not None:
+            half = angles.shape[1]
+            c, s = angles[:, None, :, 0], angles[:, None, :, 1]
+            turn = lambda t: torch.cat([t[..., :half] * c - t[..., half:2 * half] * s, t[..., half:2 * half] * c + t[..., :half] * s, t[..., 2 * half:]], dim=-1)
+            qf, kf = turn(qf), turn(kf)
+        kf = kf * kscale
+        if steps is not None:
+            dt = torch.nn.functional.softplus(steps[0] + steps[1], threshold=1e9)
+            a, b = torch.exp(-steps[2] * dt), dt
+        else:
+            a, b = torch.exp(log_decay).expand(T, H), torch.ones((T, H))
+        out = torch.zeros((T, H, dv))
+        for e in range(slot_ids.shape[0]):
+            st = state[int(slot_ids[e]), :H * d * dv].view(H, d, dv)
+            S = st.clone()
+            for t in range(int(cu_q[e]), int(cu_q[e + 1])):
+                kh, qh = kf[t].repeat_interleave(H // G, 0), qf[t].repeat_interleave(H // G, 0)
+                S = a[t][:, None, None] * S + (b[t][:, None] * kh)[:, :, None] * vf[t][:, None, :]
+                out[t] = torch.einsum("hij,hi->hj", S, qh)
+            st.copy_(S)
+        silu = torch.nn.functional.silu
+        if norm_eps is not None:
+            out = out * torch.rsqrt((out * out).mean(-1, keepdim=True) + norm_eps)
+            return (out.reshape(T, H * dv) * silu(gate.float())).to(q.dtype)
+        if skip is not None:
+            return (out + skip[:, None] * vf).reshape(T, H * dv) * silu(gate.float())
+        return out.reshape(T, H * dv)
