@@ -26,6 +26,7 @@ Other workloads, each again one JSON line:
     python bench.py --design meronex [--design-sizes 1024,2048,4096] [--layers 9]   # Meronex beside Sodedra and Qwen3 at equal size
     python bench.py --design tarunex [--design-sizes 1024,2048,4096] [--layers 8]   # Tarunex beside Sodedra, Sefevik and Qwen3 at equal size
     python bench.py --design balelorn [--design-sizes 1024,2048,4096] [--layers 8]  # Balelorn beside Sodedra, Tarunex and Qwen3 at equal size
+    python bench.py --design nolatar [--design-sizes 1024,2048,4096] [--layers 8]   # Nolatar beside Meronex, Tarunex and Qwen3 at equal size
 """
 import argparse
 import json
@@ -154,10 +155,39 @@ def balelorn_shape(width: int, layers: int, vocab: int) -> dict:
     return dict(architecture="Balelorn", vocab=vocab, width=width, norm=dict(eps=1e-5), layers=out)
 
 
+def nolatar_shape(width: int, layers: int, vocab: int) -> dict:
+    """A Nolatar configuration with the layer sizes of a real model of that width: of every four layers a state space (inner
+    size twice the width, heads of 64, a state of 128, eight groups at most, 4 taps), a differential attention (width / 128
+    heads of two maps of 64 with values of 128, a quarter as many kv heads), an attention in chunks of 1536 positions (heads
+    of 128, a quarter as many kv heads) beside a retention (heads of 128 x 128), and a state space again; from the second
+    turn on the differential attention reads the first one's cache in every other turn; every feed-forward 32 experts
+    without gates of three quarters of the width of which a token uses four, plus one of one and a half times the width for
+    everyone (as many active weights as a dense gated layer of three times the width)."""
+    heads = max(1, width // 128)
+    kv = max(1, heads // 4)
+    rot = lambda base, dims: dict(base=base, dims=dims)
+    moe = dict(kind="moe", expert=dict(ff=3 * width // 4), router=dict(experts=32, top=4), shared=dict(ff=3 * width // 2))
+    mamba = dict(heads=2 * width // 64, vdim=64, state=128, groups=min(8, heads), conv=4, norm_groups=min(8, heads))
+    diff = dict(heads=heads, kv_heads=kv, dim=64, vdim=128, scale=64 ** -0.5, diff=0.3, rot=rot(500000.0, 64))
+    both = dict(left=dict(heads=heads, kv_heads=kv, dim=128, vdim=128, scale=128 ** -0.5, mask=dict(size=1536), rot=rot(10000.0, 128)),
+                right=dict(heads=heads, dim=128, vdim=128, decay=[1.0 - 2.0 ** (-5 - 5.0 * h / heads) for h in range(heads)], rot=rot(10000.0, 128)),
+                left_scale=0.6, right_scale=0.5)
+    out = []
+    for i in range(layers):
+        if i % 4 == 1:
+            out.append(dict(type="attention", mixer=dict(diff, kv_from=i - 4) if i % 8 == 5 else dict(diff), mlp=moe))
+        elif i % 4 == 2:
+            out.append(dict(type="parallel", mixer=dict(both), mlp=moe))
+        else:
+            out.append(dict(type="mamba2", mixer=dict(mamba), mlp=moe))
+    return dict(architecture="Nolatar", vocab=vocab, width=width, norm=dict(eps=1e-5), layers=out)
+
+
 DESIGN_SHAPES = {"sefevik": ("Sefevik", sefevik_shape), "sodedra": ("Sodedra", sodedra_shape), "meronex": ("Meronex", meronex_shape),
-                 "tarunex": ("Tarunex", tarunex_shape), "balelorn": ("Balelorn", balelorn_shape)}
+                 "tarunex": ("Tarunex", tarunex_shape), "balelorn": ("Balelorn", balelorn_shape), "nolatar": ("Nolatar", nolatar_shape)}
 #: further designs that a design is measured beside (Qwen3 always is): the closest ones the engine has
-DESIGN_BESIDE = {"meronex": ("sodedra",), "tarunex": ("sodedra", "sefevik"), "balelorn": ("sodedra", "tarunex")}
+DESIGN_BESIDE = {"meronex": ("sodedra",), "tarunex": ("sodedra", "sefevik"), "balelorn": ("sodedra", "tarunex"),
+                 "nolatar": ("meronex", "tarunex")}
 #: layers, where --layers does not say: a whole number of the design's turns of layer kinds
 DESIGN_LAYERS = {"meronex": 9}
 
@@ -273,7 +303,7 @@ def main() -> int:
     ap.add_argument("--serve", type=int, default=0, metavar="N",
                     help="instead of the decode steps: N requests arriving at once, prompts of 128..2048 and outputs of 64..512 "
                          "tokens (uniform), run until all have ended; the value is generated tokens per second of the whole run")
-    ap.add_argument("--design", default="", choices=["", "sefevik", "sodedra", "meronex", "tarunex", "balelorn"],
+    ap.add_argument("--design", default="", choices=["", "sefevik", "sodedra", "meronex", "tarunex", "balelorn", "nolatar"],
                     help="instead of the decode steps: prefill and decode throughput of that design at a few layer sizes "
                          "beside the Qwen3 shape of equal width, layers, heads and feed-forward size (--design-sizes)")
     ap.add_argument("--design-sizes", default="1024,2048,4096", help="widths for --design")
