@@ -45,6 +45,7 @@ struct DecayMemory {
     int num_slots;
     float* state;
     long long state_stride;
+    int pieces8;                             // every row and head in 16-byte pieces of the operands: eight values at a time
 };
 
 __device__ __forceinline__ float dm_silu(float x) { return x / (1.0f + expf(-x)); }
@@ -58,6 +59,57 @@ __device__ __forceinline__ float dm_rotated(const TA* row, int i, const float2* 
     const float o = to_f32<TA>(row[i < half ? i + half : j]);
     const float2 c = rot[j];
     return i < half ? x * c.x - o * c.y : x * c.x + o * c.y;
+}
+
+// eight neighbouring values from a 16-byte aligned place
+template <typename TA>
+__device__ __forceinline__ void dm_load8(const TA* p, float (&v)[8]) {
+    if constexpr (sizeof(TA) == 2) {
+        typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4_t;
+        const u32x4_t r = *reinterpret_cast<const u32x4_t*>(p);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { v[2 * i] = __uint_as_float(r[i] << 16); v[2 * i + 1] = __uint_as_float(r[i] & 0xffff0000u); }
+    } else {
+        float lo[4], hi[4];
+        Vec4<float>::load(reinterpret_cast<const float*>(p), lo);
+        Vec4<float>::load(reinterpret_cast<const float*>(p) + 4, hi);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { v[i] = lo[i]; v[4 + i] = hi[i]; }
+    }
+}
+
+// values i .. i + 7 of a q or k row (d values), rotated by the token's angles; `pieces8`: i, d and half are multiples of 8
+template <typename TA>
+__device__ __forceinline__ void dm_rotated8(const DecayMemory& m, const TA* row, int i, const float2* rot, float (&v)[8]) {
+    if (!m.pieces8) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = i + e < m.d ? dm_rotated<TA>(row, i + e, rot, m.half) : 0.f;
+        return;
+    }
+    if (i >= m.d) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = 0.f;
+        return;
+    }
+    dm_load8<TA>(row + i, v);
+    if (!rot || i >= 2 * m.half) return;
+    const bool low = i < m.half;
+    const int j = low ? i : i - m.half;
+    float o[8];
+    dm_load8<TA>(row + (low ? i + m.half : j), o);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const float2 c = rot[j + e];
+        v[e] = low ? v[e] * c.x - o[e] * c.y : v[e] * c.x + o[e] * c.y;
+    }
+}
+
+// values j .. j + 7 of a head's dv values
+template <typename TA>
+__device__ __forceinline__ void dm_values8(const DecayMemory& m, const TA* row, int j, float (&v)[8]) {
+    if (m.pieces8 && j < m.dv) { dm_load8<TA>(row + j, v); return; }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = j + e < m.dv ? to_f32<TA>(row[j + e]) : 0.f;
 }
 
 // log of the decay and the write's factor of token t, head h
@@ -176,21 +228,21 @@ __global__ __launch_bounds__(DS_THREADS) void decay_memory_step_kernel(void* __r
 #define DP_THREADS 256
 #define DP_LD (64 + 16)       // floats from one staged row of 64 values to the next: four rows beside each other lie in different banks
 
-// cum[t] of the piece's tokens (inclusive) and b, by the block's first wave; la beyond the piece's end is 0
-__device__ __forceinline__ void dp_scan(const DecayMemory& m, int t0, int n, int h, float* cum, float* bs) {
+// cum[t] of the piece's tokens (inclusive) and b, by the block's first wave; la beyond the piece's end is 0.  The sums are
+// double: what is used of them is differences, and one token that forgets nearly everything must not cost the others their
+// decays' last digits.
+__device__ __forceinline__ void dp_scan(const DecayMemory& m, int t0, int n, int h, double* cum, float* bs) {
     if (threadIdx.x < 64) {
         const int lane = threadIdx.x;
         float la = 0.f, b = 0.f;
         if (lane < n) dm_scalars(m, t0 + lane, h, &la, &b);
-        if (m.log_decay) la = (float)(min(lane, n - 1) + 1) * m.log_decay[h];         // (a constant: no rounding adds up)
-        else {
+        double sum = (double)la;
 #pragma unroll
-            for (int o = 1; o < 64; o <<= 1) {
-                const float up = __shfl_up(la, o, 64);
-                if (lane >= o) la += up;
-            }
+        for (int o = 1; o < 64; o <<= 1) {
+            const double up = __shfl_up(sum, o, 64);
+            if (lane >= o) sum += up;
         }
-        cum[lane] = la;
+        cum[lane] = sum;
         bs[lane] = b;
     }
 }
@@ -201,7 +253,9 @@ template <typename TA>
 __global__ __launch_bounds__(DP_THREADS) void decay_memory_pieces_kernel(float* __restrict__ work, float* __restrict__ decay, const TA* __restrict__ k,
                                                                          const TA* __restrict__ v, DecayMemory m, const int* __restrict__ piece_t0,
                                                                          const int* __restrict__ piece_t1) {
-    __shared__ float ks[DP_TOKENS * DP_LD], vs[DP_TOKENS * DP_LD], cum[DP_TOKENS], bs[DP_TOKENS];
+    __shared__ __align__(16) float ks[DP_TOKENS * DP_LD], vs[DP_TOKENS * DP_LD];
+    __shared__ double cum[DP_TOKENS];
+    __shared__ float bs[DP_TOKENS];
     const int piece = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
     const int nd = (m.d + 63) / 64;
     const int i0 = (blockIdx.z % nd) * 64, j0 = (blockIdx.z / nd) * 64;
@@ -209,20 +263,27 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_pieces_kernel(float* 
     const int hq = h / m.per;
     dp_scan(m, t0, n, h, cum, bs);
     __syncthreads();
-    const float end = cum[n - 1];
+    const double end = cum[n - 1];
     const int rows = (n + 3) & ~3;
-    for (int e = tid; e < rows * 64; e += DP_THREADS) {
-        const int s = e >> 6, c = e & 63;
-        float kv = 0.f, vv = 0.f;
+    for (int e = tid; e < rows * 16; e += DP_THREADS) {              // eight values of k's or of v's part of a row
+        const int s = e >> 4, c = 8 * (e & 7);
+        float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        float f = 0.f;
         if (s < n) {
-            if (i0 + c < m.d)
-                kv = dm_rotated<TA>(k + (size_t)(t0 + s) * m.ks + (size_t)hq * m.d, i0 + c, m.rot ? m.rot + (size_t)(t0 + s) * m.half : nullptr, m.half) * m.kscale;
-            if (j0 + c < m.dv) vv = to_f32<TA>(v[(size_t)(t0 + s) * m.vs + (size_t)h * m.dv + j0 + c]) * (bs[s] * expf(end - cum[s]));
+            if (e & 8) {
+                dm_values8<TA>(m, v + (size_t)(t0 + s) * m.vs + (size_t)h * m.dv, j0 + c, x);
+                f = bs[s] * expf((float)(end - cum[s]));
+            } else {
+                dm_rotated8<TA>(m, k + (size_t)(t0 + s) * m.ks + (size_t)hq * m.d, i0 + c, m.rot ? m.rot + (size_t)(t0 + s) * m.half : nullptr, x);
+                f = m.kscale;
+            }
         }
-        ks[s * DP_LD + c] = kv;
-        vs[s * DP_LD + c] = vv;
+        float* dst = ((e & 8) ? vs : ks) + s * DP_LD + c;
+        const float lo[4] = {x[0] * f, x[1] * f, x[2] * f, x[3] * f}, hi[4] = {x[4] * f, x[5] * f, x[6] * f, x[7] * f};
+        Vec4<float>::store(dst, lo);
+        Vec4<float>::store(dst + 4, hi);
     }
-    if (tid == 0 && blockIdx.z == 0) decay[(size_t)piece * m.H + h] = expf(end);
+    if (tid == 0 && blockIdx.z == 0) decay[(size_t)piece * m.H + h] = expf((float)end);
     __syncthreads();
     const int wave = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
     if (i0 + 16 * wave >= m.d) return;
@@ -247,16 +308,18 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_pieces_kernel(float* 
 }
 
 // Along an entry's pieces, element by element of the state: every piece's contribution is replaced by the state that the
-// piece starts from, and the entry's last state goes to the request's slot.  Block x is a piece; the first of an entry walks.
+// piece starts from, and the entry's last state goes to the request's slot.  Block z is a piece; the first of an entry walks.
+// (Pieces are the grid's slowest dimension: blocks go to the dies in turn, and with every n-th block at work only some of
+// the dies would have any.)
 #define DF_AHEAD 8
 template <int V>
 __global__ __launch_bounds__(256) void decay_memory_fold_kernel(float* __restrict__ work, const float* __restrict__ decay, DecayMemory m,
                                                                 const int* __restrict__ piece_entry, const int* __restrict__ piece_first, int n_pieces) {
-    const int first = blockIdx.x, h = blockIdx.y;
+    const int first = blockIdx.z, h = blockIdx.y;
     if (piece_first[first] != first) return;
     const int slot = m.slot_ids[piece_entry[first]];
     if (slot < 0 || slot >= m.num_slots) return;
-    const size_t size = (size_t)m.d * m.dv, i = ((size_t)blockIdx.z * 256 + threadIdx.x) * V;
+    const size_t size = (size_t)m.d * m.dv, i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V;
     if (i >= size) return;
     int last = first;
     while (last + 1 < n_pieces && piece_first[last + 1] == first) ++last;
@@ -296,7 +359,9 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
                                                                           DecayMemory m, const int* __restrict__ piece_entry,
                                                                           const int* __restrict__ piece_t0, const int* __restrict__ piece_t1) {
     constexpr int KLD = 64 + 4, SLD = 16 * NJ + 16, VLD = 16 * NJ + 4;
-    __shared__ float ks[DP_TOKENS * KLD], sv[64 * SLD], cum[DP_TOKENS], bs[DP_TOKENS];
+    __shared__ __align__(16) float ks[DP_TOKENS * KLD], sv[64 * SLD];
+    __shared__ double cum[DP_TOKENS];
+    __shared__ float bs[DP_TOKENS];
     const int piece = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, j0 = blockIdx.z * 16 * NJ;
     const int t0 = piece_t0[piece], n = min(piece_t1[piece] - t0, DP_TOKENS);
     const int hq = h / m.per;
@@ -315,23 +380,41 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
     for (int st = 0; st < 4; ++st) sc[st] = dm_f32x4_t{0.f, 0.f, 0.f, 0.f};
     const TA* qrow = q + (size_t)(t0 + (tok ? tl : 0)) * m.qs + (size_t)hq * m.d;
     const float2* qrot = m.rot ? m.rot + (size_t)(t0 + (tok ? tl : 0)) * m.half : nullptr;
+    // Inside a slab, step st of the products takes dim 16 g + st from lane (r, g), so that a lane's 16 values of its query lie
+    // side by side in memory; in LDS, dim i of the slab has the place 4 (i % 16) + i / 16 (k: column, S_in: row).
     for (int i0 = 0; i0 < m.d; i0 += 64) {
-        const int steps = (min(64, m.d - i0) + 3) / 4;
+        const int steps = min(16, m.d - i0);                         // dims 16 g + st of this slab exist up to here for g = 0
         __syncthreads();                                             // the slab before has been read
-        for (int e = tid; e < rows * 64; e += DP_THREADS) {
-            const int s = e >> 6, c = e & 63;
-            ks[s * KLD + c] = (s < n && i0 + c < m.d)
-                ? dm_rotated<TA>(k + (size_t)(t0 + s) * m.ks + (size_t)hq * m.d, i0 + c, m.rot ? m.rot + (size_t)(t0 + s) * m.half : nullptr, m.half) * m.kscale : 0.f;
+        for (int e = tid; e < rows * 8; e += DP_THREADS) {
+            const int s = e >> 3, c = e & 7;
+            float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            if (s < n) dm_rotated8<TA>(m, k + (size_t)(t0 + s) * m.ks + (size_t)hq * m.d, i0 + 8 * c, m.rot ? m.rot + (size_t)(t0 + s) * m.half : nullptr, x);
+            float* dst = ks + s * KLD + 32 * (c & 1) + (c >> 1);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) dst[4 * i] = x[i] * m.kscale;
         }
-        for (int e = tid; e < 4 * steps * 16 * NJ; e += DP_THREADS) {
-            const int i = e / (16 * NJ), c = e - i * (16 * NJ);
-            sv[i * SLD + c] = (i0 + i < m.d && j0 + c < m.dv) ? S[(size_t)(i0 + i) * m.dv + j0 + c] : 0.f;
+        for (int e = tid; e < 64 * 4 * NJ; e += DP_THREADS) {
+            const int i = e / (4 * NJ), c = 4 * (e - i * (4 * NJ));
+            float x[4] = {0.f, 0.f, 0.f, 0.f};
+            if (i0 + i < m.d) {
+                const float* src = S + (size_t)(i0 + i) * m.dv + j0 + c;
+                if (m.pieces8) { if (j0 + c < m.dv) Vec4<float>::load(src, x); }
+                else {
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) x[u] = j0 + c + u < m.dv ? src[u] : 0.f;
+                }
+            }
+            Vec4<float>::store(sv + (4 * (i & 15) + (i >> 4)) * SLD + c, x);
         }
         float qf[16];
+        {
+            float lo[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, hi[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            if (tok) {
+                dm_rotated8<TA>(m, qrow, i0 + 16 * g, qrot, lo);
+                dm_rotated8<TA>(m, qrow, i0 + 16 * g + 8, qrot, hi);
+            }
 #pragma unroll
-        for (int st = 0; st < 16; ++st) {
-            const int i = i0 + 4 * st + g;
-            qf[st] = (tok && i < m.d) ? dm_rotated<TA>(qrow, i, qrot, m.half) : 0.f;
+            for (int i = 0; i < 8; ++i) { qf[i] = lo[i]; qf[8 + i] = hi[i]; }
         }
         __syncthreads();
         if (mine) {
@@ -348,13 +431,18 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
         }
     }
     __syncthreads();
-    for (int e = tid; e < rows * 16 * NJ; e += DP_THREADS) {
-        const int s = e / (16 * NJ), c = e - s * (16 * NJ);
-        sv[s * VLD + c] = (s < n && j0 + c < m.dv) ? to_f32<TA>(v[(size_t)(t0 + s) * m.vs + (size_t)h * m.dv + j0 + c]) : 0.f;
+    for (int e = tid; e < rows * 2 * NJ; e += DP_THREADS) {
+        const int s = e / (2 * NJ), c = 8 * (e - s * (2 * NJ));
+        float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        if (s < n) dm_values8<TA>(m, v + (size_t)(t0 + s) * m.vs + (size_t)h * m.dv, j0 + c, x);
+        const float lo[4] = {x[0], x[1], x[2], x[3]}, hi[4] = {x[4], x[5], x[6], x[7]};
+        Vec4<float>::store(sv + s * VLD + c, lo);
+        Vec4<float>::store(sv + s * VLD + c + 4, hi);
     }
     __syncthreads();
     if (!mine) return;                                               // (no barrier behind this)
-    const float ct = cum[tok ? tl : n - 1], et = expf(ct);
+    const double ct = cum[tok ? tl : n - 1];
+    const float et = expf((float)ct);
 #pragma unroll
     for (int jt = 0; jt < NJ; ++jt) acc[jt] *= et;
 #pragma unroll
@@ -363,7 +451,7 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int s = 16 * tile + 4 * g + i;
-                const float p = (s <= tl && s < n) ? sc[tile][i] * (bs[s] * expf(ct - cum[s])) : 0.f;
+                const float p = (s <= tl && s < n) ? sc[tile][i] * (bs[s] * expf((float)(ct - cum[s]))) : 0.f;
 #pragma unroll
                 for (int jt = 0; jt < NJ; ++jt) acc[jt] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[s * VLD + 16 * jt + r], p, acc[jt], 0, 0, 0);
             }
@@ -387,17 +475,32 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
 #pragma unroll
     for (int jt = 0; jt < NJ; ++jt) {
         const int jb = j0 + 16 * jt + 4 * g;
+        const size_t at = ((size_t)t * m.H + h) * m.dv + jb;
+        float y[4], gv[4] = {0.f, 0.f, 0.f, 0.f};
+        if (gr) {
+            if (m.pieces8) { if (jb < m.dv) Vec4<TA>::load(gr + jb, gv); }
+            else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) gv[i] = jb + i < m.dv ? to_f32<TA>(gr[jb + i]) : 0.f;
+            }
+        }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const int j = jb + i;
-            if (j >= m.dv) continue;
-            float o = acc[jt][i];
-            const size_t at = ((size_t)t * m.H + h) * m.dv + j;
-            if (m.epi == DM_NORM_GATE) {
-                reinterpret_cast<TA*>(out)[at] = from_f32<TA>((o * scale) * dm_silu(to_f32<TA>(gr[j])));
-            } else {
-                if (m.epi == DM_SKIP_GATE) o = fmaf(D, sv[tl * VLD + j - j0], o) * dm_silu(to_f32<TA>(gr[j]));
-                reinterpret_cast<float*>(out)[at] = o;
+            y[i] = acc[jt][i];
+            if (m.epi == DM_NORM_GATE) y[i] = (y[i] * scale) * dm_silu(gv[i]);
+            if (m.epi == DM_SKIP_GATE) y[i] = fmaf(D, sv[tl * VLD + jb + i - j0], y[i]) * dm_silu(gv[i]);
+        }
+        if (m.pieces8) {
+            if (jb < m.dv) {
+                if (m.epi == DM_NORM_GATE) Vec4<TA>::store(reinterpret_cast<TA*>(out) + at, y);
+                else Vec4<float>::store(reinterpret_cast<float*>(out) + at, y);
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (jb + i >= m.dv) continue;
+                if (m.epi == DM_NORM_GATE) reinterpret_cast<TA*>(out)[at + i] = from_f32<TA>(y[i]);
+                else reinterpret_cast<float*>(out)[at + i] = y[i];
             }
         }
     }
@@ -451,8 +554,10 @@ extern "C" int spy_decay_memory(void* out, const void* q, long long qs, const vo
     SPY_REQUIRE(half >= 0 && 2 * half <= d && (!rot || half > 0), "spy_decay_memory: %d rotated pairs of a head of %d", half, d);
     SPY_REQUIRE(epi >= 0 && epi <= 2 && (epi == DM_PLAIN || (gate && gs >= (long long)H * dv)) && (epi != DM_SKIP_GATE || skip) &&
                 (epi != DM_NORM_GATE || dv <= DS_SLICE), "spy_decay_memory: epilogue %d with heads of %d", epi, dv);
+    const uintptr_t bits = (uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)gate | (uintptr_t)work | (uintptr_t)out;
+    const bool pieces8 = d % 8 == 0 && dv % 8 == 0 && half % 8 == 0 && ((qs | ks | vs | gs) & 7) == 0 && bits % 16 == 0;
     const DecayMemory m = {H, per, d, dv, qs, ks, vs, gs, kscale, log_decay, dt, dts, dt_bias, rate, (const float2*)rot, half, skip, eps, epi,
-                           slot_ids, num_slots, state, state_stride};
+                           slot_ids, num_slots, state, state_stride, pieces8 ? 1 : 0};
     const bool v4 = dv % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)state % 16) == 0 && ((uintptr_t)work % 16) == 0;
     if (single) {
         SPY_REQUIRE(S == T, "spy_decay_memory: %d tokens of %d entries", T, S);
@@ -483,7 +588,8 @@ extern "C" int spy_decay_memory(void* out, const void* q, long long qs, const vo
     SPY_DISPATCH(dtype, TA, (decay_memory_pieces_kernel<TA><<<pgrid, DP_THREADS, 0, st>>>(work, decay, (const TA*)k, (const TA*)v, m, p0, p1)));
     SPY_CHECK_LAUNCH("spy_decay_memory (pieces)");
     const size_t size = (size_t)d * dv;
-    const dim3 fgrid(n_pieces, H, (unsigned)((size / (v4 ? 4 : 1) + 255) / 256));
+    const dim3 fgrid((unsigned)((size / (v4 ? 4 : 1) + 255) / 256), H, n_pieces);
+    SPY_REQUIRE(n_pieces <= 65535, "spy_decay_memory: %d pieces are too many", n_pieces);
     if (v4) decay_memory_fold_kernel<4><<<fgrid, 256, 0, st>>>(work, decay, m, pe, pf, n_pieces);
     else decay_memory_fold_kernel<1><<<fgrid, 256, 0, st>>>(work, decay, m, pe, pf, n_pieces);
     SPY_CHECK_LAUNCH("spy_decay_memory (fold)");

@@ -86,6 +86,37 @@ __device__ __forceinline__ void rs_widen(const rs_u32x4& r, float (&v)[8]) {
 __device__ __forceinline__ rs_u32x4 rs_narrow(const float (&v)[8]) {
     return rs_u32x4{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7])};
 }
+// 16 tokens' values of one kv head, staged as rows of `ld`, into the pages: 8 tokens of a dim that lie side by side in a page
+// leave in one store.  (P is a multiple of 8; the block has 256 threads.)
+__device__ __forceinline__ void rs_values_to_pages(const bf16_t* tile, int ld, int d, int t0, int T, const int* __restrict__ slots,
+                                                   bf16_t* __restrict__ vc, int P, int num_pages, int n_kv, int hv) {
+    for (int i = threadIdx.x; i < 2 * d; i += 256) {
+        const int tg = i / d, j = i - tg * d;                 // dim j of tokens t0 + 8 tg .. + 7
+        const int tb = t0 + 8 * tg;
+        if (tb >= T) continue;
+        const int s0 = slots[tb];
+        bool run = tb + 8 <= T && s0 >= 0 && s0 % 8 == 0 && s0 + 8 <= num_pages * P;
+        if (run) {
+#pragma unroll
+            for (int e = 1; e < 8; ++e) run = run && slots[tb + e] == s0 + e;
+        }
+        const bf16_t* col = tile + 8 * tg * ld + j;
+        if (run) {                                            // P is a multiple of 8: the 8 slots lie in one page
+            rs_u32x4 w;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) w[e] = (uint32_t)col[2 * e * ld] | ((uint32_t)col[(2 * e + 1) * ld] << 16);
+            const int page = s0 / P, off = s0 - page * P;
+            *reinterpret_cast<rs_u32x4*>(vc + (((size_t)page * n_kv + hv) * d + j) * P + off) = w;
+        } else {
+            for (int e = 0; e < 8 && tb + e < T; ++e) {
+                const int slot = slots[tb + e];
+                if (slot < 0 || slot >= num_pages * P) continue;
+                const int page = slot / P, off = slot - page * P;
+                vc[(((size_t)page * n_kv + hv) * d + j) * P + off] = col[e * ld];
+            }
+        }
+    }
+}
 template <typename TW>
 __global__ __launch_bounds__(256) void bias_rope_store_many_kernel(
     const bf16_t* __restrict__ x, long long xs, bf16_t* __restrict__ q_out, int T, int n_q, int n_kv, int d, const TW* __restrict__ bias,
@@ -170,32 +201,7 @@ __global__ __launch_bounds__(256) void bias_rope_store_many_kernel(
         *reinterpret_cast<rs_u32x4*>(tile + tt * ld + j0) = rs_narrow(v);
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < 2 * d; i += 256) {
-        const int tg = i / d, j = i - tg * d;                 // dim j of tokens t0 + 8 tg .. + 7
-        const int tb = t0 + 8 * tg;
-        if (tb >= T) continue;
-        const int s0 = slots[tb];
-        bool run = tb + 8 <= T && s0 >= 0 && s0 % 8 == 0 && s0 + 8 <= num_pages * P;
-        if (run) {
-#pragma unroll
-            for (int e = 1; e < 8; ++e) run = run && slots[tb + e] == s0 + e;
-        }
-        const bf16_t* col = tile + 8 * tg * ld + j;
-        if (run) {                                            // P is a multiple of 8: the 8 slots lie in one page
-            rs_u32x4 w;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) w[e] = (uint32_t)col[2 * e * ld] | ((uint32_t)col[(2 * e + 1) * ld] << 16);
-            const int page = s0 / P, off = s0 - page * P;
-            *reinterpret_cast<rs_u32x4*>(vc + (((size_t)page * n_kv + hv) * d + j) * P + off) = w;
-        } else {
-            for (int e = 0; e < 8 && tb + e < T; ++e) {
-                const int slot = slots[tb + e];
-                if (slot < 0 || slot >= num_pages * P) continue;
-                const int page = slot / P, off = slot - page * P;
-                vc[(((size_t)page * n_kv + hv) * d + j) * P + off] = col[e * ld];
-            }
-        }
-    }
+    rs_values_to_pages(tile, ld, d, t0, T, slots, vc, P, num_pages, n_kv, hv);
 }
 
 extern "C" int spy_bias_rope_store(const void* x, long long xs, int dtype, void* q_out, int T, int n_q, int n_kv, int d,
@@ -294,6 +300,95 @@ __global__ __launch_bounds__(RS_WAVES * 64) void norm_rope_store_kernel(
     }
 }
 
+// The same for many bfloat16 tokens, in 16-byte pieces (dim, dv, d, the rotated dims and all columns multiples of 8; pairs
+// (j, j + rot / 2): of 16).  The first T blocks have a token's query and key units each, L lanes a unit (L a power of two, one
+// piece a lane), the token's cosines and sines once in LDS for all of them; the others have 16 tokens of one value head.
+template <typename TW>
+__global__ __launch_bounds__(256) void norm_rope_store_many_kernel(
+    const bf16_t* __restrict__ x, long long xs, bf16_t* __restrict__ q_out, NormRope a, const TW* __restrict__ qw, const TW* __restrict__ kw,
+    const float* __restrict__ freq, const int* __restrict__ positions, bf16_t* __restrict__ kc, bf16_t* __restrict__ vc,
+    const int* __restrict__ slots, int T, int L) {
+    __shared__ __align__(16) bf16_t tile[16 * (RS_MAX_D + 8)];
+    __shared__ float cs[RS_MAX_D / 2], sn[RS_MAX_D / 2];
+    const rs_u32x4 none = {0u, 0u, 0u, 0u};
+    const int d8 = a.d >> 3;
+    if ((int)blockIdx.x < T) {
+        const int t = blockIdx.x, half = a.rot >> 1, c8 = a.dim >> 3;
+        const float p = (float)positions[t];
+        for (int j = threadIdx.x; j < half; j += 256) {
+            const float ang = p * freq[j];
+            cs[j] = cosf(ang);
+            sn[j] = sinf(ang);
+        }
+        __syncthreads();
+        const int slot = slots ? slots[t] : -1;
+        const bool stored = slot >= 0 && slot < a.num_pages * a.P;
+        const int page = stored ? slot / a.P : 0, off = stored ? slot - page * a.P : 0;
+        const int nq = a.n_q * a.maps, units = nq + (stored ? a.n_kv * a.maps : 0);
+        const int c = threadIdx.x & (L - 1), per = 256 / L;
+        // (every lane of a unit goes round the loop together: the sums' exchanges stay inside the unit's L lanes)
+        for (int u0 = threadIdx.x / L; u0 < units; u0 += per) {
+            const bool is_q = u0 < nq;
+            const int u = is_q ? u0 : u0 - nq, map = u % a.maps;
+            const bf16_t* src = x + (size_t)t * xs + (is_q ? a.q_off : a.k_off) + (size_t)u * a.hs;
+            const TW* w = is_q ? qw : kw;
+            bf16_t* dst = is_q ? q_out + ((size_t)t * nq + u) * a.d : kc + (((size_t)page * a.n_kv + u / a.maps) * a.P + off) * a.d;
+            float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            if (c < c8) rs_widen(*reinterpret_cast<const rs_u32x4*>(src + 8 * c), v);
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(v[e], v[e], ss);
+            for (int o = L >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+            const float r = 1.0f / sqrtf(ss / (float)a.dim + a.eps);
+            if (c < c8) {
+                const int j0 = 8 * c;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[e] = (v[e] * r) * to_f32<TW>(w[j0 + e]);
+                if (j0 < a.rot) {
+                    float y[8];
+                    if (a.inter) {
+#pragma unroll
+                        for (int e = 0; e < 8; e += 2) {
+                            const float c_ = cs[(j0 + e) >> 1], s_ = sn[(j0 + e) >> 1];
+                            y[e] = v[e] * c_ - v[e + 1] * s_;
+                            y[e + 1] = v[e + 1] * c_ + v[e] * s_;
+                        }
+                    } else {
+                        const bool low = j0 < half;
+                        const int jo = low ? j0 + half : j0 - half, jj = low ? j0 : jo;
+                        float o[8];
+                        rs_widen(*reinterpret_cast<const rs_u32x4*>(src + jo), o);
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) {
+                            const float z = (o[e] * r) * to_f32<TW>(w[jo + e]), c_ = cs[jj + e], s_ = sn[jj + e];
+                            y[e] = low ? v[e] * c_ - z * s_ : v[e] * c_ + z * s_;
+                        }
+                    }
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) v[e] = y[e];
+                }
+                *reinterpret_cast<rs_u32x4*>(dst + map * a.dim + j0) = rs_narrow(v);
+            }
+            if (is_q) {                                           // zeros: a query's other maps and its padding; a key's padding
+                for (int i = c; i < d8 - c8; i += L) *reinterpret_cast<rs_u32x4*>(dst + 8 * (i < map * c8 ? i : i + c8)) = none;
+            } else if (map == a.maps - 1) {
+                for (int i = a.maps * c8 + c; i < d8; i += L) *reinterpret_cast<rs_u32x4*>(dst + 8 * i) = none;
+            }
+        }
+        return;
+    }
+    const int vb = blockIdx.x - T;
+    const int t0 = (vb / a.n_kv) * 16, hv = vb % a.n_kv, ld = a.d + 8;
+    for (int i = threadIdx.x; i < 16 * d8; i += 256) {
+        const int tt = i / d8, j0 = 8 * (i - tt * d8);
+        if (t0 + tt >= T) continue;
+        *reinterpret_cast<rs_u32x4*>(tile + tt * ld + j0) =
+            j0 < a.dv ? *reinterpret_cast<const rs_u32x4*>(x + (size_t)(t0 + tt) * xs + a.v_off + (size_t)hv * a.hv + j0) : none;
+    }
+    __syncthreads();
+    rs_values_to_pages(tile, ld, a.d, t0, T, slots, vc, a.P, a.num_pages, a.n_kv, hv);
+}
+
 extern "C" int spy_norm_rope_store(const void* x, long long xs, int dtype, void* q_out, int T, int n_q, int n_kv, int maps, int dim, int dv,
                                    int d, long long q_off, long long k_off, long long v_off, int hs, int hv, const void* qw, const void* kw,
                                    int w_dtype, float eps, const float* freq, int rot, int inter, const int* positions, void* kc, void* vc,
@@ -308,6 +403,19 @@ extern "C" int spy_norm_rope_store(const void* x, long long xs, int dtype, void*
     const int units = (n_q + (slots ? n_kv : 0)) * maps + (slots ? n_kv : 0);
     SPY_REQUIRE(units <= 65535 * RS_WAVES, "spy_norm_rope_store: too many heads");
     const NormRope a = {n_q, n_kv, maps, dim, dv, d, q_off, k_off, v_off, hs, hv, rot, inter, P, num_pages, eps};
+    const uintptr_t bits = (uintptr_t)x | (uintptr_t)q_out | (uintptr_t)kc | (uintptr_t)vc;
+    const long long columns = q_off | (slots ? k_off | v_off | hv : 0) | hs | xs;
+    if (dtype == SPY_BF16 && T >= 64 && dim % 8 == 0 && dim <= 512 && d <= RS_MAX_D && d % 8 == 0 && dv % 8 == 0 && rot % (inter ? 8 : 16) == 0 && columns % 8 == 0 &&
+        (!slots || P % 8 == 0) && bits % 16 == 0) {
+        const long long blocks = (long long)T + (slots ? (long long)((T + 15) / 16) * n_kv : 0);
+        SPY_REQUIRE(blocks < (1ll << 31), "spy_norm_rope_store: too many tokens");
+        int L = 1;
+        while (L < dim / 8) L <<= 1;
+        SPY_DISPATCH(w_dtype, TW, (norm_rope_store_many_kernel<TW><<<(unsigned)blocks, 256, 0, st>>>(
+            (const bf16_t*)x, xs, (bf16_t*)q_out, a, (const TW*)qw, (const TW*)kw, freq, positions, (bf16_t*)kc, (bf16_t*)vc, slots, T, L)));
+        SPY_CHECK_LAUNCH("spy_norm_rope_store");
+        return 0;
+    }
     const dim3 grid(T, (units + RS_WAVES - 1) / RS_WAVES);
     SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (norm_rope_store_kernel<TA, TW><<<grid, RS_WAVES * 64, 0, st>>>(
         (const TA*)x, xs, (TA*)q_out, a, (const TW*)qw, (const TW*)kw, freq, positions, (TA*)kc, (TA*)vc, slots))));

@@ -181,7 +181,7 @@ def _whole_then_cut(parts, layers, manager, dtype, dev, x, other, refs, tol, wha
 
 # heads, kv heads, map size, value size, rotated dims, tokens
 DIFF_CASES = [(4, 2, 32, 64, 16, 150), (3, 1, 12, 10, 8, 70), (2, 2, 64, 128, 64, 300), (6, 3, 48, 96, 48, 330), (4, 1, 32, 48, 30, 1100), (16, 2, 16, 32, 16, 200),
-              (2, 1, 96, 64, 96, 140), (1, 1, 128, 256, 128, 90), (2, 2, 5, 40, 4, 60)]
+              (2, 1, 96, 64, 96, 140), (1, 1, 128, 256, 128, 90), (2, 2, 5, 40, 4, 60), (12, 1, 32, 40, 8, 100)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -386,6 +386,34 @@ def test_state_space(dtype, H, dv, N, G, conv, ng):
     g = torch.Generator().manual_seed(N)
     xs = [rnd(g, n, W).to(DT[dtype]) for n in LENGTHS]
     _recurrence_in_cuts(part, dtype, dev, xs, [plain.state_space(x.double(), w, cfg, eps) for x in xs])
+
+
+def test_a_token_that_forgets_everything_leaves_the_others_their_decays():
+    """Steps of every size beside each other: decays of e^-3000 and of 1 - 1e-3 in one piece."""
+    from spyinfer_amd.kernels import ops
+    dev = require_gpu()
+    g = torch.Generator().manual_seed(4)
+    T, H, d, dv = 150, 2, 16, 8
+    q, k, v = (rnd(g, T, H * n).float() for n in (d, d, dv))
+    raw = torch.full((T, H), -7.0)
+    raw[torch.rand((T, H), generator=g) < 0.1] = 300.0
+    bias, rate = torch.zeros(H), torch.tensor([1.0, 10.0])
+    dt = torch.nn.functional.softplus(raw.double())
+
+    def walk(q, k, v):
+        S, ref = torch.zeros((H, d, dv), dtype=torch.float64), torch.zeros((T, H, dv), dtype=torch.float64)
+        for t in range(T):
+            S = torch.exp(-rate.double() * dt[t])[:, None, None] * S + (dt[t][:, None] * k[t].double().view(H, d))[:, :, None] * v[t].double().view(H, 1, dv)
+            ref[t] = torch.einsum("hij,hi->hj", S, q[t].double().view(H, d))
+        return ref, S
+    ref, S = walk(q, k, v)
+    size, _ = walk(q.abs(), k.abs(), v.abs())          # what a sum's rounding is in proportion to
+    state = torch.zeros((1, H * d * dv), device=dev)
+    pieces = i32([0, 0, 0, 0, 64, 128, 64, 128, 150, 0, 0, 0], dev)
+    out = ops.decay_memory(*(t.to(dev) for t in (q, k, v)), H, H, d, dv, state, i32([0, T], dev), i32([0], dev), (pieces, 3, True), steps=(raw.to(dev), bias.to(dev), rate.to(dev)))
+    err = (out.double().cpu().view(T, H, dv) - ref).abs() / size
+    assert float(err.max()) < 2e-6, "decays are off by %.2g" % float(err.max())
+    assert float((state.double().cpu().view(H, d, dv) - S).abs().max()) < 2e-6 * float(S.abs().max())
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
