@@ -15,6 +15,7 @@
 //   combine: out[t] = scale * sum_k weight[t, k] * Y[row of pair (t, k)].
 #include "common.h"
 #include <math.h>
+#include <type_traits>
 
 #define MOE_TM 16
 #define MOE_MAX_EXPERTS 1024
@@ -435,9 +436,10 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(TC* __restrict__ C, 
 // (the four waves read the same rows; loaded by each of them they swept the first-level cache), while every wave's W
 // fragments still come straight from memory, asked for before the block waits for the staged rows.
 #define MOE_ROWS 128                 // 8 row tiles
+#define MOE_DIES 8
 #define MOE_LDS_STRIDE (128 + 8)     // values per staged row (16-byte pieces; the pad spreads the rows over the banks)
 template <bool GATED, typename TC>
-__global__ __launch_bounds__(256) void moe_gemm_mfma_lds_kernel(TC* __restrict__ C, const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
+__global__ __launch_bounds__(256, 2) void moe_gemm_mfma_lds_kernel(TC* __restrict__ C, const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
                                                                 const int* __restrict__ tile_expert, const int* __restrict__ sorted_pair,
                                                                 int gather, int max_tiles, int N, int K, long long w_stride, MoeAct act) {
     constexpr int MT = 8, NT = 2;
@@ -445,9 +447,21 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_lds_kernel(TC* __restrict__
     __shared__ int src_row[MOE_ROWS];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
     const int r = lane & 15, g = lane >> 4;
-    const int n0 = (blockIdx.y * 4 + wave) * (GATED ? 16 : 32);
+    // Blocks go to the chip's 8 dies in turn, by their number in the grid, and each die has an L2 of its own: the numbers are
+    // dealt out again, so that a die gets a run of blocks in (row tiles, columns) order.  Those at work on it at one time are
+    // then all columns of a few row tiles, of one or two experts, and a step's rows and matrix parts come from memory once
+    // for all of them.
+    int bx, by;
+    {
+        const int gx = gridDim.x, gy = gridDim.y, n = gx * gy, lin = blockIdx.x + gx * blockIdx.y;
+        const int die = lin % MOE_DIES, idx = lin / MOE_DIES, per = (n + MOE_DIES - 1) / MOE_DIES, rem = n % MOE_DIES;
+        const int v = (rem == 0 || die < rem) ? die * per + idx : rem * per + (die - rem) * (per - 1) + idx;
+        bx = v / gy;
+        by = v - bx * gy;
+    }
+    const int n0 = (by * 4 + wave) * (GATED ? 16 : 32);
     const bool cols = n0 < N;                        // (a wave without columns still helps to stage)
-    int t = blockIdx.x * MT;
+    int t = bx * MT;
     const int t_end = min(t + MT, max_tiles);
     const moe_bf16x8_t zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
     const int srow = threadIdx.x >> 4, spiece = threadIdx.x & 15;      // staging: rows srow + 16 i, 16-byte piece spiece
@@ -486,7 +500,9 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_lds_kernel(TC* __restrict__
 #pragma unroll
             for (int mt = 0; mt < MT; ++mt) acc[nt][mt] = moe_f32x4_t{0.f, 0.f, 0.f, 0.f};
         // the operands of a step are asked for one step ahead: W fragments into registers, the rows of A into registers
-        // on their way to LDS, both in flight while the matrix cores work on the step before
+        // on their way to LDS, both in flight while the matrix cores work on the step before.  The run's tiles are walked as
+        // eight, four or two: a tile that the run does not have is multiplied as it lies (its rows go nowhere), because a
+        // condition around every product would make the wave wait for every operand on its own.
         moe_bf16x8_t a[NT][4], stage[MT];
 #define MOE_ASK(KK)                                                                                                            \
         {                                                                                                                      \
@@ -494,34 +510,39 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_lds_kernel(TC* __restrict__
                 _Pragma("unroll") for (int nt = 0; nt < NT; ++nt)                                                              \
                     a[nt][j] = (cols && (KK) + 32 * j + 8 * g < K) ? *reinterpret_cast<const moe_bf16x8_t*>(wrow[nt] + (KK) + 32 * j) : zero8; \
             const bool kin_ = (KK) + 8 * spiece < K;                                                                           \
-            _Pragma("unroll") for (int i = 0; i < MT; ++i)                                                                     \
-                stage[i] = (i < run && srcs[i] >= 0 && kin_) ? *reinterpret_cast<const moe_bf16x8_t*>(A + (size_t)srcs[i] * K + (KK) + 8 * spiece) : zero8; \
+            _Pragma("unroll") for (int i = 0; i < TILES; ++i)                                                                  \
+                stage[i] = (srcs[i] >= 0 && kin_) ? *reinterpret_cast<const moe_bf16x8_t*>(A + (size_t)srcs[i] * K + (KK) + 8 * spiece) : zero8; \
         }
-        MOE_ASK(0)
-        for (int k = 0; k < K; k += 128) {
-            moe_bf16x8_t ac[NT][4];
-#pragma unroll
-            for (int j = 0; j < 4; ++j)
-#pragma unroll
-                for (int nt = 0; nt < NT; ++nt) ac[nt][j] = a[nt][j];
-            __syncthreads();                         // the step before has read its rows
-#pragma unroll
-            for (int i = 0; i < MT; ++i)
-                if (i < run) *reinterpret_cast<moe_bf16x8_t*>(xs + (srow + 16 * i) * MOE_LDS_STRIDE + 8 * spiece) = stage[i];
-            __syncthreads();
-            if (k + 128 < K) MOE_ASK(k + 128)
-            if (cols) {
+        auto walk = [&](auto tiles) {
+            constexpr int TILES = decltype(tiles)::value;
+            MOE_ASK(0)
+            for (int k = 0; k < K; k += 128) {
+                moe_bf16x8_t ac[NT][4];
 #pragma unroll
                 for (int j = 0; j < 4; ++j)
 #pragma unroll
-                    for (int mt = 0; mt < MT; ++mt)
-                        if (mt < run) {
+                    for (int nt = 0; nt < NT; ++nt) ac[nt][j] = a[nt][j];
+                __syncthreads();                     // the step before has read its rows
+#pragma unroll
+                for (int i = 0; i < TILES; ++i)
+                    *reinterpret_cast<moe_bf16x8_t*>(xs + (srow + 16 * i) * MOE_LDS_STRIDE + 8 * spiece) = stage[i];
+                __syncthreads();
+                if (k + 128 < K) MOE_ASK(k + 128)
+                if (cols) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+#pragma unroll
+                        for (int mt = 0; mt < TILES; ++mt) {
                             const moe_bf16x8_t b = *reinterpret_cast<const moe_bf16x8_t*>(xs + (mt * 16 + r) * MOE_LDS_STRIDE + 32 * j + 8 * g);
 #pragma unroll
                             for (int nt = 0; nt < NT; ++nt) acc[nt][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ac[nt][j], b, acc[nt][mt], 0, 0, 0);
                         }
+                }
             }
-        }
+        };
+        if (run > 4) walk(std::integral_constant<int, 8>{});
+        else if (run > 2) walk(std::integral_constant<int, 4>{});
+        else walk(std::integral_constant<int, 2>{});
 #undef MOE_ASK
         if (cols) {
 #pragma unroll
