@@ -508,19 +508,49 @@ __global__ __launch_bounds__(DP_THREADS) void decay_memory_results_kernel(void* 
 
 // out[t, :] = o / rms(o) over each of `groups` equal runs of N values, times w (null: none), times silu(gate[t, :]) (null:
 // none; rows `gs` values apart); one block per (token, run)
-template <typename TA, typename TW>
+// PASSES > 0: the run (its values in 16-byte pieces, at most 4 PASSES a thread) is read once and kept in registers.
+template <typename TA, typename TW, int PASSES>
 __global__ void group_norm_kernel(TA* __restrict__ out, const float* __restrict__ o, const TW* __restrict__ w, const TA* __restrict__ gate,
                                   long long gs, float eps, int groups, int N) {
     __shared__ float red[16];
     const int t = blockIdx.x, g = blockIdx.y, n = N / groups;
     const float* row = o + (size_t)t * N + (size_t)g * n;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < n; i += blockDim.x) ss = fmaf(row[i], row[i], ss);
-    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    const TW* wr = w ? w + (size_t)g * n : nullptr;
     TA* dst = out + (size_t)t * N + (size_t)g * n;
     const TA* gr = gate ? gate + (size_t)t * gs + (size_t)g * n : nullptr;
+    float ss = 0.f;
+    if constexpr (PASSES > 0) {
+        float v[PASSES][4], wv[PASSES][4], gv[PASSES][4];
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { v[p][e] = 0.f; wv[p][e] = 1.f; }
+            if (i < n) {
+                Vec4<float>::load(row + i, v[p]);
+                if (wr) Vec4<TW>::load(wr + i, wv[p]);
+                if (gr) Vec4<TA>::load(gr + i, gv[p]);
+            }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss = fmaf(v[p][e], v[p][e], ss);
+        }
+        const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < n) {
+                float y[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[e] = (v[p][e] * r) * wv[p][e] * (gr ? dm_silu(gv[p][e]) : 1.0f);
+                Vec4<TA>::store(dst + i, y);
+            }
+        }
+        return;
+    }
+    for (int i = threadIdx.x; i < n; i += blockDim.x) ss = fmaf(row[i], row[i], ss);
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-        float y = (row[i] * r) * (w ? to_f32<TW>(w[(size_t)g * n + i]) : 1.0f);
+        float y = (row[i] * r) * (wr ? to_f32<TW>(wr[i]) : 1.0f);
         if (gr) y *= dm_silu(to_f32<TA>(gr[i]));
         dst[i] = from_f32<TA>(y);
     }
@@ -530,9 +560,18 @@ extern "C" int spy_group_norm(void* out, int dtype, const float* o, const void* 
                               int groups, int N, hipStream_t st) {
     SPY_REQUIRE(T > 0 && groups > 0 && N > 0 && N % groups == 0 && groups <= 65535, "spy_group_norm: %d groups of %d values", groups, N);
     SPY_REQUIRE(!gate || gs >= N, "spy_group_norm: the gate's rows are too short");
-    const int n = N / groups, threads = n >= 2048 ? 256 : (n >= 512 ? 128 : 64);
-    SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, (group_norm_kernel<TA, TW><<<dim3(T, groups), threads, 0, st>>>(
-        (TA*)out, o, (const TW*)w, (const TA*)gate, gs, eps, groups, N))));
+    const int n = N / groups, threads = n >= 1024 ? 256 : (n >= 512 ? 128 : 64);
+    const bool pieces = n % 4 == 0 && gs % 4 == 0 && (((uintptr_t)out | (uintptr_t)o | (uintptr_t)w | (uintptr_t)gate) % 16) == 0;
+    const int passes = pieces ? (n / 4 + threads - 1) / threads : 0;
+#define GN(P) group_norm_kernel<TA, TW, P><<<dim3(T, groups), threads, 0, st>>>((TA*)out, o, (const TW*)w, (const TA*)gate, gs, eps, groups, N)
+    SPY_DISPATCH(dtype, TA, SPY_DISPATCH(w_dtype, TW, {
+        if (passes == 0 || passes > 8) GN(0);
+        else if (passes == 1) GN(1);
+        else if (passes == 2) GN(2);
+        else if (passes <= 4) GN(4);
+        else GN(8);
+    }));
+#undef GN
     SPY_CHECK_LAUNCH("spy_group_norm");
     return 0;
 }

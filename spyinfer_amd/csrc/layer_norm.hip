@@ -174,8 +174,8 @@ extern "C" int spy_layer_norm_residual(float* out, void* copy, const float* base
     return 0;
 }
 
-// out[r] = the layer norm of x[rows ? rows[r] : r]; one block per row, read three times (the second and third from the cache).
-template <typename TW, typename TO>
+// out[r] = the layer norm of x[rows ? rows[r] : r]; one block per row.  PASSES as above.
+template <typename TW, typename TO, int PASSES>
 __global__ void layer_norm_kernel(TO* __restrict__ out, const float* __restrict__ x, const TW* __restrict__ w, const TW* __restrict__ b,
                                   float eps, const int* __restrict__ rows, int T, int H) {
     __shared__ float red[16], red2[16];
@@ -188,6 +188,40 @@ __global__ void layer_norm_kernel(TO* __restrict__ out, const float* __restrict_
     }
     const float* row = x + (size_t)t * H;
     float s = 0.f;
+    if constexpr (PASSES > 0) {
+        float v[PASSES][4], wv[PASSES][4], bv[PASSES][4];
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[p][e] = 0.f;
+            if (i < H) { Vec4<float>::load(row + i, v[p]); Vec4<TW>::load(w + i, wv[p]); Vec4<TW>::load(b + i, bv[p]); }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) s += v[p][e];
+        }
+        const float mean = block_sum(s, red) / (float)H;
+        s = 0.f;
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < H) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { v[p][e] -= mean; s = fmaf(v[p][e], v[p][e], s); }
+            }
+        }
+        const float q = 1.0f / sqrtf(block_sum(s, red2) / (float)H + eps);
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int i = (p * blockDim.x + threadIdx.x) * 4;
+            if (i < H) {
+                float y[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[e] = fmaf(v[p][e] * q, wv[p][e], bv[p][e]);
+                Vec4<TO>::store(o + i, y);
+            }
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < H; i += blockDim.x) s += row[i];
     const float mean = block_sum(s, red) / (float)H;
     s = 0.f;
@@ -199,9 +233,18 @@ __global__ void layer_norm_kernel(TO* __restrict__ out, const float* __restrict_
 extern "C" int spy_layer_norm(void* out, int out_dtype, const float* x, const void* w, const void* b, int w_dtype, float eps, const int* rows,
                               int n_out, int T, int H, hipStream_t st) {
     SPY_REQUIRE(n_out > 0 && T > 0 && H > 0 && (rows || n_out == T), "spy_layer_norm: %d rows of %d", n_out, T);
-    const int threads = H >= 2048 ? 512 : (H >= 512 ? 256 : 64);
-    SPY_DISPATCH(w_dtype, TW, SPY_DISPATCH(out_dtype, TO, (layer_norm_kernel<TW, TO><<<n_out, threads, 0, st>>>(
-        (TO*)out, x, (const TW*)w, (const TW*)b, eps, rows, T, H))));
+    const int threads = H >= 4096 ? 512 : (H >= 1024 ? 256 : (H >= 512 ? 128 : 64));
+    const bool pieces = H % 4 == 0 && (((uintptr_t)out | (uintptr_t)x | (uintptr_t)w | (uintptr_t)b) % 16) == 0;
+    const int passes = pieces ? (H / 4 + threads - 1) / threads : 0;
+#define LNK(P) layer_norm_kernel<TW, TO, P><<<n_out, threads, 0, st>>>((TO*)out, x, (const TW*)w, (const TW*)b, eps, rows, T, H)
+    SPY_DISPATCH(w_dtype, TW, SPY_DISPATCH(out_dtype, TO, {
+        if (passes == 0 || passes > 8) LNK(0);
+        else if (passes == 1) LNK(1);
+        else if (passes == 2) LNK(2);
+        else if (passes <= 4) LNK(4);
+        else LNK(8);
+    }));
+#undef LNK
     SPY_CHECK_LAUNCH("spy_layer_norm");
     return 0;
 }

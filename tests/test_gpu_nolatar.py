@@ -72,7 +72,7 @@ def test_layer_normed_results_into_the_stream(dtype, T, H):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,H", [(9, 50), (3, 4096), (5, 1100)])
+@pytest.mark.parametrize("T,H", [(9, 50), (3, 4096), (5, 1100), (4, 1026), (3, 20000), (2, 320), (2, 9000), (3, 14336)])
 def test_layer_norm_of_the_stream_at_picked_rows(dtype, T, H):
     from spyinfer_amd.kernels import ops
     dev = require_gpu()
@@ -448,7 +448,7 @@ def test_short_convolution_of_many_tokens(dtype, C, n, with_bias):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("N,groups", [(60, 4), (4096, 1), (4096, 8), (1100, 2), (33, 33)])
+@pytest.mark.parametrize("N,groups", [(60, 4), (4096, 1), (4096, 8), (1100, 2), (33, 33), (20000, 1), (8192, 1), (1024, 8), (1000, 8)])
 def test_norm_in_groups_with_a_gate(dtype, N, groups):
     from spyinfer_amd.kernels import ops
     dev = require_gpu()
